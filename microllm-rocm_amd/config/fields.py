@@ -83,6 +83,23 @@ def string(source: Mapping[str, Any], key: str, default: Any = _MISSING) -> Opti
     return value
 
 
+def mapping(source: Mapping[str, Any], key: str, optional: bool = False) -> Optional[Mapping[str, Any]]:
+    value = source.get(key)
+    if value is None:
+        if optional:
+            return None
+        raise ConfigError(f"config is missing {key}")
+    if not isinstance(value, dict):
+        raise ConfigError(f"config key {key} must be an object, got {value!r}")
+    return value
+
+
+def positive(value, what: str):
+    if value is None or value <= 0:
+        raise ConfigError(f"{what} must be positive, got {value!r}")
+    return value
+
+
 def string_list(source: Mapping[str, Any], key: str, default: Any = _MISSING) -> Optional[Sequence[str]]:
     value = _get(source, key, default)
     if value is default and default is not _MISSING:

@@ -67,7 +67,7 @@ bias_attention_kernel(const T* __restrict__ q, const T* __restrict__ k_pages, co
                       const float* __restrict__ sink, T* __restrict__ out, int64_t out_stride, int heads, int kv_heads,
                       int key_dim, int value_dim, int page_size, float scale, float out_scale,
                       const float* __restrict__ slopes, int window, int chunk, const float* __restrict__ gate,
-                      int64_t gate_stride) {
+                      int64_t gate_stride, float softcap, int gate_channels) {
     extern __shared__ float q_row[];
     const int token = blockIdx.x / heads;
     const int head = blockIdx.x % heads;
@@ -97,6 +97,7 @@ bias_attention_kernel(const T* __restrict__ q, const T* __restrict__ k_pages, co
             place = static_cast<int64_t>(table[j / page_size]) * page_size + j % page_size;
             const T* key = k_pages + place * key_row + static_cast<int64_t>(kv_head) * key_dim;
             score = dot_row<T>(key, q_row, key_dim) * scale;
+            if (softcap > 0.0f) score = softcap * tanhf(score / softcap);
             if (bias) score += bias[static_cast<int64_t>(min(position - j, longest)) * heads + head];
             if (slopes) score -= slope * static_cast<float>(position - j);
         }
@@ -121,12 +122,13 @@ bias_attention_kernel(const T* __restrict__ q, const T* __restrict__ k_pages, co
         }
     }
     float factor = out_scale / running_sum;
-    if (gate) factor *= 1.0f / (1.0f + expf(-gate[static_cast<int64_t>(token) * gate_stride + head]));
+    const float* gate_row = gate ? gate + static_cast<int64_t>(token) * gate_stride + (gate_channels ? head * value_dim : head) : nullptr;
+    if (gate_row && !gate_channels) factor *= 1.0f / (1.0f + expf(-gate_row[0]));
     T* to = out + static_cast<int64_t>(token) * out_stride + static_cast<int64_t>(head) * value_dim;
 #pragma unroll
     for (int m = 0; m < kMaxValueChannelsALane; ++m) {
         const int c = lane + m * kWave;
-        if (c < value_dim) to[c] = from_float<T>(acc[m] * factor);
+        if (c < value_dim) to[c] = from_float<T>(gate_row && gate_channels ? acc[m] * factor / (1.0f + expf(-gate_row[c])) : acc[m] * factor);
     }
 }
 
@@ -139,7 +141,7 @@ qk_norm_store_kernel(const float* __restrict__ qkv, int n_parts, int64_t part_st
                      const int32_t* __restrict__ slot_mapping, float temp_coef, int temp_every, T* __restrict__ q_out,
                      T* __restrict__ k_pages, T* __restrict__ v_pages, int heads, int kv_heads, int key_dim, int value_dim,
                      int tiled_page_size, const float* __restrict__ bias, int normed, int queries_only, int64_t row_stride,
-                     const float* __restrict__ cos_sin, int rot_dims) {
+                     const float* __restrict__ cos_sin, int rot_dims, int values_normed) {
     const int vectors = queries_only ? heads : heads + 2 * kv_heads;
     const int token = blockIdx.x / vectors;
     const int which = blockIdx.x % vectors;
@@ -159,7 +161,7 @@ qk_norm_store_kernel(const float* __restrict__ qkv, int n_parts, int64_t part_st
         squares += value * value;
     }
     const float* weight = is_q ? q_weight : (is_k ? k_weight : nullptr);
-    const bool norm = normed && (is_q || is_k);
+    const bool norm = (is_q || is_k) ? normed : values_normed;
     float factor = 1.0f;
     if (norm) factor = 1.0f / sqrtf(wave_sum(squares) / static_cast<float>(dim) + eps);
     if (is_q && temp_coef != 0.0f) {
@@ -213,7 +215,7 @@ int mll_qk_norm_store(const float* qkv, int n_parts, int64_t part_stride, const 
                       float eps, const int32_t* positions, const int32_t* slot_mapping, float temp_coef, int temp_every,
                       void* q_out, void* k_pages, void* v_pages, int dtype, int n_tokens, int heads, int kv_heads, int key_dim,
                       int value_dim, int tiled_page_size, const float* bias, int normed, int queries_only, int64_t row_stride,
-                      const float* cos_sin, int rot_dims, hipStream_t stream) {
+                      const float* cos_sin, int rot_dims, int values_normed, hipStream_t stream) {
     MLL_REQUIRE(tiled_page_size == 0 || (tiled_page_size > 0 && tiled_page_size % 16 == 0 && key_dim == value_dim),
                 "qk_norm_store: tiled pages hold a multiple of 16 positions and keys and values of one width");
     MLL_REQUIRE(n_tokens >= 0 && heads > 0 && kv_heads > 0 && key_dim > 0 && value_dim > 0, "qk_norm_store: sizes must be positive");
@@ -223,7 +225,7 @@ int mll_qk_norm_store(const float* qkv, int n_parts, int64_t part_stride, const 
     MLL_REQUIRE(cos_sin == nullptr || (rot_dims > 0 && rot_dims % 2 == 0 && rot_dims <= key_dim),
                 "qk_norm_store: an even number of turned channels, at most the head's");
     MLL_REQUIRE((q_weight == nullptr) == (k_weight == nullptr), "qk_norm_store: norm weights for queries and keys, or for neither");
-    MLL_REQUIRE(!normed || eps > 0.0f, "qk_norm_store: eps must be positive");
+    MLL_REQUIRE(!(normed || values_normed) || eps > 0.0f, "qk_norm_store: eps must be positive");
     MLL_REQUIRE(normed || q_weight == nullptr, "qk_norm_store: norm weights without a norm");
     MLL_REQUIRE(queries_only || (slot_mapping != nullptr && k_pages != nullptr && v_pages != nullptr), "qk_norm_store: keys and values need pages and slots");
     MLL_REQUIRE(temp_coef == 0.0f || temp_every > 0, "qk_norm_store: the factor by position needs a positive step");
@@ -234,12 +236,12 @@ int mll_qk_norm_store(const float* qkv, int n_parts, int64_t part_stride, const 
         qk_norm_store_kernel<float><<<static_cast<unsigned>(blocks), kWave, 0, stream>>>(
             qkv, n_parts, part_stride, q_weight, k_weight, eps, positions, slot_mapping, temp_coef, temp_every,
             static_cast<float*>(q_out), static_cast<float*>(k_pages), static_cast<float*>(v_pages), heads, kv_heads, key_dim, value_dim,
-            tiled_page_size, bias, normed, queries_only, row_stride, cos_sin, rot_dims);
+            tiled_page_size, bias, normed, queries_only, row_stride, cos_sin, rot_dims, values_normed);
     } else if (dtype == kBF16) {
         qk_norm_store_kernel<bf16><<<static_cast<unsigned>(blocks), kWave, 0, stream>>>(
             qkv, n_parts, part_stride, q_weight, k_weight, eps, positions, slot_mapping, temp_coef, temp_every,
             static_cast<bf16*>(q_out), static_cast<bf16*>(k_pages), static_cast<bf16*>(v_pages), heads, kv_heads, key_dim, value_dim,
-            tiled_page_size, bias, normed, queries_only, row_stride, cos_sin, rot_dims);
+            tiled_page_size, bias, normed, queries_only, row_stride, cos_sin, rot_dims, values_normed);
     } else {
         return fail("qk_norm_store: unknown dtype");
     }
@@ -250,7 +252,7 @@ int mll_bias_attention(const void* q, const void* k_pages, const void* v_pages, 
                        const int32_t* seq_of_token, const int32_t* positions, const float* bias, int longest,
                        const float* sink, void* out, int64_t out_stride, int dtype, int n_tokens, int heads, int kv_heads,
                        int key_dim, int value_dim, int page_size, float scale, float out_scale, const float* slopes, int window,
-                       int chunk, const float* gate, int64_t gate_stride, hipStream_t stream) {
+                       int chunk, const float* gate, int64_t gate_stride, float softcap, int gate_channels, hipStream_t stream) {
     MLL_REQUIRE(n_tokens >= 0 && heads > 0 && kv_heads > 0 && key_dim > 0 && value_dim > 0 && page_size > 0 && table_width > 0,
                 "bias_attention: sizes must be positive");
     MLL_REQUIRE(heads % kv_heads == 0, "bias_attention: heads must divide into kv heads");
@@ -258,7 +260,8 @@ int mll_bias_attention(const void* q, const void* k_pages, const void* v_pages, 
     MLL_REQUIRE(bias == nullptr || longest >= 0, "bias_attention: the bias table needs at least one row");
     MLL_REQUIRE(out_stride >= static_cast<int64_t>(heads) * value_dim, "bias_attention: the output rows overlap");
     MLL_REQUIRE(window >= 0 && chunk >= 0 && !(window > 0 && chunk > 0), "bias_attention: a window or chunks of positions, not both");
-    MLL_REQUIRE(gate == nullptr || gate_stride >= heads, "bias_attention: one gate a head in every row");
+    MLL_REQUIRE(gate == nullptr || gate_stride >= (gate_channels ? heads * value_dim : heads), "bias_attention: one gate a head, or a channel, in every row");
+    MLL_REQUIRE(softcap >= 0.0f, "bias_attention: the cap on the scores is positive, or 0 for none");
     if (n_tokens == 0) return 0;
     const int64_t blocks = static_cast<int64_t>(n_tokens) * heads;
     MLL_REQUIRE(blocks < (1ll << 31), "bias_attention: too many rows for one launch");
@@ -268,12 +271,12 @@ int mll_bias_attention(const void* q, const void* k_pages, const void* v_pages, 
         bias_attention_kernel<float><<<static_cast<unsigned>(blocks), kWave, lds, stream>>>(
             static_cast<const float*>(q), static_cast<const float*>(k_pages), static_cast<const float*>(v_pages), block_table,
             table_width, seq_of_token, positions, bias, longest, sink, static_cast<float*>(out), out_stride, heads, kv_heads,
-            key_dim, value_dim, page_size, scale, out_scale, slopes, window, chunk, gate, gate_stride);
+            key_dim, value_dim, page_size, scale, out_scale, slopes, window, chunk, gate, gate_stride, softcap, gate_channels);
     } else if (dtype == kBF16) {
         bias_attention_kernel<bf16><<<static_cast<unsigned>(blocks), kWave, lds, stream>>>(
             static_cast<const bf16*>(q), static_cast<const bf16*>(k_pages), static_cast<const bf16*>(v_pages), block_table,
             table_width, seq_of_token, positions, bias, longest, sink, static_cast<bf16*>(out), out_stride, heads, kv_heads,
-            key_dim, value_dim, page_size, scale, out_scale, slopes, window, chunk, gate, gate_stride);
+            key_dim, value_dim, page_size, scale, out_scale, slopes, window, chunk, gate, gate_stride, softcap, gate_channels);
     } else {
         return fail("bias_attention: unknown dtype");
     }

@@ -40,16 +40,18 @@ union Frag8 {
     uint4 raw;
 };
 
-// The factor of a head's gate on its result: sigmoid(gate[token][head]), or 1 without a gate.
-__device__ inline float head_gate(const MllAttentionExtras& extras, int token, int head) {
+// The factor of the gate on channel `dim` of a head's result: sigmoid of the head's number or of the channel's own
+// (gate_channels); 1 without a gate.
+__device__ inline float result_gate(const MllAttentionExtras& extras, int token, int head, int head_dim, int dim) {
     if (extras.gate == nullptr) return 1.0f;
-    return 1.0f / (1.0f + __expf(-extras.gate[static_cast<int64_t>(token) * extras.gate_stride + head]));
+    const int column = extras.gate_channels ? head * head_dim + dim : head;
+    return 1.0f / (1.0f + __expf(-extras.gate[static_cast<int64_t>(token) * extras.gate_stride + column]));
 }
 
 // EXTRA: the scores also get extras.bias[min(position - key, longest)][head], the softmax's denominator also holds
 // exp(extras.sink[head]) (counted once, where the waves' or the splits' results meet), the result is multiplied by
-// extras.out_scale and by the head's gate and its rows lie extras.out_stride elements apart; with extras.chunk the keys
-// seen begin at the query's chunk of positions. Without EXTRA the kernel is what it was.
+// extras.out_scale and by its gate and its rows lie extras.out_stride elements apart; with extras.chunk the keys
+// seen begin at the query's chunk of positions; with extras.softcap the scaled scores pass a tanh. Without EXTRA the kernel is what it was.
 template <int HD_TILES, bool STREAM, bool EXTRA>
 __global__ __launch_bounds__(kDecodeThreads) void paged_attention_decode_kernel(
     const bf16* __restrict__ q, const bf16* __restrict__ k_cache, const bf16* __restrict__ v_cache,
@@ -168,6 +170,7 @@ __global__ __launch_bounds__(kDecodeThreads) void paged_attention_decode_kernel(
             for (int i = 0; i < 4; ++i) {
                 const int key = key0 + 8 * quad + 4 * t + i;
                 float value = s[i] * scale;
+                if (EXTRA && extras.softcap > 0.0f) value = softcap_fast(value, extras.softcap, 1.0f / extras.softcap);
                 if (EXTRA && bias_column != nullptr) {
                     const int distance = position - key;
                     value += (distance >= extras.longest || distance < 0) ? far_bias : bias_column[static_cast<int64_t>(distance) * heads];
@@ -305,7 +308,7 @@ __global__ __launch_bounds__(kDecodeThreads) void paged_attention_decode_kernel(
         const int64_t row = static_cast<int64_t>(token) * heads + head0 + h;
         const int64_t part_row = static_cast<int64_t>(blockIdx.x) * heads + head0 + h;   // partial results are kept densely
         if (n_splits == 1) {
-            if (EXTRA) out[static_cast<int64_t>(token) * extras.out_stride + (head0 + h) * HD + dim] = from_float<bf16>(total / sum * extras.out_scale * head_gate(extras, token, head0 + h));
+            if (EXTRA) out[static_cast<int64_t>(token) * extras.out_stride + (head0 + h) * HD + dim] = from_float<bf16>(total / sum * extras.out_scale * result_gate(extras, token, head0 + h, HD, dim));
             else out[row * HD + dim] = from_float<bf16>(total / sum);
         } else {
             part_o[(part_row * n_splits + split) * HD + dim] = total;
@@ -359,7 +362,7 @@ __global__ void paged_attention_join_kernel(const float* __restrict__ part_o, co
             }
         }
         if (with_sink) weight_sum += __expf(sink - top);
-        if (EXTRA) out[static_cast<int64_t>(token) * extras.out_stride + (blockIdx.x % heads) * head_dim + dim] = from_float<bf16>(total / weight_sum * extras.out_scale * head_gate(extras, token, blockIdx.x % heads));
+        if (EXTRA) out[static_cast<int64_t>(token) * extras.out_stride + (blockIdx.x % heads) * head_dim + dim] = from_float<bf16>(total / weight_sum * extras.out_scale * result_gate(extras, token, blockIdx.x % heads, head_dim, dim));
         else out[row * head_dim + dim] = from_float<bf16>(total / weight_sum);
     }
 }

@@ -180,6 +180,9 @@ __global__ __launch_bounds__(kPrefillThreads, 1) void paged_attention_prefill_ke
     float running_sum = 0.0f;         // over this lane's keys only; the two halves of the wave meet at the end
     float running_offset = 0.0f;      // -(running maximum) in units of log 2; 0 while the maximum is -inf
     const bool biased = EXTRA && extras.bias != nullptr;
+    const bool capped = EXTRA && extras.softcap > 0.0f;
+    const float cap_units = capped ? extras.softcap / scale : 0.0f;
+    const float cap_rate = capped ? 2.0f * scale_log2 / extras.softcap : 0.0f;
     if (EXTRA) {
         const float to_units = 1.0f / scale;
         if (biased) {       // read after the first block has landed, which is behind a barrier
@@ -345,6 +348,14 @@ __global__ __launch_bounds__(kPrefillThreads, 1) void paged_attention_prefill_ke
             __builtin_amdgcn_sched_group_barrier(0x008, 1, 0);
             if (j + kAhead < PRODUCTS) __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
         }
+        // Capped scores, still in the product's units: (cap / scale) tanh(s scale / cap), the tanh as 1 - 2 / (1 + e^2x).
+        if (EXTRA && capped) {
+#pragma unroll
+            for (int r = 0; r < HALVES; ++r)
+#pragma unroll
+                for (int i = 0; i < 16; ++i)
+                    s[r][i] = fmaf(-2.0f * cap_units, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(s[r][i] * cap_rate)), cap_units);
+        }
         // s[r][i] is row 8 (i / 4) + 4 half + i % 4: key key0 + 32 r + 16 (i / 8) + 8 half + i % 8, token `column`.
         if (EXTRA && biased) {
             if (block_position - (key0 + 32 * HALVES - 1) >= extras.longest) {      // every key far behind every token
@@ -486,7 +497,9 @@ __global__ __launch_bounds__(kPrefillThreads, 1) void paged_attention_prefill_ke
     // o_acc[d][i]: dim 32 d + 8 (i / 4) + 4 half + i % 4 of token `column`.
     if (column < block_valid) {
         float inverse = (EXTRA ? extras.out_scale : 1.0f) / running_sum;
-        if (EXTRA && extras.gate != nullptr)        // the head's gate: sigmoid of one number a token and head
+        const bool channel_gates = EXTRA && extras.gate != nullptr && extras.gate_channels;
+        const float* gate_row = channel_gates ? extras.gate + static_cast<int64_t>(first_token + block_first + column) * extras.gate_stride + head * HD : nullptr;
+        if (EXTRA && extras.gate != nullptr && !channel_gates)        // the head's gate: sigmoid of one number a token and head
             inverse *= 1.0f / (1.0f + __expf(-extras.gate[static_cast<int64_t>(first_token + block_first + column) * extras.gate_stride + head]));
         bf16* out_row = EXTRA ? out + static_cast<int64_t>(first_token + block_first + column) * extras.out_stride + head * HD
                               : out + (static_cast<int64_t>(first_token + block_first + column) * heads + head) * HD;
@@ -498,7 +511,10 @@ __global__ __launch_bounds__(kPrefillThreads, 1) void paged_attention_prefill_ke
                 if (HD % 32 != 0 && dim >= HD) continue;
                 bf16x4 four;
 #pragma unroll
-                for (int i = 0; i < 4; ++i) four[i] = static_cast<__bf16>(o_acc[d][4 * j + i] * inverse);
+                for (int i = 0; i < 4; ++i) {
+                    const float factor = channel_gates ? inverse / (1.0f + __expf(-gate_row[dim + i])) : inverse;
+                    four[i] = static_cast<__bf16>(o_acc[d][4 * j + i] * factor);
+                }
                 *reinterpret_cast<bf16x4*>(out_row + dim) = four;
             }
     }
@@ -546,7 +562,7 @@ extern "C" int mll_paged_attention_prefill_extra(const void* q, const void* k_ca
                                                  int n_tiles, const int32_t* positions, void* out, float scale, int window,
                                                  int heads, int kv_heads, int head_dim, int page_size,
                                                  const MllAttentionExtras* extras, hipStream_t stream) {
-    MLL_REQUIRE(!extras || scale > 0.0f, "paged_attention_prefill: a bias or a sink needs a positive scale");
+    MLL_REQUIRE(!extras || scale > 0.0f, "paged_attention_prefill: a bias, a sink or a cap on the scores needs a positive scale");
     MLL_REQUIRE(!extras || !extras->bias || (extras->longest >= 0 && extras->longest < kPrefillBiasRows),
                 "paged_attention_prefill: the bias table has more rows than the kernel keeps");
     MLL_REQUIRE(!extras || extras->out_stride >= static_cast<int64_t>(heads) * head_dim, "paged_attention_prefill: the output rows overlap");

@@ -87,6 +87,20 @@ __device__ inline float activate(float z, int act) {
     return z / (1.0f + expf(-z));
 }
 
+// The gate of a gated product's epilogue, with the fast exponential: silu(z), or the tanh form of gelu, which is
+// z sigmoid(2 sqrt(2 / pi) (z + 0.044715 z^3)).
+template <bool GELU>
+__device__ inline float gate_fast(float z) {
+    const float t = GELU ? 1.59576912160573071176f * (z + 0.044715f * z * z * z) : z;
+    return z / (1.0f + __expf(-t));
+}
+
+// cap * tanh(value / cap) as cap - 2 cap / (1 + exp(2 value / cap)), with the fast exponential and reciprocal (absolute
+// error about 1e-7 of cap).
+__device__ inline float softcap_fast(float value, float cap, float inverse_cap) {
+    return fmaf(-2.0f * cap, __builtin_amdgcn_rcpf(1.0f + __expf(2.0f * value * inverse_cap)), cap);
+}
+
 __device__ inline float wave_sum(float value) {
 #pragma unroll
     for (int offset = kWave / 2; offset > 0; offset >>= 1) value += __shfl_xor(value, offset, kWave);

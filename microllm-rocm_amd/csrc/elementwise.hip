@@ -387,20 +387,27 @@ __device__ inline float stable_sigmoid(float value) {
     return e / (1.0f + e);
 }
 
-template <typename T>
-__global__ void silu_mul_kernel(const T* __restrict__ gate, const T* __restrict__ up, int64_t in_stride,
-                                T* __restrict__ out, int width) {
+// The gate of a gated feed-forward: SiLU with the stable sigmoid, or another activation by its number.
+template <int ACT>
+__device__ inline float gate_value(float z) {
+    return ACT == kActSilu ? z * stable_sigmoid(z) : activate(z, ACT);
+}
+
+template <typename T, int ACT>
+__global__ void gated_activation_kernel(const T* __restrict__ gate, const T* __restrict__ up, int64_t in_stride,
+                                        T* __restrict__ out, int width) {
     const int token = blockIdx.y;
     const int column = blockIdx.x * blockDim.x + threadIdx.x;
     if (column >= width) return;
     const float g = to_float(gate[token * in_stride + column]);
     const float u = to_float(up[token * in_stride + column]);
-    out[static_cast<int64_t>(token) * width + column] = from_float<T>(g * stable_sigmoid(g) * u);
+    out[static_cast<int64_t>(token) * width + column] = from_float<T>(gate_value<ACT>(g) * u);
 }
 
 // The same for bfloat16 rows whose width is a multiple of 8: 16 bytes of gate and of up per thread.
-__global__ void silu_mul_bf16x8_kernel(const bf16* __restrict__ gate, const bf16* __restrict__ up, int64_t in_stride,
-                                       bf16* __restrict__ out, int width) {
+template <int ACT>
+__global__ void gated_activation_bf16x8_kernel(const bf16* __restrict__ gate, const bf16* __restrict__ up, int64_t in_stride,
+                                               bf16* __restrict__ out, int width) {
     const int token = blockIdx.y;
     const int chunk = blockIdx.x * blockDim.x + threadIdx.x;
     if (chunk * 8 >= width) return;
@@ -409,12 +416,25 @@ __global__ void silu_mul_bf16x8_kernel(const bf16* __restrict__ gate, const bf16
     u.raw = *reinterpret_cast<const uint4*>(up + token * in_stride + chunk * 8);
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
-        const float gv = to_float(g.v[i]);
-        z.v[i] = from_float<bf16>(gv * stable_sigmoid(gv) * to_float(u.v[i]));
+        z.v[i] = from_float<bf16>(gate_value<ACT>(to_float(g.v[i])) * to_float(u.v[i]));
     }
     *reinterpret_cast<uint4*>(out + static_cast<int64_t>(token) * width + chunk * 8) = z.raw;
 }
 
+
+// out[t][c] = gelu_tanh(sum of z's parts [t][c]) * table[ids[t]][column_at + c]; an id outside [0, vocab) gives NaN.
+template <typename T, typename W>
+__global__ void __launch_bounds__(256)
+token_side_gate_kernel(const float* __restrict__ z, int n_parts, int64_t part_stride, const W* __restrict__ table, int64_t table_stride,
+                       int column_at, int vocab, const int32_t* __restrict__ ids, T* __restrict__ out, int64_t count, int dim) {
+    const int64_t i = static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x;
+    if (i >= count) return;
+    float sum = z[i];
+    for (int part = 1; part < n_parts; ++part) sum += z[part * part_stride + i];
+    const int id = ids[i / dim];
+    const float side = id >= 0 && id < vocab ? to_float(table[id * table_stride + column_at + i % dim]) : NAN;
+    out[i] = from_float<T>(activate(sum, kActGeluTanh) * side);
+}
 
 // out[i] = act(in[i]): in float32 (partial sums added in order first) or T; act 0 SiLU, 1 the exact gelu
 // 0.5 z (1 + erf(z / sqrt 2)), 2 the tanh form of gelu.
@@ -595,27 +615,49 @@ int mll_rope_table(const int32_t* positions, const double* inv_freq, int n_freq,
     return check_launch("rope_table");
 }
 
-int mll_silu_mul(const void* gate, const void* up, int64_t in_stride, void* out, int dtype,
-                 int n_tokens, int width, hipStream_t stream) {
-    MLL_REQUIRE(n_tokens >= 0 && width > 0 && in_stride >= width, "silu_mul: bad sizes");
+int mll_gated_activation(const void* gate, const void* up, int64_t in_stride, void* out, int dtype,
+                         int n_tokens, int width, int act, hipStream_t stream) {
+    MLL_REQUIRE(n_tokens >= 0 && width > 0 && in_stride >= width, "gated_activation: bad sizes");
+    MLL_REQUIRE(act == kActSilu || act == kActGeluTanh, "gated_activation: SiLU or the tanh form of gelu");
     if (n_tokens == 0) return 0;
-    MLL_REQUIRE(n_tokens <= 65535, "silu_mul: more than 65535 tokens in one call");
+    MLL_REQUIRE(n_tokens <= 65535, "gated_activation: more than 65535 tokens in one call");
     const dim3 grid((width + 255) / 256, n_tokens);
+    const bool gelu = act == kActGeluTanh;
     if (dtype == kF32) {
-        silu_mul_kernel<float><<<grid, 256, 0, stream>>>(static_cast<const float*>(gate), static_cast<const float*>(up),
-                                                         in_stride, static_cast<float*>(out), width);
+        auto* kernel = gelu ? gated_activation_kernel<float, kActGeluTanh> : gated_activation_kernel<float, kActSilu>;
+        kernel<<<grid, 256, 0, stream>>>(static_cast<const float*>(gate), static_cast<const float*>(up), in_stride, static_cast<float*>(out), width);
     } else if (dtype == kBF16 && width % 8 == 0 && in_stride % 8 == 0 && reinterpret_cast<uintptr_t>(gate) % 16 == 0 &&
                reinterpret_cast<uintptr_t>(up) % 16 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0) {
         const dim3 wide_grid((width / 8 + 255) / 256, n_tokens);
-        silu_mul_bf16x8_kernel<<<wide_grid, 256, 0, stream>>>(static_cast<const bf16*>(gate), static_cast<const bf16*>(up),
-                                                             in_stride, static_cast<bf16*>(out), width);
+        auto* kernel = gelu ? gated_activation_bf16x8_kernel<kActGeluTanh> : gated_activation_bf16x8_kernel<kActSilu>;
+        kernel<<<wide_grid, 256, 0, stream>>>(static_cast<const bf16*>(gate), static_cast<const bf16*>(up), in_stride, static_cast<bf16*>(out), width);
     } else if (dtype == kBF16) {
-        silu_mul_kernel<bf16><<<grid, 256, 0, stream>>>(static_cast<const bf16*>(gate), static_cast<const bf16*>(up),
-                                                        in_stride, static_cast<bf16*>(out), width);
+        auto* kernel = gelu ? gated_activation_kernel<bf16, kActGeluTanh> : gated_activation_kernel<bf16, kActSilu>;
+        kernel<<<grid, 256, 0, stream>>>(static_cast<const bf16*>(gate), static_cast<const bf16*>(up), in_stride, static_cast<bf16*>(out), width);
     } else {
-        return fail("silu_mul: unknown dtype");
+        return fail("gated_activation: unknown dtype");
     }
-    return check_launch("silu_mul");
+    return check_launch("gated_activation");
+}
+
+int mll_token_side_gate(const float* z, int n_parts, int64_t part_stride, const void* table, int table_dtype, int64_t table_stride,
+                        int column_at, int vocab, const int32_t* ids, void* out, int dtype, int n_tokens, int dim, hipStream_t stream) {
+    MLL_REQUIRE(n_tokens >= 0 && dim > 0 && vocab > 0 && n_parts >= 1, "token_side_gate: sizes must be positive");
+    MLL_REQUIRE(column_at >= 0 && column_at + dim <= table_stride, "token_side_gate: the columns lie outside the table's rows");
+    if (n_tokens == 0) return 0;
+    const int64_t count = static_cast<int64_t>(n_tokens) * dim;
+    MLL_REQUIRE(count < (1ll << 38), "token_side_gate: too many values for one launch");
+    const unsigned blocks = static_cast<unsigned>((count + 255) / 256);
+#define MLL_SIDE(T, W)                                                                                                     \
+    token_side_gate_kernel<T, W><<<blocks, 256, 0, stream>>>(z, n_parts, part_stride, static_cast<const W*>(table), table_stride, \
+                                                            column_at, vocab, ids, static_cast<T*>(out), count, dim)
+    if (dtype == kF32 && table_dtype == kF32) MLL_SIDE(float, float);
+    else if (dtype == kF32 && table_dtype == kBF16) MLL_SIDE(float, bf16);
+    else if (dtype == kBF16 && table_dtype == kF32) MLL_SIDE(bf16, float);
+    else if (dtype == kBF16 && table_dtype == kBF16) MLL_SIDE(bf16, bf16);
+    else return fail("token_side_gate: unknown dtype");
+#undef MLL_SIDE
+    return check_launch("token_side_gate");
 }
 
 }  // extern "C"

@@ -29,7 +29,6 @@ union Piece {
     uintx4 raw;
 };
 
-__device__ inline float silu_f(float value) { return value / (1.0f + __expf(-value)); }
 
 template <int NT>
 __device__ inline void load_batch(Piece (&pieces)[kBatch][NT], const bf16* const (&w_ptr)[NT], const bool (&w_live)[NT],
@@ -165,7 +164,7 @@ __global__ __launch_bounds__(kWaves * kWave) void gemm_medium_kernel(
 #pragma unroll
                 for (int i = 0; i < 4; i += 2) {
                     const int column = n_tile * 8 + quad * 2 + i / 2;
-                    if (column < n / 2) target[column] = from_float<bf16>(silu_f(acc[nt][mt][i]) * acc[nt][mt][i + 1]);
+                    if (column < n / 2) target[column] = from_float<bf16>(gate_fast<EPILOGUE == 5>(acc[nt][mt][i]) * acc[nt][mt][i + 1]);
                 }
             }
         }
@@ -222,13 +221,14 @@ extern "C" int mll_gemm_medium(const void* a, const void* w_packed, void* out, i
     MLL_REQUIRE(waves == 4 || waves == 8, "gemm_medium: workgroups of 4 or 8 waves");
     MLL_REQUIRE(splits >= 1 && splits <= 64, "gemm_medium: between 1 and 64 splits of k");
     MLL_REQUIRE(epilogue == 0 || splits == 1, "gemm_medium: only float32 partial sums can be split over k");
-    MLL_REQUIRE(epilogue != 2 || n % 2 == 0, "gemm_medium: the gated epilogue needs an even number of weight rows");
+    MLL_REQUIRE((epilogue != 2 && epilogue != 5) || n % 2 == 0, "gemm_medium: the gated epilogue needs an even number of weight rows");
     MLL_REQUIRE(reinterpret_cast<uintptr_t>(a) % 16 == 0, "gemm_medium: the activations must be 16-byte aligned");
     if (m == 0) return 0;
     switch (epilogue) {
         case 0: return medium::launch_medium<0>(a, w_packed, out, m, n, k, tiles_per_wave, waves, splits, stream);
         case 1: return medium::launch_medium<1>(a, w_packed, out, m, n, k, tiles_per_wave, waves, splits, stream);
         case 2: return medium::launch_medium<2>(a, w_packed, out, m, n, k, tiles_per_wave, waves, splits, stream);
+        case 5: return medium::launch_medium<5>(a, w_packed, out, m, n, k, tiles_per_wave, waves, splits, stream);
         default: return fail("gemm_medium: unknown epilogue");
     }
 }

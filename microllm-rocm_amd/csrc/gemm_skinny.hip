@@ -26,15 +26,12 @@ union Piece {
     uintx4 raw;
 };
 
-__device__ inline float silu_f(float value) {
-    return value / (1.0f + __expf(-value));
-}
-
 // EPILOGUE: 0 = float32 [M, N]; 1 = bfloat16 [M, N]; 2 = bfloat16 [M, N / 2] = silu(even rows of W) * (odd rows).
 // 3 = the q/k/v projection of an attention layer finished in place: bias, rotation of the position, queries to
 // `q_out`, keys and values into their pages (at most 16 rows; see MllQkvStore). 4 = the product is added to the
 // float32 residual stream and the sum, times the next norm's weight, is written as the next product's input,
 // with each workgroup's share of the rows' sums of squares (at most 16 rows; see MllResidualNorm).
+// 5 = 2 with the tanh form of gelu for silu.
 // Whatever the epilogue, a row of the product is first multiplied by the factor that MllRowScale describes,
 // if one is given (at most 16 rows).
 // W is read past the caches (non-temporal loads): a step reads every weight once, and all of them together are far
@@ -276,12 +273,12 @@ __global__ __launch_bounds__(1024) void gemm_skinny_kernel(
                     const int column = n_tile * 16 + quad * 4 + i;
                     if (column < n) target[column] = from_float<bf16>(acc[nt][mt][i]);
                 }
-            } else if (EPILOGUE == 2) {
+            } else if (EPILOGUE == 2 || EPILOGUE == 5) {
                 bf16* target = static_cast<bf16*>(out) + static_cast<int64_t>(row) * (n / 2);
 #pragma unroll
                 for (int i = 0; i < 4; i += 2) {
                     const int column = n_tile * 8 + quad * 2 + i / 2;
-                    if (column < n / 2) target[column] = from_float<bf16>(silu_f(acc[nt][mt][i]) * acc[nt][mt][i + 1]);
+                    if (column < n / 2) target[column] = from_float<bf16>(gate_fast<EPILOGUE == 5>(acc[nt][mt][i]) * acc[nt][mt][i + 1]);
                 }
             } else {
                 // The lane's 4 columns lie in one head (head_dim is a multiple of 16). In a query or key head the
@@ -381,7 +378,7 @@ static int launch_skinny(const void* a, const void* w_packed, void* out, int m, 
     const bf16* w_ = static_cast<const bf16*>(w_packed);
     const int m_tiles = (m + 15) / 16;
     const bool two = tiles_per_group(m, n_tiles) == 2;
-    if constexpr (EPILOGUE >= 3) {
+    if constexpr (EPILOGUE == 3 || EPILOGUE == 4) {
         if (m_tiles != 1) return fail("gemm_skinny: this epilogue takes at most 16 rows");
         if (two) launch_one<1, 2, EPILOGUE>(a_, w_, out, m, n, k, n_tiles, k_steps, extras, stream);
         else launch_one<1, 1, EPILOGUE>(a_, w_, out, m, n, k, n_tiles, k_steps, extras, stream);
@@ -421,7 +418,7 @@ extern "C" int mll_gemm_skinny(const void* a, const void* w_packed, void* out, i
                                const MllRowScale* scale, hipStream_t stream) {
     MLL_REQUIRE(m >= 0 && m <= 64, "gemm_skinny: takes at most 64 rows");
     MLL_REQUIRE(n > 0 && k > 0 && k % 8 == 0, "gemm_skinny: k must be a positive multiple of 8");
-    MLL_REQUIRE(epilogue != 2 || n % 2 == 0, "gemm_skinny: the gated epilogue needs an even number of weight rows");
+    MLL_REQUIRE((epilogue != 2 && epilogue != 5) || n % 2 == 0, "gemm_skinny: the gated epilogue needs an even number of weight rows");
     if (check_scale(scale, m) != 0) return 1;
     if (m == 0) return 0;
     MllSkinnyExtras extras{};
@@ -430,6 +427,7 @@ extern "C" int mll_gemm_skinny(const void* a, const void* w_packed, void* out, i
         case 0: return launch_skinny<0>(a, w_packed, out, m, n, k, extras, stream);
         case 1: return launch_skinny<1>(a, w_packed, out, m, n, k, extras, stream);
         case 2: return launch_skinny<2>(a, w_packed, out, m, n, k, extras, stream);
+        case 5: return launch_skinny<5>(a, w_packed, out, m, n, k, extras, stream);
         default: return fail("gemm_skinny: unknown epilogue");
     }
 }

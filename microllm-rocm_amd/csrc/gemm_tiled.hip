@@ -48,7 +48,6 @@ constexpr int kSuperM = 4, kSuperN = 8;                   // tiles of C that run
 
 __device__ __align__(16) const unsigned zero_piece[256] = {};      // a piece of W past the end of k
 
-__device__ inline float silu_fast(float value) { return value / (1.0f + __expf(-value)); }
 
 __device__ inline unsigned lds_address(bf16* place) { return static_cast<unsigned>(reinterpret_cast<uintptr_t>((lds_bf16*)place)); }
 
@@ -363,12 +362,12 @@ __global__ __launch_bounds__(kTiledThreads, 1) void gemm_tiled_kernel(const bf16
                 if (column + 3 < n && n % 4 == 0) {
                     bf16x2 two;
 #pragma unroll
-                    for (int i = 0; i < 2; ++i) two[i] = static_cast<__bf16>(silu_fast(acc[nt][mt][2 * i]) * acc[nt][mt][2 * i + 1]);
+                    for (int i = 0; i < 2; ++i) two[i] = static_cast<__bf16>(gate_fast<EPILOGUE == 5>(acc[nt][mt][2 * i]) * acc[nt][mt][2 * i + 1]);
                     *reinterpret_cast<bf16x2*>(target) = two;
                 } else {
 #pragma unroll
                     for (int i = 0; i < 4; i += 2)
-                        if (column + i < n) target[i / 2] = from_float<bf16>(silu_fast(acc[nt][mt][i]) * acc[nt][mt][i + 1]);
+                        if (column + i < n) target[i / 2] = from_float<bf16>(gate_fast<EPILOGUE == 5>(acc[nt][mt][i]) * acc[nt][mt][i + 1]);
                 }
             }
         }
@@ -427,13 +426,14 @@ extern "C" int mll_gemm_tiled(const void* a, const void* w_packed, void* out, in
     MLL_REQUIRE(k % 32 == 0, "gemm_tiled: k must be a multiple of 32");
     MLL_REQUIRE(splits >= 1 && splits <= 64 && (splits == 1 || epilogue == 0), "gemm_tiled: only the float32 epilogue takes k in parts");
     MLL_REQUIRE(static_cast<int64_t>(kTileN) * k < (int64_t{1} << 30), "gemm_tiled: k is too long");
-    MLL_REQUIRE(epilogue != 2 || n % 2 == 0, "gemm_tiled: the gated epilogue needs an even number of weight rows");
+    MLL_REQUIRE((epilogue != 2 && epilogue != 5) || n % 2 == 0, "gemm_tiled: the gated epilogue needs an even number of weight rows");
     MLL_REQUIRE(reinterpret_cast<uintptr_t>(a) % 16 == 0, "gemm_tiled: the activations must be 16-byte aligned");
     if (m == 0) return 0;
     switch (epilogue) {
         case 0: return launch_tiled<0>(a, w_packed, out, m, n, k, splits, tile_rows, stream);
         case 1: return launch_tiled<1>(a, w_packed, out, m, n, k, splits, tile_rows, stream);
         case 2: return launch_tiled<2>(a, w_packed, out, m, n, k, splits, tile_rows, stream);
+        case 5: return launch_tiled<5>(a, w_packed, out, m, n, k, splits, tile_rows, stream);
         default: return fail("gemm_tiled: unknown epilogue");
     }
 }

@@ -4,9 +4,10 @@
 //   S_t = diag(a_t) S_(t-1) + k_t v_t^T        (S: [key_dim, value_dim], a_t in (0, 1) per key channel)
 //   o_t = S_t^T q_t
 //
-// with a_t = sigmoid(z_t)^(1 / tau), z_t = A2 (low-rank input) + b. Three kernels: the decays of a step's tokens
+// (a design may pass queries, keys and values through SiLU first) with a_t = sigmoid(z_t)^(1 / tau), z_t = A2 (low-rank input) + b. Three kernels: the decays of a step's tokens
 // (all tokens at once), the walk over each request's tokens in order (the state's columns are independent, so a
-// request's head is spread over workgroups by value channel), and the norm and gate of the results. State, decays
+// request's head is spread over workgroups by value channel), and the norm (a head, or all heads together) and gate
+// of the results. State, decays
 // and everything the walk touches are float32, whatever the engine's element type.
 #include <type_traits>
 
@@ -40,8 +41,9 @@ __global__ void gla_decay_kernel(const float* __restrict__ proj, int64_t proj_st
 // One wave a (request, head, group of value channels). lane = column_in_group * lanes_a_column + r; lane r of a
 // column keeps the key channels ROWS r .. ROWS r + ROWS - 1. A token's result is the sum over a lane's channels in order, then
 // over the column's lanes in order (the lanes leave their sums in LDS and one adds them up): both kernels below add
-// in this order, so a request gives the same bits whichever of them walks its tokens.
-template <int ROWS>
+// in this order, so a request gives the same bits whichever of them walks its tokens. SILU: queries, keys and values
+// pass the activation as they are read (a step of few tokens; many tokens get a kernel of their own before the walk).
+template <int ROWS, bool SILU>
 __global__ void __launch_bounds__(kWave)
 gla_scan_kernel(const float* __restrict__ proj, int64_t proj_stride, int q_offset, int k_offset, int v_offset,
                 const float* __restrict__ decay, float* __restrict__ state, const int32_t* __restrict__ cu_tokens,
@@ -79,12 +81,13 @@ gla_scan_kernel(const float* __restrict__ proj, int64_t proj_stride, int q_offse
         }
         v_next = row[v_offset + head * value_dim + safe_column];
     };
+    auto read = [](float value) { return SILU ? activate(value, kActSilu) : value; };
     fetch(first);
     for (int token = first; token < last; ++token) {
         float a[ROWS], k[ROWS], q[ROWS];
 #pragma unroll
-        for (int m = 0; m < ROWS; ++m) a[m] = a_next[m], k[m] = k_next[m], q[m] = q_next[m];
-        const float v = v_next;
+        for (int m = 0; m < ROWS; ++m) a[m] = a_next[m], k[m] = read(k_next[m]), q[m] = read(q_next[m]);
+        const float v = read(v_next);
         if (token + 1 < last) fetch(token + 1);
         float partial = 0.0f;
 #pragma unroll
@@ -259,6 +262,31 @@ gla_scan_tiled_kernel(const float* __restrict__ proj, int64_t proj_stride, int q
     }
 }
 
+// columns first .. first + count - 1 of every row of proj, in place: silu.
+__global__ void __launch_bounds__(256)
+gla_silu_kernel(float* __restrict__ proj, int64_t proj_stride, int first, int count) {
+    const int column = blockIdx.x * blockDim.x + threadIdx.x;
+    if (column >= count) return;
+    float* place = proj + static_cast<int64_t>(blockIdx.y) * proj_stride + first + column;
+    *place = activate(*place, kActSilu);
+}
+
+// out[t, :] = rms_norm(o[t, :]) * weight * sigmoid(gate[t, :]) over all heads of a token together; one workgroup a token.
+template <typename T>
+__global__ void gla_gate_all_kernel(const float* __restrict__ o, const float* __restrict__ proj, int64_t proj_stride, int gate_offset,
+                                    const float* __restrict__ weight, float eps, T* __restrict__ out, int64_t out_stride, int width,
+                                    float out_scale) {
+    __shared__ float scratch[16];
+    const float* row = o + static_cast<int64_t>(blockIdx.x) * width;
+    const float* gate = proj + static_cast<int64_t>(blockIdx.x) * proj_stride + gate_offset;
+    float squares = 0.0f;
+    for (int c = threadIdx.x; c < width; c += blockDim.x) squares = fmaf(row[c], row[c], squares);
+    const float factor = 1.0f / sqrtf(block_sum(squares, scratch) / static_cast<float>(width) + eps);
+    T* to = out + static_cast<int64_t>(blockIdx.x) * out_stride;
+    for (int c = threadIdx.x; c < width; c += blockDim.x)
+        to[c] = from_float<T>((weight ? row[c] * factor * weight[c] : row[c] * factor) / (1.0f + expf(-gate[c])) * out_scale);
+}
+
 // out[t, head, :] = rms_norm(o[t, head, :]) * weight * silu(gate[t, head, :]) * out_scale (weight null: none); one wave a (token, head).
 template <typename T>
 __global__ void __launch_bounds__(kWave)
@@ -308,7 +336,7 @@ int mll_gla_decay(const float* proj, int64_t proj_stride, int low_offset, int ra
 
 int mll_gla_scan(const float* proj, int64_t proj_stride, int q_offset, int k_offset, int v_offset, const float* decay,
                  float* state, const int32_t* cu_tokens, const int32_t* slots, float* out, int n_seqs, int heads, int key_dim,
-                 int value_dim, float q_scale, int long_portions, int64_t decay_stride, hipStream_t stream) {
+                 int value_dim, float q_scale, int long_portions, int64_t decay_stride, int silu_inputs, hipStream_t stream) {
     MLL_REQUIRE(n_seqs >= 0 && heads > 0 && key_dim > 0 && value_dim > 0, "gla_scan: sizes must be positive");
     MLL_REQUIRE(key_dim <= kWideHeadRows * kWave, "gla_scan: key heads wider than 512 are not supported");
     MLL_REQUIRE(q_offset >= 0 && k_offset >= 0 && v_offset >= 0 && q_offset + heads * key_dim <= proj_stride &&
@@ -316,6 +344,7 @@ int mll_gla_scan(const float* proj, int64_t proj_stride, int q_offset, int k_off
                 "gla_scan: a projection lies outside its row");
     MLL_REQUIRE(decay_stride == 0 || decay_stride >= static_cast<int64_t>(heads) * key_dim,
                 "gla_scan: the decays of a token are heads * key_dim numbers; a stride of 0 gives every token the same");
+    MLL_REQUIRE(!(silu_inputs && long_portions), "gla_scan: the walk over long portions takes inputs that have passed their activation");
     if (n_seqs == 0) return 0;
     const int rows = key_dim <= kUsualRows * kWave ? kUsualRows : kWideHeadRows;
     int lanes_a_column = 1;
@@ -342,13 +371,14 @@ int mll_gla_scan(const float* proj, int64_t proj_stride, int q_offset, int k_off
 #undef MLL_SCAN_TILED
         return check_launch("gla_scan_tiled");
     }
-    if (rows == kUsualRows) {
-        gla_scan_kernel<kUsualRows><<<grid, kWave, 0, stream>>>(proj, proj_stride, q_offset, k_offset, v_offset, decay, state, cu_tokens,
-                                                               slots, out, heads, key_dim, value_dim, lanes_a_column, q_scale, decay_stride);
-    } else {
-        gla_scan_kernel<kWideHeadRows><<<grid, kWave, 0, stream>>>(proj, proj_stride, q_offset, k_offset, v_offset, decay, state, cu_tokens,
-                                                                  slots, out, heads, key_dim, value_dim, lanes_a_column, q_scale, decay_stride);
-    }
+#define MLL_SCAN(ROWS, SILU)                                                                                                  \
+    gla_scan_kernel<ROWS, SILU><<<grid, kWave, 0, stream>>>(proj, proj_stride, q_offset, k_offset, v_offset, decay, state, cu_tokens, \
+                                                            slots, out, heads, key_dim, value_dim, lanes_a_column, q_scale, decay_stride)
+    if (rows == kUsualRows && silu_inputs) MLL_SCAN(kUsualRows, true);
+    else if (rows == kUsualRows) MLL_SCAN(kUsualRows, false);
+    else if (silu_inputs) MLL_SCAN(kWideHeadRows, true);
+    else MLL_SCAN(kWideHeadRows, false);
+#undef MLL_SCAN
     return check_launch("gla_scan");
 }
 
@@ -371,6 +401,34 @@ int mll_gla_gate(const float* o, const float* proj, int64_t proj_stride, int gat
         return fail("gla_gate: unknown dtype");
     }
     return check_launch("gla_gate");
+}
+
+int mll_gla_silu(float* proj, int64_t proj_stride, int first, int count, int n_tokens, hipStream_t stream) {
+    MLL_REQUIRE(n_tokens >= 0 && first >= 0 && count > 0 && first + count <= proj_stride, "gla_silu: the columns lie outside their row");
+    for (int done = 0; done < n_tokens; done += 65535) {
+        const dim3 grid((count + 255) / 256, n_tokens - done < 65535 ? n_tokens - done : 65535);
+        gla_silu_kernel<<<grid, 256, 0, stream>>>(proj + done * proj_stride, proj_stride, first, count);
+    }
+    return check_launch("gla_silu");
+}
+
+int mll_gla_gate_all(const float* o, const float* proj, int64_t proj_stride, int gate_offset, const float* weight, float eps,
+                     void* out, int64_t out_stride, int dtype, int n_tokens, int width, float out_scale, hipStream_t stream) {
+    MLL_REQUIRE(n_tokens >= 0 && width > 0 && eps > 0.0f, "gla_gate_all: sizes and eps must be positive");
+    MLL_REQUIRE(gate_offset >= 0 && gate_offset + width <= proj_stride, "gla_gate_all: the gate lies outside its row");
+    MLL_REQUIRE(out_stride >= width, "gla_gate_all: the output rows overlap");
+    if (n_tokens == 0) return 0;
+    const int threads = width <= 128 ? 64 : (width <= 512 ? 256 : (width <= 2048 ? 512 : 1024));
+    if (dtype == kF32) {
+        gla_gate_all_kernel<float><<<n_tokens, threads, 0, stream>>>(o, proj, proj_stride, gate_offset, weight, eps, static_cast<float*>(out),
+                                                                     out_stride, width, out_scale);
+    } else if (dtype == kBF16) {
+        gla_gate_all_kernel<bf16><<<n_tokens, threads, 0, stream>>>(o, proj, proj_stride, gate_offset, weight, eps, static_cast<bf16*>(out),
+                                                                    out_stride, width, out_scale);
+    } else {
+        return fail("gla_gate_all: unknown dtype");
+    }
+    return check_launch("gla_gate_all");
 }
 
 }  // extern "C"

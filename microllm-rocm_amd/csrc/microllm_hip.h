@@ -35,9 +35,12 @@ int mll_rms_norm(float* h, const void* delta, int delta_dtype, int n_partials, i
 // h[r] = v; out[i] = v * rsqrt(mean(v^2) + eps) * weight (weight null: no output). A sublayer's result that is normed
 // itself before it joins the stream, fused with the norm that follows (csrc/norm_after.hip). extra (null: none): float32
 // rows like h's, added to v after the delta (what a model adds to its stream between two layers).
+// delta null (with after_weight): v = h[r]. weight null: out = v as it is; out null: the sum alone. groups > 1: a row is
+// cut into that many equal runs of neighbouring columns, and either norm's mean of squares is over the run.
 int mll_rms_norm_after(float* h, const void* delta, int delta_dtype, int n_partials, int64_t partial_stride,
                        const int32_t* rows, const float* after_weight, float after_eps, float mult, const float* extra,
-                       const float* weight, float eps, void* out, int dtype, int n_rows, int width, int write_h, hipStream_t stream);
+                       const float* weight, float eps, void* out, int dtype, int n_rows, int width, int write_h, int groups,
+                       hipStream_t stream);
 
 // values[r][c] += bias[c] for n_rows rows of `width` float32 values, in place.
 int mll_add_bias(float* values, const float* bias, int64_t n_rows, int width, hipStream_t stream);
@@ -105,9 +108,15 @@ int mll_paged_attention_prefill(const void* q, const void* k_cache, const void* 
                                 int heads, int kv_heads, int head_dim, int page_size, hipStream_t stream);
 int mll_paged_attention_prefill_tile();
 
-// out[t, c] = silu(gate[t, c]) * up[t, c]; gate and up rows are `in_stride` elements apart.
-int mll_silu_mul(const void* gate, const void* up, int64_t in_stride, void* out, int dtype,
-                 int n_tokens, int width, hipStream_t stream);
+// out[t, c] = act(gate[t, c]) * up[t, c]; gate and up rows are `in_stride` elements apart. act: 0 SiLU, 2 the tanh gelu.
+int mll_gated_activation(const void* gate, const void* up, int64_t in_stride, void* out, int dtype,
+                         int n_tokens, int width, int act, hipStream_t stream);
+
+// out[t][c] = gelu_tanh(z[t][c]) * table[ids[t]][column_at + c] for c < dim, in `dtype`: z float32 [n_tokens][dim], perhaps
+// in n_parts parts that are added in order; table rows (in `table_dtype`) are table_stride elements apart. An id outside
+// [0, vocab) gives a row of NaN.
+int mll_token_side_gate(const float* z, int n_parts, int64_t part_stride, const void* table, int table_dtype, int64_t table_stride,
+                        int column_at, int vocab, const int32_t* ids, void* out, int dtype, int n_tokens, int dim, hipStream_t stream);
 
 // C[m, n] = sum_k A[m, k] * W[n, k] (+ bias[n]), all float32, k summed in ascending order by one
 // thread per output element, so a row's result does not depend on the other rows. With splits > 1
@@ -123,7 +132,7 @@ int mll_gemm_f32(const float* a, const float* w, const float* bias, float* c,
 // C = A . W^T for bfloat16 A [m <= 64, k] and a weight packed as [n/16][k/32][4][16][8] (zero padded):
 // element (row, col) of W sits at piece (row / 16, col / 32), position ((col % 32) / 8, row % 16, col % 8).
 // epilogue 0: float32 [m, n]; 1: bfloat16 [m, n]; 2: bfloat16 [m, n / 2] = silu(even weight rows' results) *
-// (odd rows' results). The order of additions is fixed by (n, k): the same in every run and whatever the
+// (odd rows' results); 5: the same with the tanh form of gelu for silu. The order of additions is fixed by (n, k): the same in every run and whatever the
 // other rows of A.
 // With `scale` (may be null; at most 16 rows) row r of the product is first multiplied by
 // 1 / sqrt(sum_{g < groups} sumsq[r][g] / width + eps): the factor of an RMS norm whose input came without it.
@@ -184,7 +193,7 @@ int mll_gemm_medium(const void* a, const void* w_packed, void* out, int epilogue
                     int tiles_per_wave, int waves, int splits, hipStream_t stream);
 
 // The same product for many rows: 256 x 256 tiles of C per workgroup, pieces of A and W brought into LDS by
-// direct global-to-LDS loads. A is row-major [m, k] with k a multiple of 32; epilogues 0, 1 and 2 of
+// direct global-to-LDS loads. A is row-major [m, k] with k a multiple of 32; epilogues 0, 1, 2 and 5 of
 // mll_gemm_skinny. With epilogue 0, `splits` > 1 deals the stages of 64 of k to that many workgroups per tile:
 // out is then [splits, m, n] partial sums for the caller to add in order. For weights that are kept in the packed
 // order alone.
@@ -247,6 +256,8 @@ typedef struct MllAttentionExtras {
     int chunk;              // > 0 (and no window): a query at p sees the keys from floor(p / chunk) * chunk on
     const float* gate;      // null, or float32 rows gate_stride apart, one number a head: the head's result times sigmoid(gate[t][head])
     int64_t gate_stride;
+    float softcap;          // > 0: the scaled score becomes softcap * tanh(score / softcap), before a bias is added
+    int gate_channels;      // with gate: its rows hold heads * head_dim numbers, one for every channel of the result
 } MllAttentionExtras;
 
 int mll_paged_attention_decode_extra(const void* q, const void* k_cache, const void* v_cache,
@@ -300,12 +311,13 @@ int mll_clamped_glu(const float* gate_up, void* out, int dtype, int n_tokens, in
 // page; key_dim == value_dim), into pages in the MFMA kernels' order (cache_layout.h).
 // Rows of qkv lie row_stride floats apart (they may hold further columns after the values). With cos_sin (float32
 // [n_tokens][rot_dims / 2][cos, sin]) queries and keys are turned after their norm: channel i < rot_dims / 2 of a head
-// with channel i + rot_dims / 2, (u, v) -> (u cos - v sin, v cos + u sin); the other channels pass.
+// with channel i + rot_dims / 2, (u, v) -> (u cos - v sin, v cos + u sin); the other channels pass. values_normed: values
+// are divided by their root mean square over their head (no weight) before they are stored.
 int mll_qk_norm_store(const float* qkv, int n_parts, int64_t part_stride, const float* q_weight, const float* k_weight,
                       float eps, const int32_t* positions, const int32_t* slot_mapping, float temp_coef, int temp_every,
                       void* q_out, void* k_pages, void* v_pages, int dtype, int n_tokens, int heads, int kv_heads, int key_dim,
                       int value_dim, int tiled_page_size, const float* bias, int normed, int queries_only, int64_t row_stride,
-                      const float* cos_sin, int rot_dims, hipStream_t stream);
+                      const float* cos_sin, int rot_dims, int values_normed, hipStream_t stream);
 
 // Causal attention of every token over its request's pages: score_j = (q . k_j) * scale + bias[min(p - j, longest)][head]
 // (bias null: none; float32 [longest + 1][heads]) - slopes[head] * (p - j) (slopes null: none); softmax over j <= p
@@ -313,12 +325,14 @@ int mll_qk_norm_store(const float* qkv, int n_parts, int64_t part_stride, const 
 // (sink null: not); out[t][head] = out_scale * sum_j weight_j v_j, rows out_stride elements apart.
 // A token whose seq_of_token is negative is skipped. The order of every sum depends on p alone.
 // With chunk > 0 (and no window) a query at p sees the keys from floor(p / chunk) * chunk on. With gate (float32, rows
-// gate_stride apart, one number a head) the head's result is multiplied by sigmoid(gate[t][head]).
+// gate_stride apart, one number a head) the head's result is multiplied by sigmoid(gate[t][head]); with gate_channels its
+// rows hold heads * value_dim numbers, one for every channel. softcap > 0: the scaled score becomes softcap *
+// tanh(score / softcap) before anything is added to it.
 int mll_bias_attention(const void* q, const void* k_pages, const void* v_pages, const int32_t* block_table, int table_width,
                        const int32_t* seq_of_token, const int32_t* positions, const float* bias, int longest,
                        const float* sink, void* out, int64_t out_stride, int dtype, int n_tokens, int heads, int kv_heads,
                        int key_dim, int value_dim, int page_size, float scale, float out_scale, const float* slopes, int window,
-                       int chunk, const float* gate, int64_t gate_stride, hipStream_t stream);
+                       int chunk, const float* gate, int64_t gate_stride, float softcap, int gate_channels, hipStream_t stream);
 
 // ---- gated linear attention --------------------------------------------------------------------------------
 
@@ -332,16 +346,25 @@ int mll_gla_decay(const float* proj, int64_t proj_stride, int low_offset, int ra
 // q, k, v are float32 columns of proj's rows at the given offsets. A request without tokens is passed over.
 // long_portions: the kernel that brings tiles of tokens through LDS (for steps with portions of many tokens); the
 // same operations per token in the same order either way, so the same bits.
+// silu_inputs: q, k and v pass SiLU as they are read (not with long_portions, which takes them after mll_gla_silu).
 // decay: float32, token t's heads * key_dim numbers at decay + t * decay_stride (0: one row for every token).
 int mll_gla_scan(const float* proj, int64_t proj_stride, int q_offset, int k_offset, int v_offset, const float* decay,
                  float* state, const int32_t* cu_tokens, const int32_t* slots, float* out, int n_seqs, int heads, int key_dim,
-                 int value_dim, float q_scale, int long_portions, int64_t decay_stride, hipStream_t stream);
+                 int value_dim, float q_scale, int long_portions, int64_t decay_stride, int silu_inputs, hipStream_t stream);
 
 // out[t][head] = o[t][head] / rms(o[t][head]) * weight * silu(gate[t][head]) * out_scale, gate at gate_offset of
 // proj's rows (weight null: none); out in `dtype`, rows out_stride elements apart.
 int mll_gla_gate(const float* o, const float* proj, int64_t proj_stride, int gate_offset, const float* weight, float eps,
                  void* out, int64_t out_stride, int dtype, int n_tokens, int heads, int value_dim, float out_scale,
                  hipStream_t stream);
+
+// Columns first .. first + count - 1 of every row of proj, in place: silu.
+int mll_gla_silu(float* proj, int64_t proj_stride, int first, int count, int n_tokens, hipStream_t stream);
+
+// mll_gla_gate with one norm over all heads of a token, a weight [width] (nullable) and a sigmoid gate:
+// out[t][c] = o[t][c] / rms(o[t]) * weight[c] * sigmoid(gate[t][c]) * out_scale for c < width = heads * value_dim.
+int mll_gla_gate_all(const float* o, const float* proj, int64_t proj_stride, int gate_offset, const float* weight, float eps,
+                     void* out, int64_t out_stride, int dtype, int n_tokens, int width, float out_scale, hipStream_t stream);
 
 // ---- attention through latents (csrc/latent_attention.hip) ----------------------------------------------------
 

@@ -111,25 +111,32 @@ def rms_norm(h: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype: torch
     return out
 
 
-def rms_norm_after(h: torch.Tensor, delta: torch.Tensor, after_weight: torch.Tensor, after_eps: float, mult: float,
+def rms_norm_after(h: torch.Tensor, delta: Optional[torch.Tensor], after_weight: Optional[torch.Tensor], after_eps: float, mult: float,
                    weight: Optional[torch.Tensor], eps: float, out_dtype: torch.dtype, rows: Optional[torch.Tensor] = None,
-                   write_h: bool = False, extra: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+                   write_h: bool = False, extra: Optional[torch.Tensor] = None, groups: int = 1,
+                   raw: bool = False) -> Optional[torch.Tensor]:
     """``v = h[rows] + mult * rms_norm(delta[rows]) * after_weight`` (``delta`` may be float32 partial sums ``[parts,
     tokens, width]``, added in order first), plus ``extra[rows]`` (float32 rows like ``h``'s) if given; with ``write_h`` the
-    sum replaces ``h``; returns ``rms_norm(v) * weight``, or None without ``weight``."""
+    sum replaces ``h``; returns ``rms_norm(v) * weight``, without ``weight`` ``v`` itself if ``raw``, else None. With
+    ``delta`` None (and no weight of it) ``v = h[rows]``. With ``groups`` the mean of squares of either norm is taken over
+    each of that many equal runs of neighbouring columns."""
     lib = library.load()
     _device_tensor(h, "residual stream", torch.float32)
-    _device_tensor(after_weight, "norm weight of the delta", torch.float32)
-    _need(h.dim() == 2 and tuple(after_weight.shape) == (h.shape[1],), "the delta's norm weight must match the stream's width")
+    _need(h.dim() == 2 and (delta is None) == (after_weight is None), "a stream [tokens, width]; a delta and its norm's weight, or neither")
     width = h.shape[1]
-    _device_tensor(delta, "delta")
-    _need(delta.dtype in (torch.float32, out_dtype), "delta must be float32 or have the output's dtype")
-    n_partials = 1
-    if delta.dim() == 3:
-        n_partials = delta.shape[0]
-        _need(n_partials >= 1 and tuple(delta.shape[1:]) == tuple(h.shape), "delta parts must have the residual stream's shape")
-    else:
-        _need(tuple(delta.shape) == tuple(h.shape), "delta must have the residual stream's shape")
+    _need(groups >= 1 and width % groups == 0, "a norm in groups cuts the width into equal parts")
+    n_partials, delta_code = 1, F32
+    if delta is not None:
+        _device_tensor(after_weight, "norm weight of the delta", torch.float32)
+        _need(tuple(after_weight.shape) == (width,), "the delta's norm weight must match the stream's width")
+        _device_tensor(delta, "delta")
+        _need(delta.dtype in (torch.float32, out_dtype), "delta must be float32 or have the output's dtype")
+        delta_code = _code(delta.dtype)
+        if delta.dim() == 3:
+            n_partials = delta.shape[0]
+            _need(n_partials >= 1 and tuple(delta.shape[1:]) == tuple(h.shape), "delta parts must have the residual stream's shape")
+        else:
+            _need(tuple(delta.shape) == tuple(h.shape), "delta must have the residual stream's shape")
     if rows is not None:
         _device_tensor(rows, "row selection", torch.int32)
         _need(not write_h, "cannot write h through a row selection")
@@ -143,10 +150,11 @@ def rms_norm_after(h: torch.Tensor, delta: torch.Tensor, after_weight: torch.Ten
     if weight is not None:
         _device_tensor(weight, "norm weight", torch.float32)
         _need(tuple(weight.shape) == (width,), "the norm weight must match the stream's width")
+    if weight is not None or raw:
         out = torch.empty((n_rows, width), dtype=out_dtype, device=h.device)
-    _check(lib.mll_rms_norm_after(_ptr(h), _ptr(delta), _code(delta.dtype), n_partials, ctypes.c_int64(h.numel()), _ptr(rows),
+    _check(lib.mll_rms_norm_after(_ptr(h), _ptr(delta), delta_code, n_partials, ctypes.c_int64(h.numel()), _ptr(rows),
                                   _ptr(after_weight), ctypes.c_float(after_eps), ctypes.c_float(mult), _ptr(extra), _ptr(weight),
-                                  ctypes.c_float(eps), _ptr(out), _code(out_dtype), n_rows, width, int(write_h), _stream()), lib)
+                                  ctypes.c_float(eps), _ptr(out), _code(out_dtype), n_rows, width, int(write_h), int(groups), _stream()), lib)
     return out
 
 
@@ -461,24 +469,50 @@ def paged_attention_rowwise(q: torch.Tensor, k_cache: torch.Tensor, v_cache: tor
     return out
 
 
+GATED_ACTIVATIONS = {"silu": "gated", "gelu_tanh": "gated_gelu"}      # a gate's activation -> the products' epilogue
+
+
 def silu_mul(gate_up: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """``silu(gate) * up`` of fused rows ``[tokens, 2 * width]`` (gate first)."""
+    return gated_activation(gate_up, "silu", out)
+
+
+def gated_activation(gate_up: torch.Tensor, kind: str, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``act(gate) * up`` of fused rows ``[tokens, 2 * width]`` (gate first); ``kind``: ``silu`` or ``gelu_tanh``."""
     lib = library.load()
+    _need(kind in GATED_ACTIVATIONS, f"no gate with the activation {kind!r}")
     _device_tensor(gate_up, "gate/up")
     _need(gate_up.dim() == 2 and gate_up.shape[1] % 2 == 0, "gate/up must be [tokens, 2 * width]")
     n_tokens, double = gate_up.shape
     width = double // 2
     if out is None:
         out = torch.empty((n_tokens, width), dtype=gate_up.dtype, device=gate_up.device)
-    _device_tensor(out, "silu_mul output", gate_up.dtype)
-    _need(tuple(out.shape) == (n_tokens, width), "silu_mul output has the wrong shape")
+    _device_tensor(out, "gated output", gate_up.dtype)
+    _need(tuple(out.shape) == (n_tokens, width), "the gated output has the wrong shape")
     element = gate_up.element_size()
     for start in range(0, n_tokens, 65535):
         count = min(65535, n_tokens - start)
         gate_ptr = gate_up.data_ptr() + start * double * element
-        _check(lib.mll_silu_mul(ctypes.c_void_p(gate_ptr), ctypes.c_void_p(gate_ptr + width * element),
+        _check(lib.mll_gated_activation(ctypes.c_void_p(gate_ptr), ctypes.c_void_p(gate_ptr + width * element),
                                 ctypes.c_int64(double), ctypes.c_void_p(out.data_ptr() + start * width * element),
-                                _code(gate_up.dtype), count, width, _stream()), lib)
+                                _code(gate_up.dtype), count, width, ACTIVATIONS[kind], _stream()), lib)
+    return out
+
+
+def token_side_gate(z: torch.Tensor, table: torch.Tensor, column_at: int, ids: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
+    """``gelu_tanh(z) * table[ids][:, column_at : column_at + dim]`` in ``out_dtype``: ``z`` float32 ``[tokens, dim]`` or partial
+    sums ``[parts, tokens, dim]``, added in order first; an id outside the table gives a row of NaN."""
+    lib = library.load()
+    n_parts, part_stride = _parts_of(z, "side gate")
+    n_tokens, dim = z.shape[-2:]
+    _device_tensor(table, "side table")
+    _device_tensor(ids, "token ids", torch.int32)
+    _need(table.dim() == 2 and 0 <= column_at and column_at + dim <= table.shape[1], "the layer's columns lie inside the side table")
+    _need(ids.shape[0] >= n_tokens, "an id for every token")
+    out = torch.empty((n_tokens, dim), dtype=out_dtype, device=z.device)
+    _check(lib.mll_token_side_gate(_ptr(z), n_parts, ctypes.c_int64(part_stride), _ptr(table), _code(table.dtype),
+                                   ctypes.c_int64(table.shape[1]), int(column_at), table.shape[0], _ptr(ids), _ptr(out),
+                                   _code(out_dtype), n_tokens, dim, _stream()), lib)
     return out
 
 
@@ -683,7 +717,7 @@ def gemm_bf16_split(x: torch.Tensor, weight: torch.Tensor, parts: int) -> torch.
 class _AttentionExtras(ctypes.Structure):
     _fields_ = [("bias", ctypes.c_void_p), ("longest", ctypes.c_int), ("sink", ctypes.c_void_p),
                 ("out_scale", ctypes.c_float), ("out_stride", ctypes.c_int64), ("chunk", ctypes.c_int), ("gate", ctypes.c_void_p),
-                ("gate_stride", ctypes.c_int64)]
+                ("gate_stride", ctypes.c_int64), ("softcap", ctypes.c_float), ("gate_channels", ctypes.c_int)]
 
 
 class AttentionExtras(NamedTuple):
@@ -691,12 +725,24 @@ class AttentionExtras(NamedTuple):
     the scaled scores by ``min(distance, last row)``; ``sink`` float32 ``[heads]``, one more term ``exp(sink)`` of the
     softmax's denominator; a factor on the result; ``chunk``: a query at ``p`` sees the keys from ``floor(p / chunk) *
     chunk`` on (no window then); ``gate`` float32 ``[tokens, heads]`` (columns of a wider buffer allowed): a head's result
-    is multiplied by ``sigmoid(gate)``."""
+    is multiplied by ``sigmoid(gate)``; ``[tokens, heads * head_dim]``: every channel of the result by its own;
+    ``softcap`` c (0: none): the scaled score becomes ``c * tanh(score / c)`` before a bias is added."""
     bias: Optional[torch.Tensor] = None
     sink: Optional[torch.Tensor] = None
     out_scale: float = 1.0
     chunk: int = 0
     gate: Optional[torch.Tensor] = None
+    softcap: float = 0.0
+
+
+def _gate_stride(gate: Optional[torch.Tensor], n_tokens: int, heads: int, value_dim: int) -> Tuple[int, bool]:
+    """The stride of a gate's rows and whether it has a number for every channel (else one a head)."""
+    if gate is None:
+        return 0, False
+    _need(gate.is_cuda and gate.dtype == torch.float32 and gate.dim() == 2 and gate.stride(1) == 1 and gate.shape[0] == n_tokens
+          and gate.shape[1] in (heads, heads * value_dim),
+          "the gate is float32 [tokens, heads] or [tokens, heads * value_dim] with unit column stride")
+    return max(gate.stride(0), gate.shape[1]), gate.shape[1] != heads
 
 
 def prefill_bias_rows() -> int:
@@ -718,17 +764,14 @@ def _extras_argument(extras: Optional[AttentionExtras], heads: int, head_dim: in
         _need(tuple(extras.sink.shape) == (heads,), "one sink a head")
     _need(out.dim() == 2 and out.stride(1) == 1 and out.shape[1] == heads * head_dim, "the output is [tokens, heads * head_dim] with unit column stride")
     stride = max(out.stride(0), heads * head_dim)
-    gate_stride = 0
-    if extras.gate is not None:
-        gate = extras.gate
-        _need(gate.is_cuda and gate.dtype == torch.float32 and gate.dim() == 2 and tuple(gate.shape) == (out.shape[0], heads)
-              and gate.stride(1) == 1, "the gate is float32 [tokens, heads] with unit column stride")
-        gate_stride = max(gate.stride(0), heads)
+    gate_stride, gate_channels = _gate_stride(extras.gate, out.shape[0], heads, head_dim)
+    _need(extras.softcap >= 0.0, "the cap on the scores is positive, or 0 for none")
     _need(extras.chunk >= 0, "chunks of positions are positive, or 0 for none")
     return ctypes.byref(_AttentionExtras(extras.bias.data_ptr() if extras.bias is not None else None, longest,
                                          extras.sink.data_ptr() if extras.sink is not None else None,
                                          float(extras.out_scale), stride, int(extras.chunk),
-                                         extras.gate.data_ptr() if extras.gate is not None else None, gate_stride))
+                                         extras.gate.data_ptr() if extras.gate is not None else None, gate_stride,
+                                         float(extras.softcap), int(gate_channels)))
 
 
 def decode_splits(n_tokens: int, kv_heads: int, longest: int) -> int:
@@ -911,7 +954,7 @@ def gemm_skinny(x: torch.Tensor, packed: torch.Tensor, n: int, epilogue: str = "
     """``x @ W.T`` for at most 64 bfloat16 rows and a packed weight.
 
     ``f32``: float32 ``[m, n]``; ``bf16``: bfloat16 ``[m, n]``; ``gated``: bfloat16 ``[m, n / 2]`` of
-    silu(gate) * up for interleaved rows. With ``scale`` (at most 16 rows) the rows of the product are
+    silu(gate) * up for interleaved rows; ``gated_gelu`` the same with the tanh form of gelu. With ``scale`` (at most 16 rows) the rows of the product are
     multiplied by its factors first.
     """
     lib = library.load()
@@ -929,6 +972,8 @@ def gemm_skinny(x: torch.Tensor, packed: torch.Tensor, n: int, epilogue: str = "
         code, out = 1, torch.empty((m, n), dtype=torch.bfloat16, device=x.device)
     elif epilogue == "gated":
         code, out = 2, torch.empty((m, n // 2), dtype=torch.bfloat16, device=x.device)
+    elif epilogue == "gated_gelu":
+        code, out = 5, torch.empty((m, n // 2), dtype=torch.bfloat16, device=x.device)
     else:
         raise KernelLibraryError(f"unknown epilogue {epilogue!r}")
     _check(lib.mll_gemm_skinny(_ptr(x), _ptr(packed), _ptr(out), code, m, n, k, _scale_argument(scale, m), _stream()), lib)
@@ -966,7 +1011,7 @@ def gemm_medium(x: torch.Tensor, packed: torch.Tensor, n: int, epilogue: str = "
     ``plan`` is ``medium_plan``'s by default; pass ``medium_plan(n, k, may_split=False)`` for a plain ``[m, n]``.
 
     ``f32``: float32 ``[m, n]``, or ``[splits, m, n]`` partial sums to be added in order when the plan splits k;
-    ``bf16`` and ``gated`` as in ``gemm_skinny`` (they never split).
+    ``bf16``, ``gated`` and ``gated_gelu`` as in ``gemm_skinny`` (they never split).
     """
     lib = library.load()
     _device_tensor(x, "gemm input", torch.bfloat16)
@@ -986,6 +1031,8 @@ def gemm_medium(x: torch.Tensor, packed: torch.Tensor, n: int, epilogue: str = "
         code, out = 1, torch.empty((m, n), dtype=torch.bfloat16, device=x.device)
     elif epilogue == "gated":
         code, out = 2, torch.empty((m, n // 2), dtype=torch.bfloat16, device=x.device)
+    elif epilogue == "gated_gelu":
+        code, out = 5, torch.empty((m, n // 2), dtype=torch.bfloat16, device=x.device)
     else:
         raise KernelLibraryError(f"unknown epilogue {epilogue!r}")
     _check(lib.mll_gemm_medium(_ptr(x), _ptr(packed), _ptr(out), code, m, n, k, tiles_per_wave, waves, splits, _stream()), lib)
@@ -1036,14 +1083,16 @@ def gemm_tiled(x: torch.Tensor, packed: torch.Tensor, n: int, epilogue: str = "f
     m, k = x.shape
     _need(k % 32 == 0, "gemm_tiled needs k to be a multiple of 32")
     _need(packed.shape[0] == -(-n // 16) and packed.shape[1] == k // 32, "the packed weight does not fit n and k")
+    _need(epilogue not in ("gated", "gated_gelu") or n % 2 == 0, "the gated epilogue needs an even number of weight rows")
     _need(splits >= 1 and (splits == 1 or epilogue == "f32"), "only the float32 epilogue takes the reduction in parts")
     if epilogue == "f32":
         code, out = 0, torch.empty((m, n) if splits == 1 else (splits, m, n), dtype=torch.float32, device=x.device)
     elif epilogue == "bf16":
         code, out = 1, torch.empty((m, n), dtype=torch.bfloat16, device=x.device)
     elif epilogue == "gated":
-        _need(n % 2 == 0, "the gated epilogue needs an even number of weight rows")
         code, out = 2, torch.empty((m, n // 2), dtype=torch.bfloat16, device=x.device)
+    elif epilogue == "gated_gelu":
+        code, out = 5, torch.empty((m, n // 2), dtype=torch.bfloat16, device=x.device)
     else:
         raise KernelLibraryError(f"unknown epilogue {epilogue!r}")
     _check(lib.mll_gemm_tiled(_ptr(x), _ptr(packed), _ptr(out), code, m, n, k, splits, tile_rows, _stream()), lib)
@@ -1233,7 +1282,7 @@ def qk_norm_store(qkv: torch.Tensor, q_weight: Optional[torch.Tensor], k_weight:
                   k_pages: torch.Tensor, v_pages: torch.Tensor, heads: int, kv_heads: int, key_dim: int, value_dim: int,
                   out_dtype: torch.dtype, tiled_page_size: int = 0, bias: Optional[torch.Tensor] = None,
                   normed: Optional[bool] = None, queries_only: bool = False, cos_sin: Optional[torch.Tensor] = None,
-                  further_columns: int = 0) -> torch.Tensor:
+                  further_columns: int = 0, values_normed: bool = False) -> torch.Tensor:
     """Norm of queries and keys over their head, the queries' factor by position, keys and values into their pages
     (``[page, position, kv_head, dim]``, or with ``tiled_page_size`` the pages of ``cache.layout`` with that many
     positions each); returns the queries ``[tokens, heads * key_dim]``. ``bias`` (one number a column of a row) is
@@ -1241,7 +1290,8 @@ def qk_norm_store(qkv: torch.Tensor, q_weight: Optional[torch.Tensor], k_weight:
     also without weights. With ``queries_only`` the rows hold queries alone and nothing is stored (a layer that
     reads another's keys and values). With ``cos_sin`` (``rope_table``'s ``[tokens, n, 2]``) queries and keys are turned
     after their norm in their first ``2 n`` channels, channel ``i`` with ``i + n``. The rows may hold
-    ``further_columns`` after the values (what another kernel reads from the same product)."""
+    ``further_columns`` after the values (what another kernel reads from the same product). ``values_normed``: values are
+    divided by their root mean square over their head before they are stored."""
     lib = library.load()
     n_parts, part_stride = _parts_of(qkv, "q/k/v")
     n_tokens = qkv.shape[-2]
@@ -1269,7 +1319,7 @@ def qk_norm_store(qkv: torch.Tensor, q_weight: Optional[torch.Tensor], k_weight:
                                      ctypes.c_float(eps), _ptr(positions), None, ctypes.c_float(temp_coef),
                                      int(temp_every), _ptr(q_out), None, None, _code(out_dtype), n_tokens,
                                      heads, kv_heads, key_dim, value_dim, 0, _ptr(bias), int(normed), 1, row_stride, _ptr(cos_sin),
-                                     rot_dims, _stream()), lib)
+                                     rot_dims, 0, _stream()), lib)
         return q_out
     _device_tensor(slot_mapping, "slot mapping", torch.int32)
     _need(slot_mapping.shape[0] >= n_tokens, "a slot for every token")
@@ -1290,7 +1340,7 @@ def qk_norm_store(qkv: torch.Tensor, q_weight: Optional[torch.Tensor], k_weight:
                                  ctypes.c_float(eps), _ptr(positions), _ptr(slot_mapping), ctypes.c_float(temp_coef),
                                  int(temp_every), _ptr(q_out), _ptr(k_pages), _ptr(v_pages), _code(out_dtype), n_tokens,
                                  heads, kv_heads, key_dim, value_dim, int(tiled_page_size), _ptr(bias), int(normed), 0,
-                                 row_stride, _ptr(cos_sin), rot_dims, _stream()), lib)
+                                 row_stride, _ptr(cos_sin), rot_dims, int(values_normed), _stream()), lib)
     return q_out
 
 
@@ -1298,12 +1348,13 @@ def bias_attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor
                    seq_of_token: torch.Tensor, positions: torch.Tensor, bias: Optional[torch.Tensor],
                    sink: Optional[torch.Tensor], scale: float, out_scale: float, heads: int, kv_heads: int, key_dim: int,
                    value_dim: int, out: Optional[torch.Tensor] = None, slopes: Optional[torch.Tensor] = None,
-                   window: int = 0, chunk: int = 0, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                   window: int = 0, chunk: int = 0, gate: Optional[torch.Tensor] = None, softcap: float = 0.0) -> torch.Tensor:
     """Causal attention with ``bias[min(distance, last row), head]`` added to the scaled scores, ``slopes[head] *
     distance`` taken off them, and ``exp(sink[head])`` in the softmax's denominator; with ``window`` a query sees
     itself and the ``window - 1`` keys before it; with ``chunk`` the keys from ``floor(p / chunk) * chunk`` on; with ``gate``
-    (float32 ``[tokens, heads]``, columns of a wider buffer allowed) a head's result is multiplied by ``sigmoid(gate)``;
-    ``out`` may be columns of a wider buffer (its row stride is taken)."""
+    (float32 ``[tokens, heads]``, columns of a wider buffer allowed) a head's result is multiplied by ``sigmoid(gate)``, with
+    ``[tokens, heads * value_dim]`` every channel by its own; ``softcap`` c (0: none): the scaled score becomes ``c * tanh(score
+    / c)`` before anything is added to it; ``out`` may be columns of a wider buffer (its row stride is taken)."""
     lib = library.load()
     _device_tensor(q, "queries")
     n_tokens = q.shape[0]
@@ -1331,11 +1382,7 @@ def bias_attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor
         _device_tensor(slopes, "slopes", torch.float32)
         _need(tuple(slopes.shape) == (heads,), "one slope a head")
     _need(window >= 0 and chunk >= 0 and not (window and chunk), "a window or chunks of positions (0 for none), not both")
-    gate_stride = 0
-    if gate is not None:
-        _need(gate.is_cuda and gate.dtype == torch.float32 and gate.dim() == 2 and tuple(gate.shape) == (n_tokens, heads)
-              and gate.stride(1) == 1, "the gate is float32 [tokens, heads] with unit column stride")
-        gate_stride = max(gate.stride(0), heads)
+    gate_stride, gate_channels = _gate_stride(gate, n_tokens, heads, value_dim)
     if out is None:
         out = torch.empty((n_tokens, heads * value_dim), dtype=q.dtype, device=q.device)
     _need(out.is_cuda and out.dtype == q.dtype and out.dim() == 2 and tuple(out.shape) == (n_tokens, heads * value_dim)
@@ -1345,7 +1392,8 @@ def bias_attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor
                                   ctypes.c_void_p(out.data_ptr()), ctypes.c_int64(out.stride(0) if n_tokens > 1 else max(out.stride(0), heads * value_dim)),
                                   _code(q.dtype), n_tokens, heads, kv_heads, key_dim, value_dim, page_size,
                                   ctypes.c_float(scale), ctypes.c_float(out_scale), _ptr(slopes), int(window), int(chunk),
-                                  ctypes.c_void_p(gate.data_ptr()) if gate is not None else None, ctypes.c_int64(gate_stride), _stream()), lib)
+                                  ctypes.c_void_p(gate.data_ptr()) if gate is not None else None, ctypes.c_int64(gate_stride),
+                                  ctypes.c_float(softcap), int(gate_channels), _stream()), lib)
     return out
 
 
@@ -1372,11 +1420,13 @@ def gla_decay(proj: torch.Tensor, low_offset: int, a2: torch.Tensor, bias: Optio
 
 def gla_scan(proj: torch.Tensor, q_offset: int, k_offset: int, v_offset: int, decay: torch.Tensor, state: torch.Tensor,
              cu_tokens: torch.Tensor, slots: torch.Tensor, n_seqs: int, heads: int, key_dim: int, value_dim: int,
-             q_scale: float, long_portions: bool = False) -> torch.Tensor:
+             q_scale: float, long_portions: bool = False, silu_inputs: bool = False) -> torch.Tensor:
     """The recurrence over every request's tokens of the step; ``state`` is ``[slots, heads, key_dim, value_dim]``
     float32, read and written at ``slots``. Returns ``[tokens, heads * value_dim]`` float32. ``long_portions``: the
-    kernel that stages tiles of tokens through LDS, for steps whose requests bring many tokens (the same bits)."""
+    kernel that stages tiles of tokens through LDS, for steps whose requests bring many tokens (the same bits).
+    ``silu_inputs``: queries, keys and values pass SiLU as they are read (short steps only; ``gla_silu`` before a long one)."""
     lib = library.load()
+    _need(not (silu_inputs and long_portions), "the walk over long portions takes inputs that have passed their activation")
     _device_tensor(proj, "projections", torch.float32)
     _device_tensor(decay, "decays", torch.float32)
     _device_tensor(state, "state", torch.float32)
@@ -1391,25 +1441,41 @@ def gla_scan(proj: torch.Tensor, q_offset: int, k_offset: int, v_offset: int, de
     out = torch.empty((n_tokens, heads * value_dim), dtype=torch.float32, device=proj.device)
     _check(lib.mll_gla_scan(_ptr(proj), ctypes.c_int64(proj.shape[1]), q_offset, k_offset, v_offset, _ptr(decay), _ptr(state),
                             _ptr(cu_tokens), _ptr(slots), _ptr(out), n_seqs, heads, key_dim, value_dim,
-                            ctypes.c_float(q_scale), int(long_portions), ctypes.c_int64(decay_stride), _stream()), lib)
+                            ctypes.c_float(q_scale), int(long_portions), ctypes.c_int64(decay_stride), int(silu_inputs), _stream()), lib)
     return out
 
 
+def gla_silu(proj: torch.Tensor, first: int, count: int) -> None:
+    """``silu`` of the columns ``first .. first + count - 1`` of every row, in place."""
+    lib = library.load()
+    _device_tensor(proj, "projections", torch.float32)
+    _need(proj.dim() == 2, "projections are [tokens, columns]")
+    _check(lib.mll_gla_silu(_ptr(proj), ctypes.c_int64(proj.shape[1]), first, count, proj.shape[0], _stream()), lib)
+
+
 def gla_gate(o: torch.Tensor, proj: torch.Tensor, gate_offset: int, weight: Optional[torch.Tensor], eps: float, heads: int,
-             value_dim: int, out_scale: float, out_dtype: torch.dtype, out: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """Per head: ``o / rms(o) * weight * silu(gate) * out_scale`` (``weight`` None: none); ``out`` may be columns of a wider buffer."""
+             value_dim: int, out_scale: float, out_dtype: torch.dtype, out: Optional[torch.Tensor] = None,
+             heads_together: bool = False) -> torch.Tensor:
+    """Per head: ``o / rms(o) * weight * silu(gate) * out_scale`` (``weight`` None: none); ``out`` may be columns of a wider
+    buffer. ``heads_together``: one root mean square over all heads, a weight ``[heads * value_dim]`` and ``sigmoid(gate)``."""
     lib = library.load()
     _device_tensor(o, "recurrence output", torch.float32)
     _device_tensor(proj, "projections", torch.float32)
     if weight is not None:
         _device_tensor(weight, "norm weight", torch.float32)
     n_tokens = o.shape[0]
-    _need(tuple(o.shape) == (n_tokens, heads * value_dim) and proj.shape[0] == n_tokens and (weight is None or tuple(weight.shape) == (value_dim,)),
-          "gla_gate takes [tokens, heads * value_dim], the projections of the same tokens and a weight [value_dim]")
+    _need(tuple(o.shape) == (n_tokens, heads * value_dim) and proj.shape[0] == n_tokens and
+          (weight is None or tuple(weight.shape) == (heads * value_dim if heads_together else value_dim,)),
+          "gla_gate takes [tokens, heads * value_dim], the projections of the same tokens and a weight of the normed size")
     if out is None:
         out = torch.empty((n_tokens, heads * value_dim), dtype=out_dtype, device=o.device)
     _need(out.is_cuda and out.dtype == out_dtype and tuple(out.shape) == (n_tokens, heads * value_dim) and out.stride(1) == 1,
           "the output is [tokens, heads * value_dim] with unit column stride")
+    if heads_together:
+        _check(lib.mll_gla_gate_all(_ptr(o), _ptr(proj), ctypes.c_int64(proj.shape[1]), gate_offset, _ptr(weight), ctypes.c_float(eps),
+                                    ctypes.c_void_p(out.data_ptr()), ctypes.c_int64(max(out.stride(0), heads * value_dim)), _code(out_dtype),
+                                    n_tokens, heads * value_dim, ctypes.c_float(out_scale), _stream()), lib)
+        return out
     _check(lib.mll_gla_gate(_ptr(o), _ptr(proj), ctypes.c_int64(proj.shape[1]), gate_offset, _ptr(weight), ctypes.c_float(eps),
                             ctypes.c_void_p(out.data_ptr()), ctypes.c_int64(max(out.stride(0), heads * value_dim)), _code(out_dtype),
                             n_tokens, heads, value_dim, ctypes.c_float(out_scale), _stream()), lib)

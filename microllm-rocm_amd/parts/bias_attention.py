@@ -1,6 +1,7 @@
 """Causal softmax attention with the pieces that designs put around it, each a parameter: a norm of queries and keys, a
 learned bias by distance bucket or a slope a head times the distance, a rotation of queries and keys, a sink in the
-softmax, a query factor that grows with the position, a sliding window or a mask by chunks of positions, a gate a head.
+softmax, a query factor that grows with the position, a sliding window or a mask by chunks of positions, a cap on the
+scores, a norm of values, a gate a head or a channel.
 
 ``q = Wq x``, ``k = Wk x``, ``v = Wv x`` (with ``projection_bias`` each and the output projection have a bias, named
 as the weight with ``_bias``); query head ``h`` uses kv head ``h // (heads / kv_heads)``; keys
@@ -15,8 +16,12 @@ softmax's denominator also holds ``exp(sink[h])``, which has no key and no value
 that number instead of a tensor (0: one is added to the denominator). With ``chunk`` a query sees ``j <= i`` with
 ``floor(j / chunk) = floor(i / chunk)``, positions counted from the sequence's start. With ``position`` (a split-half
 rotary encoding, which may turn fewer channels than the head has and stretch positions) queries and keys are turned
-after their norm. With ``head_gate`` head ``h``'s result is multiplied by ``sigmoid(Wg x)_h``, ``Wg`` being ``[heads,
-hidden]``, one more block of rows of the stacked input product. With ``window`` a query sees
+after their norm; an encoding that pairs neighbouring channels has the rows of ``Wq`` and ``Wk`` that make them (and their
+biases and norm weights) reordered once, at load, since queries and keys only meet in their dot product. With
+``softcap`` ``c`` the scaled score becomes ``c * tanh(score / c)`` before bias or slopes. With ``value_norm`` every head of
+values is divided by its root mean square (no weight) before it is cached. With ``head_gate`` head ``h``'s result is multiplied by ``sigmoid(Wg x)_h``, ``Wg`` being ``[heads,
+hidden]``, one more block of rows of the stacked input product; with ``channel_gate`` ``Wg`` is ``[heads * value_dim,
+hidden]`` and every channel of the results has a gate of its own. With ``window`` a query sees
 ``0 <= i - j < window``. With ``owns_kv`` false the layer has no ``Wk`` and ``Wv``: it reads the keys (as cached, after
 their norm) and values of another run entry, with queries, bias and window of its own.
 
@@ -79,12 +84,21 @@ class BucketBiasAttention(Mixer):
         self.window = int(p["window"]) if p.get("window") else 0
         self.chunk = int(p["chunk"]) if p.get("chunk") else 0
         self.head_gate = bool(p.get("head_gate", False))
+        self.channel_gate = bool(p.get("channel_gate", False))
+        # columns of the stacked input product that hold the gates
+        self.gate_width = self.heads * self.value_dim if self.channel_gate else (self.heads if self.head_gate else 0)
+        self.softcap = float(p["softcap"]) if p.get("softcap") else 0.0
+        self.value_norm = bool(p.get("value_norm", False))
         self.sink_value = float(p["sink_value"]) if p.get("sink_value") is not None else None
         if self.sink_value is not None:
             self.has_sink = False       # no tensor in the files: the number is the sink of every head
         self.position = build_part("position", p["position"], runtime) if p.get("position") is not None else None
         if self.position is not None and (not self.position.fused_split_half or 2 * self.position.inv_freq.shape[0] > self.key_dim):
             raise ValueError("queries and keys turn by a split-half encoding over at most their head's channels")
+        if self.head_gate and self.channel_gate:
+            raise ValueError("a gate a head or a gate a channel, not both")
+        if self.softcap < 0.0:
+            raise ValueError("the cap on the scores must be positive")
         if self.window and self.chunk:
             raise ValueError("a window or chunks of positions, not both")
         # how long the keys and values are kept: the widest window of the layers that read them (0: for ever)
@@ -132,8 +146,8 @@ class BucketBiasAttention(Mixer):
             decls[self.name("bias")] = TensorDecl((self.bias_rows, self.heads), VECTOR)
         if self.has_sink:
             decls[self.name("sink")] = TensorDecl((self.heads,), VECTOR)
-        if self.head_gate:
-            decls[self.name("g")] = TensorDecl((self.heads, self.hidden), MATRIX)
+        if self.gate_width:
+            decls[self.name("g")] = TensorDecl((self.gate_width, self.hidden), MATRIX)
         return decls
 
     def _in_roles(self):
@@ -142,8 +156,22 @@ class BucketBiasAttention(Mixer):
     def sub_parts(self):
         return (self.position,) if self.position is not None else ()
 
+    def _turned(self, tensor: torch.Tensor, heads: int) -> torch.Tensor:
+        """A tensor with one row a query or key channel (``heads`` heads of them), its rows in the order in which the
+        position encoding turns channels by the split-half rule."""
+        if not hasattr(self.position, "split_half_order"):
+            return tensor
+        order = torch.arange(self.key_dim)
+        turned = self.position.split_half_order()
+        order[:len(turned)] = turned
+        rows = torch.cat([order + head * self.key_dim for head in range(heads)]).to(tensor.device)
+        return tensor[rows].contiguous()
+
     def bind(self, tensors: Mapping[str, torch.Tensor]) -> None:
-        weights = [tensors[self.name(role)] for role in self._in_roles() + (("g",) if self.head_gate else ())]
+        weights = [tensors[self.name(role)] for role in self._in_roles() + (("g",) if self.gate_width else ())]
+        weights[0] = self._turned(weights[0], self.heads)
+        if self.owns_kv:
+            weights[1] = self._turned(weights[1], self.kv_heads)
         if len({w.dtype for w in weights}) != 1:
             raise TypeError("the q, k and v weights of one layer must share a dtype to be stacked")
         self.qkv_weight = Weight(torch.cat(weights, dim=0).contiguous() if len(weights) > 1 else weights[0],
@@ -151,11 +179,14 @@ class BucketBiasAttention(Mixer):
         del weights
         self.o_tensor = tensors[self.name("o")]
         if self.projection_bias:
-            self.qkv_bias = torch.cat([tensors[self.name(f"{role}_bias")] for role in self._in_roles()]).contiguous()
+            turned_heads = {"q": self.heads, "k": self.kv_heads}
+            biases = [tensors[self.name(f"{role}_bias")] for role in self._in_roles()]
+            self.qkv_bias = torch.cat([self._turned(bias, turned_heads[role]) if role in turned_heads else bias
+                                       for role, bias in zip(self._in_roles(), biases)]).contiguous()
             self.o_bias = tensors[self.name("o_bias")]
         if self.qk_norm_weight:
-            self.q_norm = tensors[self.name("q_norm")]
-            self.k_norm = tensors[self.name("k_norm")] if self.owns_kv else None
+            self.q_norm = self._turned(tensors[self.name("q_norm")], 1)
+            self.k_norm = self._turned(tensors[self.name("k_norm")], 1) if self.owns_kv else None
         if self.slope_values is not None:
             device = self.o_tensor.device
             self.slopes = torch.tensor(self.slope_values, dtype=torch.float32, device=device)
@@ -196,7 +227,7 @@ class BucketBiasAttention(Mixer):
             columns += self.heads * self.value_dim
         if self.chunk:
             pairs = sum(position % self.chunk + 1 for position in range(tokens))
-        columns += self.heads if self.head_gate else 0
+        columns += self.gate_width
         return 2.0 * tokens * self.hidden * columns + 2.0 * self.heads * (self.key_dim + self.value_dim) * pairs
 
     def forward_inner(self, x, ctx, cache, out: Optional[torch.Tensor] = None, out_scale: float = 1.0) -> torch.Tensor:
@@ -204,23 +235,24 @@ class BucketBiasAttention(Mixer):
         projection; written into ``out`` if given (columns of a wider buffer)."""
         view = ctx.paged[cache.group]
         # rounded once, after norm and factor; the gate's columns, which the attention kernel reads as they are, want whole sums
-        qkv = linear(x, self.qkv_weight, out_dtype=torch.float32, partials=not self.head_gate)
+        qkv = linear(x, self.qkv_weight, out_dtype=torch.float32, partials=not self.gate_width)
         q = kernels.qk_norm_store(qkv, self.q_norm, self.k_norm, self.eps, ctx.positions, view.slot_mapping, self.temp_coef,
                                   self.temp_every, cache.k, cache.v, self.heads, self.kv_heads, self.key_dim, self.value_dim,
                                   self.runtime.dtype, tiled_page_size=view.page_size if self.tiled else 0, bias=self.qkv_bias,
                                   normed=self.qk_norm, queries_only=not self.owns_kv,
                                   cos_sin=self.position.table(ctx) if self.position is not None else None,
-                                  further_columns=self.heads if self.head_gate else 0)
-        gate = qkv[:, qkv.shape[1] - self.heads:] if self.head_gate else None
+                                  further_columns=self.gate_width, values_normed=self.value_norm)
+        gate = qkv[:, qkv.shape[1] - self.gate_width:] if self.gate_width else None
         if self.tiled:
             if out is None:
                 out = torch.empty((x.shape[0], self.heads * self.value_dim), dtype=self.runtime.dtype, device=x.device)
-            extras = kernels.AttentionExtras(self.bias, self.sink, out_scale, chunk=self.chunk, gate=gate)
+            extras = kernels.AttentionExtras(self.bias, self.sink, out_scale, chunk=self.chunk, gate=gate, softcap=self.softcap)
             return kernels.paged_attention(q, cache.k, cache.v, view, ctx, self.scale, self.window, self.heads, self.kv_heads,
                                            self.key_dim, planner=self.planner, extras=extras, out=out)
         return kernels.bias_attention(q, cache.k, cache.v, view.block_table, ctx.seq_of_token, ctx.positions, self.bias,
                                       self.sink, self.scale, out_scale, self.heads, self.kv_heads, self.key_dim,
-                                      self.value_dim, out=out, slopes=self.slopes, window=self.window, chunk=self.chunk, gate=gate)
+                                      self.value_dim, out=out, slopes=self.slopes, window=self.window, chunk=self.chunk, gate=gate,
+                                      softcap=self.softcap)
 
     def forward(self, x, ctx, cache):
         if self.o_weight is None:

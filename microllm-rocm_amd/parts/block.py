@@ -91,7 +91,9 @@ class SandwichNormBlock(Block):
     """A norm before and a norm after each sublayer, and a factor on what joins the stream:
     ``h' = h + m * NormA(Mixer(Norm1(h)))``, ``h'' = h' + m * NormB(FFN(Norm2(h')))``. The norms after are RMS norms
     named ``mixer_after`` and ``ffn_after`` in ``LayerSpec.extra``; ``m`` is ``LayerSpec.params["residual_mult"]``
-    (1 if absent). A sublayer's result is handed on as a ``NormedDelta``: the norm that reads the stream next norms
+    (1 if absent). A design without norms before its sublayers names ``unnormed`` there. With ``side`` in
+    ``LayerSpec.extra`` (and ``side_norm`` before it, ``side_after`` after it) one more sublayer of that kind follows, which
+    needs the step's token ids beside the stream. A sublayer's result is handed on as a ``NormedDelta``: the norm that reads the stream next norms
     and adds it in the same kernel, so no product adds into the stream itself here."""
 
     def __init__(self, spec: LayerSpec, runtime: Runtime):
@@ -99,23 +101,27 @@ class SandwichNormBlock(Block):
         self.mult = float(spec.params.get("residual_mult", 1.0))
         self.mixer_after = self.extra["mixer_after"]
         self.ffn_after = self.extra.get("ffn_after")
+        self.side = self.extra.get("side")
         if (self.ffn is None) != (self.ffn_after is None):
             raise ValueError("a feed-forward and the norm after it come together")
+        if self.side is not None and not ("side_norm" in self.extra and "side_after" in self.extra):
+            raise ValueError("a side sublayer comes with what stands before and after it")
 
     def _normed(self, values, norm) -> NormedDelta:
-        pieces = norm.weight_then_factor()
-        if pieces is None:
-            raise TypeError("the norm after a sublayer must be an RMS norm with a float32 weight")
-        weight, _, eps = pieces
-        return NormedDelta(values, weight, eps, self.mult)
+        if not hasattr(norm, "delayed"):
+            raise TypeError("the norm after a sublayer must be an RMS norm")
+        return norm.delayed(values, self.mult)
 
     def forward(self, h, pending, ctx, cache, next_block=None):
         x = pending if isinstance(pending, UnscaledRows) else self.mixer_norm.forward(h, delta=pending, write_h=True)
-        mixed = self._normed(self.mixer.forward(x, ctx, cache), self.mixer_after)
-        if self.ffn is None:
-            return mixed
-        x = self.ffn_norm.forward(h, delta=mixed, write_h=True)
-        return self._normed(self.ffn.forward(x, ctx), self.ffn_after)
+        pending = self._normed(self.mixer.forward(x, ctx, cache), self.mixer_after)
+        if self.ffn is not None:
+            x = self.ffn_norm.forward(h, delta=pending, write_h=True)
+            pending = self._normed(self.ffn.forward(x, ctx), self.ffn_after)
+        if self.side is not None:
+            x = self.extra["side_norm"].forward(h, delta=pending, write_h=True)
+            pending = self._normed(self.side.forward(x, ctx), self.extra["side_after"])
+        return pending
 
 
 _ARRANGEMENTS = {"pre_norm": PreNormBlock, "sandwich_norm": SandwichNormBlock}

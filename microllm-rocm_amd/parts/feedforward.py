@@ -1,4 +1,5 @@
-"""The SwiGLU feed-forward: ``down(silu(gate(x)) * up(x))``, no biases.
+"""The SwiGLU feed-forward: ``down(silu(gate(x)) * up(x))``, no biases; ``activation`` may name the tanh form of gelu
+for the gate instead (``gelu_tanh``).
 
 ``z = g * sigmoid(g) * u`` with the sigmoid evaluated branch-stably
 (src/ops/ops.cpp:72-76, 779-783; src/model/model.cpp:787-789). Gate and up are
@@ -24,6 +25,9 @@ class SwiGLU(FeedForward):
         super().__init__(spec, runtime)
         self.hidden = int(spec.params["hidden_size"])
         self.intermediate = int(spec.params["intermediate_size"])
+        self.activation = str(spec.params.get("activation", "silu"))
+        if self.activation not in kernels.GATED_ACTIVATIONS:
+            raise ValueError(f"a gate's activation is one of {', '.join(sorted(kernels.GATED_ACTIVATIONS))}")
         self.gate_up_weight: Optional[torch.Tensor] = None
         self.down_weight: Optional[torch.Tensor] = None
 
@@ -47,7 +51,7 @@ class SwiGLU(FeedForward):
         return takes_unscaled(self.gate_up_weight, rows)
 
     def forward(self, x, ctx, residual=None):
-        z = linear(x, self.gate_up_weight, gated=True)
+        z = linear(x, self.gate_up_weight, gated=True, activation=self.activation)
         if residual is not None:
             begun = linear_into_stream(z, self.down_weight, residual)
             if begun is not None:

@@ -101,11 +101,11 @@ def takes_packed(weight: "Weight", rows: int, gated: bool = False) -> bool:
 
 
 def linear(x: Union[torch.Tensor, UnscaledRows], weight, out_dtype: Optional[torch.dtype] = None, gated: bool = False,
-           partials: bool = False) -> torch.Tensor:
+           partials: bool = False, activation: str = "silu") -> torch.Tensor:
     """``x @ W.T`` with float32 accumulation; the result has ``out_dtype`` (default: x's).
 
-    With ``gated`` the weight's rows are [gate; up] and the result is ``silu(gate) * up`` of half the
-    width, in x's dtype. With ``partials`` a float32 result may come as ``[parts, rows, out]``: sums over
+    With ``gated`` the weight's rows are [gate; up] and the result is ``act(gate) * up`` of half the
+    width, in x's dtype (``activation``: ``silu`` or ``gelu_tanh``). With ``partials`` a float32 result may come as ``[parts, rows, out]``: sums over
     ranges of ``in`` that the caller adds in order (the norms and ``qkv_rope_store`` do). For a weight with a
     ``row_order`` the columns of the result are in that order whenever ``takes_packed`` says so.
     """
@@ -123,20 +123,21 @@ def linear(x: Union[torch.Tensor, UnscaledRows], weight, out_dtype: Optional[tor
         a = x if x.dtype == torch.float32 else x.to(torch.float32)
         y = kernels.gemm_f32(a, w, partials=partials and not gated and out_dtype == torch.float32)
         if gated:
-            return kernels.silu_mul(y if x.dtype == torch.float32 else y.to(x.dtype))
+            return kernels.gated_activation(y if x.dtype == torch.float32 else y.to(x.dtype), activation)
         return y if out_dtype == torch.float32 else y.to(out_dtype)
     if x.dtype != weight.dtype:
         raise TypeError(f"cannot multiply {x.dtype} activations with a {weight.dtype} weight")
     rows = x.shape[0]
+    gate = kernels.GATED_ACTIVATIONS[activation]
     if weight.packed is not None and rows <= SKINNY_ROWS:
         if gated:
-            return kernels.gemm_skinny(x, weight.packed, weight.out_features, "gated", scale=scale)
+            return kernels.gemm_skinny(x, weight.packed, weight.out_features, gate, scale=scale)
         return kernels.gemm_skinny(x, weight.packed, weight.out_features, "bf16" if out_dtype == torch.bfloat16 else "f32",
                                    scale=scale)
     if w is None and rows > MEDIUM_ROWS:
         # Only the packed copy is kept: many rows go through this package's tiled product, or, where the
         # reduction is no multiple of 32, through the product for 64 rows, a piece at a time.
-        epilogue = "gated" if gated else ("f32" if out_dtype == torch.float32 else "bf16")
+        epilogue = gate if gated else ("f32" if out_dtype == torch.float32 else "bf16")
         if weight.in_features % 32 == 0:
             splits = kernels.tiled_splits(rows, weight.out_features, weight.in_features) if partials and epilogue == "f32" else 1
             return kernels.gemm_tiled(x, weight.packed, weight.out_features, epilogue, splits=splits)
@@ -146,13 +147,13 @@ def linear(x: Union[torch.Tensor, UnscaledRows], weight, out_dtype: Optional[tor
         return torch.cat(pieces)
     if w is None or takes_packed(weight, rows, gated):
         if gated:
-            return kernels.gemm_medium(x, weight.packed, weight.out_features, "gated")
+            return kernels.gemm_medium(x, weight.packed, weight.out_features, gate)
         if out_dtype == torch.float32:
             plan = kernels.medium_plan(weight.out_features, weight.in_features, may_split=partials)
             return kernels.gemm_medium(x, weight.packed, weight.out_features, "f32", plan=plan)
         return kernels.gemm_medium(x, weight.packed, weight.out_features, "bf16")
     if gated:
-        return kernels.silu_mul(kernels.gemm_bf16(x, w, torch.bfloat16))
+        return kernels.gated_activation(kernels.gemm_bf16(x, w, torch.bfloat16), activation)
     if partials and out_dtype == torch.float32:
         parts = kernels.library_splits(rows, weight.out_features, weight.in_features)
         if parts > 1:

@@ -9,7 +9,9 @@ key channel ``c`` is ``a = sigmoid(z)^(1 / tau)`` with ``z = A2 (A1 x) + b`` thr
 ``A1``, ``A2`` and ``b``: every key channel of head ``h`` decays by ``fixed_decay[h]`` at every token (retention). A
 scale on the keys instead of the queries is the same ``query_scale``: ``o`` is linear in both. Each head's ``o`` is divided by its root mean square
 over ``value_dim`` and multiplied by a weight ``[value_dim]`` that all heads share (``norm_weight`` false: by none); the heads side by side are
-multiplied by ``silu(Wg x)`` and projected by ``Wo``. The state starts at zero, is float32, and lives in the
+multiplied by ``silu(Wg x)`` and projected by ``Wo``. With ``heads_together`` all heads of a token are divided by one root
+mean square instead, the weight is ``[heads * value_dim]`` and the gate ``sigmoid(Wg x)``; with ``silu_inputs`` queries, keys
+and values pass SiLU before they enter the recurrence (lightning attention is both, with a fixed decay). The state starts at zero, is float32, and lives in the
 request's state slot, so a request can be cut into steps anywhere. The five projections that read ``x`` are one
 stacked product with a float32 result; decays, the recurrence, the norm and the gate are float32.
 """
@@ -45,6 +47,8 @@ class GatedLinearAttention(Mixer):
         self.rank = int(p["decay_rank"]) if self.fixed_decay is None else 0
         self.tau = float(p["tau"]) if self.fixed_decay is None else 1.0
         self.has_norm_weight = bool(p.get("norm_weight", True))
+        self.heads_together = bool(p.get("heads_together", False))
+        self.silu_inputs = bool(p.get("silu_inputs", False))
         self.eps = float(p.get("eps", 1e-6))
         self.query_scale = float(p.get("query_scale", self.key_dim ** -0.5))
         keys, values = self.heads * self.key_dim, self.heads * self.value_dim
@@ -68,7 +72,7 @@ class GatedLinearAttention(Mixer):
                  self.name("v"): TensorDecl((values, self.hidden), MATRIX), self.name("g"): TensorDecl((values, self.hidden), MATRIX),
                  self.name("o"): TensorDecl((self.hidden, values), MATRIX)}
         if self.has_norm_weight:
-            decls[self.name("norm")] = TensorDecl((self.value_dim,), VECTOR)
+            decls[self.name("norm")] = TensorDecl((values if self.heads_together else self.value_dim,), VECTOR)
         if self.fixed_decay is None:
             decls.update({self.name("a1"): TensorDecl((self.rank, self.hidden), MATRIX), self.name("a2"): TensorDecl((keys, self.rank), MATRIX),
                           self.name("a2_bias"): TensorDecl((keys,), VECTOR)})
@@ -108,11 +112,14 @@ class GatedLinearAttention(Mixer):
             decay = kernels.gla_decay(proj, self.low_at, self.decay_weight, self.decay_bias, self.tau)
         else:
             decay = self.decay_row
+        long_portions = ctx.max_count >= self.LONG_PORTION
+        if self.silu_inputs and long_portions:      # one pass over many tokens; few tokens pass it as the walk reads them
+            kernels.gla_silu(proj, self.q_at, self.g_at - self.q_at)
         o = kernels.gla_scan(proj, self.q_at, self.k_at, self.v_at, decay, cache.state, ctx.cu_tokens, ctx.slots, ctx.n_seqs,
                              self.heads, self.key_dim, self.value_dim, self.query_scale,
-                             long_portions=ctx.max_count >= self.LONG_PORTION)
+                             long_portions=long_portions, silu_inputs=self.silu_inputs and not long_portions)
         return kernels.gla_gate(o, proj, self.g_at, self.norm_weight, self.eps, self.heads, self.value_dim, out_scale,
-                                self.runtime.dtype, out=out)
+                                self.runtime.dtype, out=out, heads_together=self.heads_together)
 
     def forward(self, x, ctx, cache):
         if self.o_weight is None:

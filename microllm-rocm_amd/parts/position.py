@@ -7,7 +7,9 @@ in float64 so that the angle of any position is exact before cos and sin are
 rounded to float32. cos and sin of a step's positions are computed once and
 shared by the layers whose encoding has the same parameters; the attention
 mixer's fused kernels apply the rotation. With ``scaling_factor`` every rate is
-divided by that number (positions stretched linearly).
+divided by that number (positions stretched linearly). With ``scaling_bands``
+(``factor``, ``low``, ``high``, ``original``) only slow rates are divided by the
+factor (``stretched_by_bands``).
 
 ``rope_neighbours`` pairs channel ``2i`` with ``2i + 1`` instead. Moving channel
 ``2i`` to ``i`` and ``2i + 1`` to ``i + d/2`` makes it the split-half rule, and a
@@ -18,12 +20,24 @@ and runs the split-half kernels.
 """
 from __future__ import annotations
 
+import math
+
 import torch
 
 from ..ops import kernels
 from .base import PositionEncoding, Runtime
 from .registry import register_part
 from .spec import PartSpec
+
+
+def stretched_by_bands(rates: torch.Tensor, factor: float, low: float, high: float, original: float) -> torch.Tensor:
+    """Rates (angle a position, float64) stretched by how often they turn over ``original`` positions, ``n = original *
+    rate / (2 pi)``: below ``low`` turns a rate is divided by ``factor``, above ``high`` it stays, between the two the
+    stretched and the plain rate are blended, linearly in ``n``."""
+    turns = original * rates / (2.0 * math.pi)
+    blend = ((turns - low) / (high - low)).clamp(0.0, 1.0) if high > low else (turns > high).to(rates.dtype)
+    mixed = (1.0 - blend) * rates / factor + blend * rates
+    return torch.where(turns < low, rates / factor, torch.where(turns > high, rates, mixed))
 
 
 class RopeSplitHalf(PositionEncoding):
@@ -41,11 +55,16 @@ class RopeSplitHalf(PositionEncoding):
         if self.scaling_factor <= 0.0:
             raise ValueError("scaling_factor must be positive")
         exponents = torch.arange(0, self.rotary_dim, 2, dtype=torch.float64) / self.rotary_dim
-        self.inv_freq = ((self.theta ** -exponents) / self.scaling_factor).to(runtime.device)
+        rates = (self.theta ** -exponents) / self.scaling_factor
+        bands = spec.params.get("scaling_bands")
+        self.scaling_bands = tuple(float(bands[key]) for key in ("factor", "low", "high", "original")) if bands is not None else None
+        if self.scaling_bands is not None:
+            rates = stretched_by_bands(rates, *self.scaling_bands)
+        self.inv_freq = rates.to(runtime.device)
 
     def table(self, ctx) -> torch.Tensor:
         """``[tokens, rotary_dim / 2, 2]`` float32: cos and sin for the step's tokens."""
-        key = ("rope_split_half", self.theta, self.rotary_dim, self.scaling_factor)
+        key = ("rope_split_half", self.theta, self.rotary_dim, self.scaling_factor, self.scaling_bands)
         if key not in ctx.memo:
             ctx.memo[key] = kernels.rope_table(ctx.positions, self.inv_freq)
         return ctx.memo[key]
