@@ -138,6 +138,23 @@ def kalevik_config(size: dict):
     return KalevikConfig(vocab=DESIGN_VOCAB, width=width, norm_eps=1e-6, layers=tuple(layers), embedding_scale=2.0)
 
 
+def mapedra_config(size: dict):
+    """A Mapedra configuration of the given layer sizes: layers in turn lightning attention (half as many heads, keys of half
+    the head size, values of the whole, as Siditar's and Kalevik's linear attention), then three of softmax attention (the
+    model's heads and key/value heads of the head size, half of every head turned, scores capped at 30); every layer with
+    a dense feed-forward, norms in four parts, a side vector of a sixteenth of the width."""
+    from microllm_rocm_amd.config.mapedra import (AttentionConfig, BandScalingConfig, DenseMlpConfig, LightningConfig, MapedraConfig,
+                                                  MapedraLayerConfig)
+    width, heads, dim = size["width"], size["heads"], size["head_dim"]
+    attention = AttentionConfig(heads=heads, kv_heads=size["kv_heads"], dim=dim, vdim=dim, scale=dim ** -0.5, rot_base=1e6,
+                                rot_dims=dim // 2, softcap=30.0, rot_scaling=BandScalingConfig(8.0, 1.0, 4.0, 8192.0))
+    lightning = LightningConfig(heads=heads // 2, dim=dim // 2, vdim=dim, decay=tuple(1.0 - 0.1 / (1 + head % 6) for head in range(heads // 2)))
+    layers = [MapedraLayerConfig("lightning", lightning, DenseMlpConfig(size["ff"])) if index % 4 == 0 else
+              MapedraLayerConfig("attention", attention, DenseMlpConfig(size["ff"])) for index in range(size["layers"])]
+    return MapedraConfig(vocab=DESIGN_VOCAB, width=width, norm_eps=1e-5, norm_groups=4, side_dim=width // 16, layers=tuple(layers),
+                         embedding_scale=width ** 0.5)
+
+
 def design_configs(size: dict, design: str = "siditar"):
     """The design's configuration at the given layer sizes and the Qwen2 configuration of equal width, heads, head size,
     feed-forward width, depth and vocabulary."""
@@ -152,6 +169,9 @@ def design_configs(size: dict, design: str = "siditar"):
         return {"zabozen": zabozen_config(size), "gupitar": gupitar_config(size), "qwen2": qwen2}
     if design == "kalevik":     # beside the designs whose layers are most like its own (latents and experts; a parallel mixer)
         return {"kalevik": kalevik_config(size), "gupitar": gupitar_config(size), "siditar": design_configs(size, "siditar")["siditar"],
+                "qwen2": qwen2}
+    if design == "mapedra":     # beside the designs whose parts are most like its own (norms after sublayers; a linear attention)
+        return {"mapedra": mapedra_config(size), "zabozen": zabozen_config(size), "siditar": design_configs(size, "siditar")["siditar"],
                 "qwen2": qwen2}
     from microllm_rocm_amd.config.siditar import (BiasAttentionConfig, DenseMlpConfig, LinearAttentionConfig,
                                                   ParallelMixerConfig, SiditarConfig, SiditarLayerConfig)
@@ -232,11 +252,11 @@ def main() -> int:
     parser.add_argument("--no-extras", action="store_true",
                         help="leave out what the default run adds to its line after the main figures: decoding on the 32-bit path "
                              "at batch 8 and the continuous-batching workload at Qwen2-0.5B sizes")
-    parser.add_argument("--design", default=None, choices=["siditar", "gupitar", "zabozen", "kalevik"],
+    parser.add_argument("--design", default=None, choices=["siditar", "gupitar", "zabozen", "kalevik", "mapedra"],
                         help="instead of the default workload: prefill and decode throughput of this design beside Qwen2 at equal "
                              "layer sizes (--design-sizes), random weights; --batch, --context, --prefill-tokens, --steps apply")
     parser.add_argument("--design-sizes", default="1k,2k,4k", help="of " + ", ".join(sorted(DESIGN_SIZES)))
-    parser.add_argument("--design-only", default=None, choices=["siditar", "gupitar", "zabozen", "kalevik", "qwen2"], help="one of the designs alone (profiles)")
+    parser.add_argument("--design-only", default=None, choices=["siditar", "gupitar", "zabozen", "kalevik", "mapedra", "qwen2"], help="one of the designs alone (profiles)")
     args = parser.parse_args()
     if args.gpus != 1:
         print(f"bench.py measures one GPU; --gpus {args.gpus} is not supported (this engine runs on a single MI355X)")

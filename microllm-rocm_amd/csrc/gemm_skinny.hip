@@ -31,7 +31,8 @@ union Piece {
 // `q_out`, keys and values into their pages (at most 16 rows; see MllQkvStore). 4 = the product is added to the
 // float32 residual stream and the sum, times the next norm's weight, is written as the next product's input,
 // with each workgroup's share of the rows' sums of squares (at most 16 rows; see MllResidualNorm).
-// 5 = 2 with the tanh form of gelu for silu.
+// 5 = 2 with the tanh form of gelu for silu. 6 = bfloat16 [M, N] = gelu_tanh(product) * the token's columns of a side
+// table (at most 16 rows; see MllSideTable).
 // Whatever the epilogue, a row of the product is first multiplied by the factor that MllRowScale describes,
 // if one is given (at most 16 rows).
 // W is read past the caches (non-temporal loads): a step reads every weight once, and all of them together are far
@@ -102,6 +103,23 @@ __global__ __launch_bounds__(1024) void gemm_skinny_kernel(
                 const bool live = col < m && column < n;
                 h_before[nt][i] = live ? extras.residual.h[static_cast<int64_t>(col) * n + column] : 0.0f;
                 norm_weight[nt][i] = live ? extras.residual.norm_weight[column] : 0.0f;
+            }
+    }
+
+    float side[NT][4];
+    if (EPILOGUE == 6 && wave == 0) {
+        const MllSideTable& table = extras.side;
+        const int id = col < m ? table.ids[col] : 0;
+        const bool known = id >= 0 && id < table.vocab;
+#pragma unroll
+        for (int nt = 0; nt < NT; ++nt)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int column = (tile0 + nt) * 16 + quad * 4 + i;
+                const int64_t at = static_cast<int64_t>(id) * table.stride + table.column_at + column;
+                side[nt][i] = known ? 0.0f : NAN;
+                if (known && column < n)
+                    side[nt][i] = table.dtype == kF32 ? static_cast<const float*>(table.rows)[at] : to_float(static_cast<const bf16*>(table.rows)[at]);
             }
     }
 
@@ -273,6 +291,13 @@ __global__ __launch_bounds__(1024) void gemm_skinny_kernel(
                     const int column = n_tile * 16 + quad * 4 + i;
                     if (column < n) target[column] = from_float<bf16>(acc[nt][mt][i]);
                 }
+            } else if (EPILOGUE == 6) {
+                bf16* target = static_cast<bf16*>(out) + static_cast<int64_t>(row) * n;
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const int column = n_tile * 16 + quad * 4 + i;
+                    if (column < n) target[column] = from_float<bf16>(activate(acc[nt][mt][i], kActGeluTanh) * side[nt][i]);
+                }
             } else if (EPILOGUE == 2 || EPILOGUE == 5) {
                 bf16* target = static_cast<bf16*>(out) + static_cast<int64_t>(row) * (n / 2);
 #pragma unroll
@@ -378,7 +403,7 @@ static int launch_skinny(const void* a, const void* w_packed, void* out, int m, 
     const bf16* w_ = static_cast<const bf16*>(w_packed);
     const int m_tiles = (m + 15) / 16;
     const bool two = tiles_per_group(m, n_tiles) == 2;
-    if constexpr (EPILOGUE == 3 || EPILOGUE == 4) {
+    if constexpr (EPILOGUE == 3 || EPILOGUE == 4 || EPILOGUE == 6) {
         if (m_tiles != 1) return fail("gemm_skinny: this epilogue takes at most 16 rows");
         if (two) launch_one<1, 2, EPILOGUE>(a_, w_, out, m, n, k, n_tiles, k_steps, extras, stream);
         else launch_one<1, 1, EPILOGUE>(a_, w_, out, m, n, k, n_tiles, k_steps, extras, stream);
@@ -430,6 +455,20 @@ extern "C" int mll_gemm_skinny(const void* a, const void* w_packed, void* out, i
         case 5: return launch_skinny<5>(a, w_packed, out, m, n, k, extras, stream);
         default: return fail("gemm_skinny: unknown epilogue");
     }
+}
+
+extern "C" int mll_gemm_skinny_side(const void* a, const void* w_packed, void* out, int m, int n, int k, const MllSideTable* side,
+                                    hipStream_t stream) {
+    MLL_REQUIRE(side != nullptr && side->rows && side->ids, "gemm_skinny_side: a side table and the rows' ids are needed");
+    MLL_REQUIRE(m >= 0 && m <= 16, "gemm_skinny_side: takes at most 16 rows");
+    MLL_REQUIRE(n > 0 && k > 0 && k % 8 == 0, "gemm_skinny_side: k must be a positive multiple of 8");
+    MLL_REQUIRE(side->dtype == kF32 || side->dtype == kBF16, "gemm_skinny_side: unknown dtype of the side table");
+    MLL_REQUIRE(side->vocab > 0 && side->column_at >= 0 && side->column_at + n <= side->stride,
+                "gemm_skinny_side: the columns lie outside the table's rows");
+    if (m == 0) return 0;
+    MllSkinnyExtras extras{};
+    extras.side = *side;
+    return launch_skinny<6>(a, w_packed, out, m, n, k, extras, stream);
 }
 
 extern "C" int mll_gemm_skinny_qkv(const void* a, const void* w_packed, int m, int k, const MllQkvStore* store,

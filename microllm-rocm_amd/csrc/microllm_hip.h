@@ -178,8 +178,23 @@ struct MllResidualNorm {
 int mll_gemm_skinny_residual(const void* a, const void* w_packed, int m, int n, int k, const MllResidualNorm* residual,
                              const MllRowScale* scale, hipStream_t stream);
 
+// What mll_token_side_gate takes beside its input: columns column_at .. of the rows of a table (in `dtype`, rows `stride`
+// elements apart) named by the tokens' ids.
+struct MllSideTable {
+    const void* rows;
+    const int32_t* ids;      // [m]
+    int64_t stride;
+    int dtype;
+    int column_at;
+    int vocab;
+};
+// The product of at most 16 rows finished as mll_token_side_gate does: bfloat16 out [m, n].
+int mll_gemm_skinny_side(const void* a, const void* w_packed, void* out, int m, int n, int k, const MllSideTable* side,
+                         hipStream_t stream);
+
 // What the kernel takes beside the product's operands (internal to the library's launches).
 struct MllSkinnyExtras {
+    MllSideTable side;
     MllQkvStore store;
     MllRowScale scale;
     MllResidualNorm residual;

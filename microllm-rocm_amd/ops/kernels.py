@@ -980,6 +980,29 @@ def gemm_skinny(x: torch.Tensor, packed: torch.Tensor, n: int, epilogue: str = "
     return out
 
 
+class _SideTable(ctypes.Structure):
+    _fields_ = [("rows", ctypes.c_void_p), ("ids", ctypes.c_void_p), ("stride", ctypes.c_int64), ("dtype", ctypes.c_int),
+                ("column_at", ctypes.c_int), ("vocab", ctypes.c_int)]
+
+
+def gemm_skinny_side(x: torch.Tensor, packed: torch.Tensor, n: int, table: torch.Tensor, column_at: int, ids: torch.Tensor) -> torch.Tensor:
+    """``token_side_gate`` of ``x @ W.T`` in the product's epilogue: at most 16 bfloat16 rows and a packed weight of ``n`` rows."""
+    lib = library.load()
+    _device_tensor(x, "gemm input", torch.bfloat16)
+    _device_tensor(packed, "packed weight", torch.bfloat16)
+    _device_tensor(table, "side table")
+    _device_tensor(ids, "token ids", torch.int32)
+    _need(x.dim() == 2 and packed.dim() == 5 and tuple(packed.shape[2:]) == (4, 16, 8), "gemm_skinny_side takes [m, k] and a packed weight")
+    m, k = x.shape
+    _need(m <= 16 and k % 8 == 0 and ids.shape[0] >= m, "at most 16 rows of a multiple of 8, an id for each")
+    _need(packed.shape[0] == -(-n // 16) and packed.shape[1] == -(-k // 32), "the packed weight does not fit n and k")
+    _need(table.dim() == 2 and 0 <= column_at and column_at + n <= table.shape[1], "the layer's columns lie inside the side table")
+    out = torch.empty((m, n), dtype=torch.bfloat16, device=x.device)
+    side = _SideTable(table.data_ptr(), ids.data_ptr(), table.shape[1], _code(table.dtype), int(column_at), table.shape[0])
+    _check(lib.mll_gemm_skinny_side(_ptr(x), _ptr(packed), _ptr(out), m, n, k, ctypes.byref(side), _stream()), lib)
+    return out
+
+
 MEDIUM_WORKGROUPS = 224     # workgroups of 8 waves that gemm_medium wants at least (MI355X has 256 compute units)
 MEDIUM_WHOLE_WORKGROUPS = 128     # where the reduction cannot be split, two tiles a wave from this many workgroups on
 

@@ -3,7 +3,8 @@
 One table beside the embedding holds, for every token id, a row of ``dim`` numbers a layer, side by side. Layer ``i``
 takes ``e``, its ``dim`` columns of the token's row, and adds ``P (gelu(G x) * e)`` to the stream, ``G`` being ``[dim,
 hidden]``, ``P`` ``[hidden, dim]`` and gelu its tanh form (what stands before and after it is the arrangement's). The
-table is one tensor that all layers name; each reads its own columns of the step's rows where it multiplies. The gate's
+table is one tensor that all layers name; each reads its own columns of the step's rows where it multiplies (for few
+rows in the gate product's epilogue). The gate's
 sums, its activation and the product with ``e`` are float32 and rounded once.
 """
 from __future__ import annotations
@@ -14,7 +15,7 @@ import torch
 
 from ..ops import kernels
 from .base import FeedForward, MATRIX, Runtime, TensorDecl
-from .linear import Weight, linear
+from .linear import SKINNY_ROWS, Weight, linear
 from .registry import register_part
 from .spec import PartSpec
 
@@ -53,6 +54,9 @@ class TokenSideInput(FeedForward):
         return weights + rows * self.dim * self.table.element_size()
 
     def forward(self, x, ctx):
+        if x.shape[0] <= SKINNY_ROWS and self.gate_weight.packed is not None and x.dtype == torch.bfloat16:
+            g = kernels.gemm_skinny_side(x, self.gate_weight.packed, self.dim, self.table, self.column_at, ctx.tokens)
+            return linear(g, self.out_weight, out_dtype=torch.float32, partials=True)
         z = linear(x, self.gate_weight, out_dtype=torch.float32, partials=True)
         g = kernels.token_side_gate(z, self.table, self.column_at, ctx.tokens, self.runtime.dtype)
         return linear(g, self.out_weight, out_dtype=torch.float32, partials=True)

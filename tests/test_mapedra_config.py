@@ -1,0 +1,177 @@
+"""Host logic of the Mapedra decoder: its configuration (keys, what may be absent, refusals), the model it is built into and
+the cache needs of its mixers, the rates stretched by bands, the reordered rows of neighbouring channels, and the plain
+implementation's own pieces against values worked out by hand."""
+import copy
+import json
+import math
+import os
+
+import pytest
+import torch
+
+import plain_mapedra as plain
+from mapedra_tiny import CONFIGS, make_mapedra_folder
+from microllm_rocm_amd.cache import PagedKVNeed, StateNeed
+from microllm_rocm_amd.config import ConfigError, load_config
+from microllm_rocm_amd.config.mapedra import MapedraConfig
+from microllm_rocm_amd.parts import Model, PartSpec, Runtime, build_part
+from microllm_rocm_amd.parts.base import PagedKeyValueNeed
+from microllm_rocm_amd.parts.position import stretched_by_bands
+
+F = torch.float64
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("which", ["A", "B", "C"])
+def test_folder_round_trip(tmp_path, which, dtype):
+    folder = make_mapedra_folder(tmp_path, which)
+    written = json.load(open(os.path.join(folder, "config.json")))
+    assert written["architecture"] == "Mapedra"
+    architecture, config = load_config(folder)
+    assert architecture.name == "Mapedra" and config == CONFIGS[which]
+    spec = architecture.build_spec(config)
+    assert [entry.layer for entry in spec.order] == list(range(len(written["layers"])))
+    model = Model(spec, Runtime(dtype, torch.device("cpu")))
+    tensors = plain.read_tensors(folder)
+    assert set(model.tensors()) == set(tensors)
+    assert all(tuple(tensors[name].shape) == tuple(decl.shape) for name, decl in model.tensors().items())
+    assert tuple(tensors["side.embed"].shape) == (written["vocab"], len(written["layers"]) * written["token_side"]["dim"])
+    for need, layer in zip(model.cache_needs(), written["layers"]):
+        mixer = layer["mixer"]
+        if layer["type"] == "lightning":
+            assert need == StateNeed((mixer["heads"], mixer["dim"], mixer["vdim"]), torch.float32)
+        elif dtype == torch.bfloat16 and mixer["dim"] == mixer["vdim"] and mixer["dim"] % 16 == 0:
+            assert need == PagedKVNeed(mixer["kv_heads"], mixer["dim"], None)
+        else:
+            assert need == PagedKeyValueNeed(mixer["kv_heads"], mixer["dim"], mixer["vdim"], None)
+    columns = [block.extra["side"].column_at for block in model.blocks]
+    assert columns == [index * written["token_side"]["dim"] for index in range(len(written["layers"]))]
+
+
+def test_what_a_file_may_leave_out():
+    """No factor on the embedding, norms in one part, no stretched rates, no cap, no feed-forward."""
+    source = CONFIGS["B"].to_dict()
+    del source["embedding"], source["norm"]["groups"]
+    assert "softcap" not in source["layers"][1]["mixer"] and "scaling" not in source["layers"][1]["mixer"]["rot"]
+    config = MapedraConfig.from_dict(source)
+    assert config == CONFIGS["B"]
+    assert config.layers[1].mixer.softcap is None and config.layers[1].mixer.rot_scaling is None and config.layers[0].mlp is None
+
+
+@pytest.mark.parametrize("change,text", [
+    (lambda c: c["layers"][0].__setitem__("type", "window"), "unknown layer type"),
+    (lambda c: c["layers"][1]["mlp"].__setitem__("kind", "moe"), "unknown feed-forward kind"),
+    (lambda c: c["layers"][0]["mixer"]["rot"].__setitem__("dims", 18), "at most mixer.dim"),
+    (lambda c: c["layers"][0]["mixer"]["rot"].__setitem__("dims", 7), "must be even"),
+    (lambda c: c["layers"][0]["mixer"]["rot"]["scaling"].__setitem__("high", 0.5), "must not lie below"),
+    (lambda c: c["layers"][0]["mixer"]["rot"]["scaling"].__delitem__("low"), "missing low"),
+    (lambda c: c["layers"][0]["mixer"].__setitem__("kv_heads", 3), "must divide"),
+    (lambda c: c["layers"][0]["mixer"].__setitem__("softcap", -1.0), "must be positive"),
+    (lambda c: c["layers"][1]["mixer"].__setitem__("decay", [0.5, 0.5]), "one number a head"),
+    (lambda c: c["layers"][1]["mixer"].__setitem__("decay", [0.5, 1.5, 0.5]), "between 0 and 1"),
+    (lambda c: c["norm"].__setitem__("groups", 5), "equal parts"),
+    (lambda c: c["layers"][0]["mixer"].__delitem__("scale"), "missing scale"),
+    (lambda c: c.__delitem__("token_side"), "missing token_side"),
+    (lambda c: c.__setitem__("vocab", 3.5), "must be an integer"),
+])
+def test_refusals(change, text):
+    source = copy.deepcopy(CONFIGS["A"].to_dict())
+    change(source)
+    with pytest.raises(ConfigError, match=text):
+        MapedraConfig.from_dict(source)
+
+
+@pytest.mark.parametrize("base,n,bands", [(10000.0, 8, (3.0, 1.0, 8.0, 64.0)), (5e5, 64, (4.0, 1.0, 4.0, 512.0)), (77.0, 10, (1.0, 1.0, 4.0, 300.0)),
+                                          (100.0, 4, (2.0, 0.5, 0.5, 40.0)), (1e4, 2, (8.0, 2.0, 3.0, 9.0))])
+def test_rates_stretched_by_bands(base, n, bands):
+    scaling = dict(zip(("factor", "low", "high", "original"), bands))
+    plain_rates = torch.tensor(plain.rates(base, n), dtype=F)
+    want = torch.tensor(plain.rates(base, n, scaling), dtype=F)
+    assert torch.allclose(stretched_by_bands(plain_rates, *bands), want, rtol=1e-14, atol=0)
+    part = build_part("position", PartSpec("rope_neighbours", {"theta": base, "head_dim": n, "scaling_bands": scaling}),
+                      Runtime(torch.float32, torch.device("cpu")))
+    assert torch.allclose(part.inv_freq, want, rtol=1e-14, atol=0)
+
+
+def test_the_three_bands_by_hand():
+    """Over 64 positions with low 1 and high 8: a rate of 2 pi / 4 turns 16 times and stays, one of 2 pi / 128 turns half a
+    time and is divided by the factor, one of 2 pi / 16 turns 4 times: 3/7 of it stays and 4/7 is divided."""
+    rates = torch.tensor([2 * math.pi / 4, 2 * math.pi / 128, 2 * math.pi / 16], dtype=F)
+    got = stretched_by_bands(rates, 3.0, 1.0, 8.0, 64.0) / rates
+    assert torch.allclose(got, torch.tensor([1.0, 1 / 3, 3 / 7 + 4 / 21], dtype=F))
+    table = plain.rates(10000.0, 8, {"factor": 3.0, "low": 1.0, "high": 8.0, "original": 64.0})
+    ratio = [a / b for a, b in zip(table, plain.rates(10000.0, 8))]
+    assert ratio[0] == 1.0 and 1 / 3 < ratio[1] < 1.0 and ratio[3] == pytest.approx(1 / 3)       # all three occur in the tests' model
+
+
+def test_rows_that_make_neighbouring_channels_are_reordered():
+    """After the reordering the split-half rule turns what the rule of neighbours turned before it, the norm's weight
+    goes with its channel, channels that do not turn stay in place, and scores are unchanged."""
+    rng = torch.Generator().manual_seed(3)
+    mixer = CONFIGS["A"].layers[0].mixer
+    heads, kv_heads, dim, width = mixer.heads, mixer.kv_heads, mixer.dim, 64
+    spec = CONFIGS["A"]
+    architecture_spec = load_config_spec(spec)
+    part = build_part("mixer", architecture_spec.layers[0].mixer, Runtime(torch.float32, torch.device("cpu")))
+    tensors = {name: torch.randn(decl.shape, generator=rng) for name, decl in part.tensors().items()}
+    part.bind(tensors)
+    x = torch.randn(9, width, generator=rng).to(F)
+    eps, rot = 1e-5, mixer.rot_dims
+    bands = mixer.rot_scaling.to_dict()
+    positions = torch.arange(9)
+    half = rot // 2
+
+    def split_half(a):
+        angle = positions.to(F)[:, None] * part.position.inv_freq[None, :]
+        cos, sin = torch.cos(angle)[:, None], torch.sin(angle)[:, None]
+        u, v = a[..., :half], a[..., half:rot]
+        return torch.cat([u * cos - v * sin, v * cos + u * sin, a[..., rot:]], dim=-1)
+
+    qk = (x @ part.qkv_weight.tensor.to(F).T)[:, :(heads + kv_heads) * dim].view(9, heads + kv_heads, dim)
+    weights = torch.cat([part.q_norm.to(F).expand(heads, dim), part.k_norm.to(F).expand(kv_heads, dim)])
+    mine = split_half(plain.rms(qk, eps) * weights)
+    q = plain.turn_neighbours(plain.rms((x @ tensors["l0.mix.q"].to(F).T).view(9, heads, dim), eps) * tensors["l0.mix.q.norm"].to(F), positions, 10000.0, rot, bands)
+    k = plain.turn_neighbours(plain.rms((x @ tensors["l0.mix.k"].to(F).T).view(9, kv_heads, dim), eps) * tensors["l0.mix.k.norm"].to(F), positions, 10000.0, rot, bands)
+    for head in range(heads):
+        group = head // (heads // kv_heads)
+        assert torch.allclose(mine[:, head] @ mine[:, heads + group].T, q[:, head] @ k[:, group].T, atol=1e-10)
+    assert torch.allclose(mine[:, :heads, rot:], q[..., rot:], atol=1e-12)
+    assert torch.allclose(mine[:, :heads, :half], q[..., 0:rot:2], atol=1e-12) and torch.allclose(mine[:, :heads, half:rot], q[..., 1:rot:2], atol=1e-12)
+
+
+def load_config_spec(config):
+    from microllm_rocm_amd.config.registry import architecture_named
+    return architecture_named("Mapedra").build_spec(config)
+
+
+def test_norm_in_groups_by_hand():
+    a = torch.tensor([[3.0, 4.0, 0.0, 2.0]], dtype=F)
+    got = plain.grouped_rms(a, 2, 0.0)
+    assert torch.allclose(got, torch.tensor([[3.0 / 12.5 ** 0.5, 4.0 / 12.5 ** 0.5, 0.0, 2.0 / 2.0 ** 0.5]], dtype=F))
+    assert torch.allclose(plain.grouped_rms(a, 1, 1e-5), plain.rms(a, 1e-5))
+
+
+def test_capped_scores_by_hand():
+    """One head of one channel, cap 2: scores 0 and 2 tanh(1) for the second query."""
+    q = torch.tensor([[[0.0]], [[1.0]]], dtype=F)
+    k = torch.tensor([[[0.0]], [[2.0]]], dtype=F)
+    v = torch.tensor([[[1.0]], [[5.0]]], dtype=F)
+    got = plain.attend_capped(q, k, v, 1.0, 2.0)
+    w = math.exp(2.0 * math.tanh(1.0))
+    assert got[0, 0, 0] == 1.0 and float(got[1, 0, 0]) == pytest.approx((1.0 + 5.0 * w) / (1.0 + w))
+    w = math.exp(2.0)
+    assert float(plain.attend_capped(q, k, v, 1.0, None)[1, 0, 0]) == pytest.approx((1.0 + 5.0 * w) / (1.0 + w))
+
+
+def test_the_side_vector_takes_its_layers_columns():
+    tensors = {"side.embed": torch.arange(12.0).view(2, 6), "l1.side.gate": torch.tensor([[1.0], [0.0], [0.0]]), "l1.side.proj": torch.eye(3)[:1]}
+    got = plain.token_side_input(torch.tensor([[2.0]], dtype=F), tensors, 1, 3, torch.tensor([1]))
+    assert float(got[0, 0]) == pytest.approx(float(plain.gelu_tanh(torch.tensor(2.0, dtype=F))) * 9.0)      # row 1, columns 3 .. 5
+
+
+def test_lightning_by_hand():
+    q = torch.ones(3, 1, 1, dtype=F)
+    k = torch.tensor([[[1.0]], [[2.0]], [[0.0]]], dtype=F)
+    v = torch.tensor([[[1.0, 1.0]], [[0.0, 1.0]], [[5.0, 5.0]]], dtype=F)
+    got = plain.retain(q, k, v, [0.5])
+    assert torch.allclose(got[:, 0], torch.tensor([[1.0, 1.0], [0.5, 2.5], [0.25, 1.25]], dtype=F))
