@@ -39,7 +39,7 @@ def _lightning_spec(width: int, prefix: str, mixer: LightningConfig, eps: float)
     names = {role: f"{prefix}.{role}" for role in ("q", "k", "v", "g", "o", "norm")}
     return PartSpec("gated_linear_attention", {
         "hidden_size": width, "heads": mixer.heads, "key_dim": mixer.dim, "value_dim": mixer.vdim, "fixed_decay": list(mixer.decay),
-        "silu_inputs": True, "heads_together": True, "eps": eps, "query_scale": 1.0}, names)
+        "silu_inputs": True, "heads_together": True, "chunked": True, "eps": eps, "query_scale": 1.0}, names)
 
 
 def build_spec(config: MapedraConfig) -> ModelSpec:

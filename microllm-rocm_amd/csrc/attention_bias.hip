@@ -132,20 +132,24 @@ bias_attention_kernel(const T* __restrict__ q, const T* __restrict__ k_pages, co
     }
 }
 
-// One wave a (token, head of q, k or v): the norm of queries and keys over their head, the queries' factor by
+constexpr int kNormStoreWaves = 4;
+
+// One wave a (token, head of q, k or v), four to a workgroup: the norm of queries and keys over their head, the queries' factor by
 // position, and the write of keys and values into their pages.
 template <typename T>
-__global__ void __launch_bounds__(kWave)
+__global__ void __launch_bounds__(kNormStoreWaves * kWave)
 qk_norm_store_kernel(const float* __restrict__ qkv, int n_parts, int64_t part_stride, const float* __restrict__ q_weight,
                      const float* __restrict__ k_weight, float eps, const int32_t* __restrict__ positions,
                      const int32_t* __restrict__ slot_mapping, float temp_coef, int temp_every, T* __restrict__ q_out,
                      T* __restrict__ k_pages, T* __restrict__ v_pages, int heads, int kv_heads, int key_dim, int value_dim,
                      int tiled_page_size, const float* __restrict__ bias, int normed, int queries_only, int64_t row_stride,
-                     const float* __restrict__ cos_sin, int rot_dims, int values_normed) {
+                     const float* __restrict__ cos_sin, int rot_dims, int values_normed, int total) {
     const int vectors = queries_only ? heads : heads + 2 * kv_heads;
-    const int token = blockIdx.x / vectors;
-    const int which = blockIdx.x % vectors;
-    const int lane = threadIdx.x;
+    const int vector = blockIdx.x * kNormStoreWaves + threadIdx.x / kWave;
+    if (vector >= total) return;
+    const int token = vector / vectors;
+    const int which = vector % vectors;
+    const int lane = threadIdx.x % kWave;
     const float* row = qkv + static_cast<int64_t>(token) * row_stride;
     const bool is_q = which < heads, is_k = !is_q && which < heads + kv_heads;
     const int head = is_q ? which : (is_k ? which - heads : which - heads - kv_heads);
@@ -230,18 +234,19 @@ int mll_qk_norm_store(const float* qkv, int n_parts, int64_t part_stride, const 
     MLL_REQUIRE(queries_only || (slot_mapping != nullptr && k_pages != nullptr && v_pages != nullptr), "qk_norm_store: keys and values need pages and slots");
     MLL_REQUIRE(temp_coef == 0.0f || temp_every > 0, "qk_norm_store: the factor by position needs a positive step");
     if (n_tokens == 0) return 0;
-    const int64_t blocks = static_cast<int64_t>(n_tokens) * (queries_only ? heads : heads + 2 * kv_heads);
-    MLL_REQUIRE(blocks < (1ll << 31), "qk_norm_store: too many rows for one launch");
+    const int64_t total = static_cast<int64_t>(n_tokens) * (queries_only ? heads : heads + 2 * kv_heads);
+    MLL_REQUIRE(total < (1ll << 31) - kNormStoreWaves, "qk_norm_store: too many rows for one launch");
+    const int64_t blocks = (total + kNormStoreWaves - 1) / kNormStoreWaves;
     if (dtype == kF32) {
-        qk_norm_store_kernel<float><<<static_cast<unsigned>(blocks), kWave, 0, stream>>>(
+        qk_norm_store_kernel<float><<<static_cast<unsigned>(blocks), kNormStoreWaves * kWave, 0, stream>>>(
             qkv, n_parts, part_stride, q_weight, k_weight, eps, positions, slot_mapping, temp_coef, temp_every,
             static_cast<float*>(q_out), static_cast<float*>(k_pages), static_cast<float*>(v_pages), heads, kv_heads, key_dim, value_dim,
-            tiled_page_size, bias, normed, queries_only, row_stride, cos_sin, rot_dims, values_normed);
+            tiled_page_size, bias, normed, queries_only, row_stride, cos_sin, rot_dims, values_normed, static_cast<int>(total));
     } else if (dtype == kBF16) {
-        qk_norm_store_kernel<bf16><<<static_cast<unsigned>(blocks), kWave, 0, stream>>>(
+        qk_norm_store_kernel<bf16><<<static_cast<unsigned>(blocks), kNormStoreWaves * kWave, 0, stream>>>(
             qkv, n_parts, part_stride, q_weight, k_weight, eps, positions, slot_mapping, temp_coef, temp_every,
             static_cast<bf16*>(q_out), static_cast<bf16*>(k_pages), static_cast<bf16*>(v_pages), heads, kv_heads, key_dim, value_dim,
-            tiled_page_size, bias, normed, queries_only, row_stride, cos_sin, rot_dims, values_normed);
+            tiled_page_size, bias, normed, queries_only, row_stride, cos_sin, rot_dims, values_normed, static_cast<int>(total));
     } else {
         return fail("qk_norm_store: unknown dtype");
     }

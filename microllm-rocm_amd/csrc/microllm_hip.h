@@ -373,6 +373,14 @@ int mll_gla_gate(const float* o, const float* proj, int64_t proj_stride, int gat
                  void* out, int64_t out_stride, int dtype, int n_tokens, int heads, int value_dim, float out_scale,
                  hipStream_t stream);
 
+// mll_gla_scan for steps with long portions and one decay a head (`decay`: heads numbers): the recurrence in chunks of 64
+// tokens on the matrix units (csrc/linear_attention_chunks.hip), the same result but for rounding. key_dim at most 128;
+// `scratch`: mll_gla_chunks_scratch(...) floats.
+int64_t mll_gla_chunks_scratch(int n_tokens, int n_seqs, int heads, int key_dim, int value_dim);
+int mll_gla_chunks(const float* proj, int64_t proj_stride, int q_offset, int k_offset, int v_offset, const float* decay, float* state,
+                   const int32_t* cu_tokens, const int32_t* slots, float* out, float* scratch, int n_tokens, int n_seqs, int heads,
+                   int key_dim, int value_dim, float q_scale, int silu_inputs, hipStream_t stream);
+
 // Columns first .. first + count - 1 of every row of proj, in place: silu.
 int mll_gla_silu(float* proj, int64_t proj_stride, int first, int count, int n_tokens, hipStream_t stream);
 

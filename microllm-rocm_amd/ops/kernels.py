@@ -1468,6 +1468,33 @@ def gla_scan(proj: torch.Tensor, q_offset: int, k_offset: int, v_offset: int, de
     return out
 
 
+GLA_CHUNK_KEYS = 128       # the widest key heads the recurrence in chunks takes
+
+
+def gla_chunks(proj: torch.Tensor, q_offset: int, k_offset: int, v_offset: int, decay: torch.Tensor, state: torch.Tensor,
+               cu_tokens: torch.Tensor, slots: torch.Tensor, n_seqs: int, heads: int, key_dim: int, value_dim: int,
+               q_scale: float, silu_inputs: bool = False) -> torch.Tensor:
+    """``gla_scan`` with one decay a head (``decay`` float32 ``[heads]``) for long portions: chunks of 64 tokens side by side on
+    the matrix units, the same result but for rounding."""
+    lib = library.load()
+    _device_tensor(proj, "projections", torch.float32)
+    _device_tensor(decay, "decays", torch.float32)
+    _device_tensor(state, "state", torch.float32)
+    _device_tensor(cu_tokens, "token offsets", torch.int32)
+    _device_tensor(slots, "state slots", torch.int32)
+    n_tokens = proj.shape[0]
+    _need(proj.dim() == 2 and tuple(decay.shape) == (heads,), "projections [tokens, columns] and one decay a head")
+    _need(key_dim <= GLA_CHUNK_KEYS, "the recurrence in chunks takes key heads of at most 128 channels")
+    _need(state.dim() == 4 and tuple(state.shape[1:]) == (heads, key_dim, value_dim), "state is [slots, heads, key_dim, value_dim]")
+    _need(cu_tokens.shape[0] >= n_seqs + 1 and slots.shape[0] >= n_seqs, "offsets and slots for every request")
+    out = torch.empty((n_tokens, heads * value_dim), dtype=torch.float32, device=proj.device)
+    scratch = torch.empty(int(lib.mll_gla_chunks_scratch(n_tokens, n_seqs, heads, key_dim, value_dim)), dtype=torch.float32, device=proj.device)
+    _check(lib.mll_gla_chunks(_ptr(proj), ctypes.c_int64(proj.shape[1]), q_offset, k_offset, v_offset, _ptr(decay), _ptr(state),
+                              _ptr(cu_tokens), _ptr(slots), _ptr(out), _ptr(scratch), n_tokens, n_seqs, heads, key_dim, value_dim,
+                              ctypes.c_float(q_scale), int(silu_inputs), _stream()), lib)
+    return out
+
+
 def gla_silu(proj: torch.Tensor, first: int, count: int) -> None:
     """``silu`` of the columns ``first .. first + count - 1`` of every row, in place."""
     lib = library.load()

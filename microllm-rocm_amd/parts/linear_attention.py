@@ -11,7 +11,9 @@ scale on the keys instead of the queries is the same ``query_scale``: ``o`` is l
 over ``value_dim`` and multiplied by a weight ``[value_dim]`` that all heads share (``norm_weight`` false: by none); the heads side by side are
 multiplied by ``silu(Wg x)`` and projected by ``Wo``. With ``heads_together`` all heads of a token are divided by one root
 mean square instead, the weight is ``[heads * value_dim]`` and the gate ``sigmoid(Wg x)``; with ``silu_inputs`` queries, keys
-and values pass SiLU before they enter the recurrence (lightning attention is both, with a fixed decay). The state starts at zero, is float32, and lives in the
+and values pass SiLU before they enter the recurrence (lightning attention is both, with a fixed decay). With ``chunked``
+(and a fixed decay, key heads of at most 128 channels) long portions run in chunks of 64 tokens side by side on the matrix
+units instead of token after token: the same sums in another order. The state starts at zero, is float32, and lives in the
 request's state slot, so a request can be cut into steps anywhere. The five projections that read ``x`` are one
 stacked product with a float32 result; decays, the recurrence, the norm and the gate are float32.
 """
@@ -34,6 +36,8 @@ class GatedLinearAttention(Mixer):
     graph_safe = True
     LONG_PORTION = 8        # from this many tokens of one request in a step on, the walk stages its operands through LDS
 
+    CHUNKED_PORTION = 128   # and with ``chunked`` chunks of 64 tokens are taken side by side from this many on
+
     def __init__(self, spec: PartSpec, runtime: Runtime):
         super().__init__(spec, runtime)
         p = spec.params
@@ -49,6 +53,7 @@ class GatedLinearAttention(Mixer):
         self.has_norm_weight = bool(p.get("norm_weight", True))
         self.heads_together = bool(p.get("heads_together", False))
         self.silu_inputs = bool(p.get("silu_inputs", False))
+        self.chunked = bool(p.get("chunked", False)) and self.fixed_decay is not None and self.key_dim <= kernels.GLA_CHUNK_KEYS
         self.eps = float(p.get("eps", 1e-6))
         self.query_scale = float(p.get("query_scale", self.key_dim ** -0.5))
         keys, values = self.heads * self.key_dim, self.heads * self.value_dim
@@ -58,6 +63,7 @@ class GatedLinearAttention(Mixer):
         self.decay_weight: Optional[torch.Tensor] = None
         self.decay_bias: Optional[torch.Tensor] = None
         self.decay_row: Optional[torch.Tensor] = None
+        self.head_decay: Optional[torch.Tensor] = None
         self.norm_weight: Optional[torch.Tensor] = None
         self.o_tensor: Optional[torch.Tensor] = None
         self.o_weight: Optional[Weight] = None
@@ -90,6 +96,7 @@ class GatedLinearAttention(Mixer):
             self.decay_bias = tensors[self.name("a2_bias")]
         else:       # one row of decays for every token: the head's number for each of its key channels
             per_head = torch.tensor(self.fixed_decay, dtype=torch.float32, device=self.o_tensor.device)
+            self.head_decay = per_head
             self.decay_row = per_head.repeat_interleave(self.key_dim).contiguous()
         self.norm_weight = tensors[self.name("norm")] if self.has_norm_weight else None
 
@@ -112,6 +119,11 @@ class GatedLinearAttention(Mixer):
             decay = kernels.gla_decay(proj, self.low_at, self.decay_weight, self.decay_bias, self.tau)
         else:
             decay = self.decay_row
+        if self.chunked and ctx.max_count >= self.CHUNKED_PORTION:
+            o = kernels.gla_chunks(proj, self.q_at, self.k_at, self.v_at, self.head_decay, cache.state, ctx.cu_tokens, ctx.slots, ctx.n_seqs,
+                                   self.heads, self.key_dim, self.value_dim, self.query_scale, silu_inputs=self.silu_inputs)
+            return kernels.gla_gate(o, proj, self.g_at, self.norm_weight, self.eps, self.heads, self.value_dim, out_scale,
+                                    self.runtime.dtype, out=out, heads_together=self.heads_together)
         long_portions = ctx.max_count >= self.LONG_PORTION
         if self.silu_inputs and long_portions:      # one pass over many tokens; few tokens pass it as the walk reads them
             kernels.gla_silu(proj, self.q_at, self.g_at - self.q_at)

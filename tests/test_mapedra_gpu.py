@@ -388,9 +388,10 @@ def test_a_cap_beside_a_window(mfma):
                 assert np.abs(got[query, 0] - want).max() < (0.03 if mfma else 1e-4), (query, key)
 
 
-def lightened(q, k, v, gate, weight, decay, portions_of, eps=1e-5, dtype=torch.float32):
-    """Lightning attention's kernels on one request in the given portions: SiLU, the walk with one decay a head, one norm
-    over all heads and the sigmoid gate; the state carried in a slot."""
+def lightened(q, k, v, gate, weight, decay, portions_of, eps=1e-5, dtype=torch.float32, chunks_from=1 << 30):
+    """Lightning attention's kernels on one request in the given portions: SiLU, the walk with one decay a head (from
+    ``chunks_from`` tokens on the recurrence in chunks), one norm over all heads and the sigmoid gate; the state carried in
+    a slot."""
     from microllm_rocm_amd.ops import kernels
     n, heads, dim = q.shape
     vdim = v.shape[2]
@@ -405,11 +406,15 @@ def lightened(q, k, v, gate, weight, decay, portions_of, eps=1e-5, dtype=torch.f
             break
         rows = slice(first, first + portion)
         proj = device(np.concatenate([a[rows].reshape(portion, -1) for a in (q, k, v, gate)], axis=1))
-        long_portions = portion >= 8
-        if long_portions:
-            kernels.gla_silu(proj, 0, 2 * keys + values)
-        walked = kernels.gla_scan(proj, 0, keys, 2 * keys, decay_row, state, device([0, portion], torch.int32), device([1], torch.int32), 1,
-                                  heads, dim, vdim, 1.0, long_portions=long_portions, silu_inputs=not long_portions)
+        cu, slots = device([0, portion], torch.int32), device([1], torch.int32)
+        if portion >= chunks_from:
+            walked = kernels.gla_chunks(proj, 0, keys, 2 * keys, device(decay), state, cu, slots, 1, heads, dim, vdim, 1.0, silu_inputs=True)
+        else:
+            long_portions = portion >= 8
+            if long_portions:
+                kernels.gla_silu(proj, 0, 2 * keys + values)
+            walked = kernels.gla_scan(proj, 0, keys, 2 * keys, decay_row, state, cu, slots, 1, heads, dim, vdim, 1.0, long_portions=long_portions,
+                                      silu_inputs=not long_portions)
         found = kernels.gla_gate(walked, proj, 2 * keys + values, device(weight), eps, heads, vdim, 1.0, dtype, heads_together=True)
         out.append(found.float().cpu().numpy())
         first += portion
@@ -431,6 +436,9 @@ def test_lightning_attention(heads, dim, vdim, n):
     for portions_of in ([max(n - 30, 2)] + [1] * 30, [2] * (n // 2 + 1), [1] * 5 + [3, 16, 1, 2, 31, 129, 1, 1, 500]):
         again = lightened(q, k, v, gate, weight, decay, portions_of)
         assert np.abs(again - want).max() < 3e-5 * np.abs(want).max(), portions_of
+        if dim <= 128:
+            chunked = lightened(q, k, v, gate, weight, decay, portions_of, chunks_from=2)
+            assert np.abs(chunked - want).max() < 3e-5 * np.abs(want).max(), portions_of
     rounded = lightened(q, k, v, gate, weight, decay, [n], dtype=torch.bfloat16)
     assert np.abs(rounded - want).max() < 0.01 * np.abs(want).max()
 
@@ -450,8 +458,37 @@ def test_a_far_token_stays_in_the_state():
     together = torch.cat([first, torch.zeros(vdim, dtype=F)])
     want = plain.rms(together, 1e-5).numpy()
     for portions_of in ([n], [n - 1, 1], [100, 2, 2, 297]):
-        got = lightened(q, k, v, gate, np.ones(2 * vdim), [1.0, 0.5], portions_of)
-        assert np.abs(got[n - 1] - want).max() < 1e-4, portions_of
+        for chunks_from in (1 << 30, 2):
+            got = lightened(q, k, v, gate, np.ones(2 * vdim), [1.0, 0.5], portions_of, chunks_from=chunks_from)
+            assert np.abs(got[n - 1] - want).max() < 1e-4, portions_of
+
+
+@pytest.mark.parametrize("heads,dim,vdim", [(2, 64, 128), (3, 20, 70), (1, 128, 16), (4, 100, 33)])
+def test_chunks_of_several_requests(heads, dim, vdim):
+    """Requests of unequal lengths in one step (one without tokens, ends on a chunk's edge, one before and one past it), each
+    from a state of its own, against each request's tokens one after the other; no SiLU and a factor on the read-out."""
+    from microllm_rocm_amd.ops import kernels
+    rng = np.random.default_rng(dim)
+    lengths, slots = [130, 1, 0, 64, 63, 65, 200], [3, 0, 7, 5, 1, 2, 6]
+    cu = np.concatenate([[0], np.cumsum(lengths)])
+    n, keys, values = cu[-1], heads * dim, heads * vdim
+    q, k, v = (rng.normal(size=(n, heads, size)) for size in (dim, dim, vdim))
+    decay = [0.99, 0.0, 1.0, 0.6][:heads]
+    before = rng.normal(size=(8, heads, dim, vdim))
+    proj = device(np.concatenate([a.reshape(n, -1) for a in (q, k, v)], axis=1))
+    state = device(before)
+    got = kernels.gla_chunks(proj, 0, keys, 2 * keys, device(decay), state, device(cu, torch.int32), device(slots, torch.int32), len(lengths),
+                             heads, dim, vdim, 0.5).cpu().numpy().reshape(n, heads, vdim)
+    walked = device(before)
+    kernels.gla_scan(proj, 0, keys, 2 * keys, device(np.repeat(decay, dim)), walked, device(cu, torch.int32), device(slots, torch.int32),
+                     len(lengths), heads, dim, vdim, 0.5, long_portions=True)
+    assert (state - walked).abs().max() < 2e-5 * walked.abs().max() and torch.equal(state[4], device(before)[4])
+    assert torch.equal(state[7], device(before)[7])        # the request that brought nothing
+    for index, slot in enumerate(slots):
+        rows = slice(cu[index], cu[index + 1])
+        want = 0.5 * plain.retain(t64(q[rows]), t64(k[rows]), t64(v[rows]), decay, t64(before[slot])).numpy()
+        if lengths[index]:
+            assert np.abs(got[rows] - want).max() < 2e-5 * np.abs(want).max(), index
 
 
 # ---- the engine ---------------------------------------------------------------------------------------------------
@@ -494,7 +531,7 @@ def test_whole_decode_and_portions(tmp_path_factory, tmp_path, which, dtype):
         steps = prefill_then_decode(rid, requests[rid], tail=tail)
         run_trace(folder, dtype, steps, tmp_path / f"decode_{rid}", max_tokens=round_up(len(requests[rid]), 64))
         check_against_plain(steps, tmp_path / f"decode_{rid}", {rid: requests[rid]}, config, weights, dtype)
-    for sizes in ([2], [3, 16, 1, 2, 31], [64, 2, 17]):
+    for sizes in ([2], [3, 16, 1, 2, 31], [64, 2, 17], [131, 2, 7]):
         steps = portions("long", requests["long"], sizes)
         run_trace(folder, dtype, steps, tmp_path / f"portions_{sizes[0]}", max_tokens=192)
         check_against_plain(steps, tmp_path / f"portions_{sizes[0]}", {"long": requests["long"]}, config, weights, dtype)
