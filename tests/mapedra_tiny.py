@@ -47,12 +47,12 @@ TINY_B = MapedraConfig(
         _layer(_attention(2, 2, 14, 20, 0.3, 4, 2.5, base=100.0, bands=(2.0, 0.5, 0.5, 40.0)), 33),
     ))
 # Norms in parts of six channels (no multiple of four), a side vector as wide as the model, a large factor on the
-# embedding, eps that matters; heads of 96 (three tiles of 32) with 64 turned; a lightning layer last.
+# embedding, eps that matters; heads of 112 (an odd number of tiles of 16) with 64 turned; a lightning layer last.
 TINY_C = MapedraConfig(
     vocab=150, width=96, norm_eps=1e-3, norm_groups=16, side_dim=96, embedding_scale=12.0,
     layers=(
         _layer(_lightning(16, 24, [0.75, 0.95]), 128),
-        _layer(_attention(8, 2, 96, 96, 0.1, 64, 15.0, base=5e5, bands=(4.0, 1.0, 4.0, 512.0)), 160),
+        _layer(_attention(8, 2, 112, 112, 0.1, 64, 15.0, base=3e5, bands=(5.0, 1.0, 6.0, 512.0)), 160),
         _layer(_attention(2, 1, 24, 40, 0.3, 24, 6.0), 16),
         _layer(_lightning(5, 32, [0.9375, 0.875, 0.6, 0.999, 0.3, 0.98, 0.2]), None),
     ))

@@ -81,7 +81,7 @@ def test_refusals(change, text):
         MapedraConfig.from_dict(source)
 
 
-@pytest.mark.parametrize("base,n,bands", [(10000.0, 8, (3.0, 1.0, 8.0, 64.0)), (5e5, 64, (4.0, 1.0, 4.0, 512.0)), (77.0, 10, (1.0, 1.0, 4.0, 300.0)),
+@pytest.mark.parametrize("base,n,bands", [(10000.0, 8, (3.0, 1.0, 8.0, 64.0)), (3e5, 64, (5.0, 1.0, 6.0, 512.0)), (77.0, 10, (1.0, 1.0, 4.0, 300.0)),
                                           (100.0, 4, (2.0, 0.5, 0.5, 40.0)), (1e4, 2, (8.0, 2.0, 3.0, 9.0))])
 def test_rates_stretched_by_bands(base, n, bands):
     scaling = dict(zip(("factor", "low", "high", "original"), bands))
