@@ -1,2 +1,2 @@
 """Architectures this package provides; importing the package registers them."""
-from . import gupitar, kalevik, mapedra, qwen2, siditar, zabozen  # noqa: F401
+from . import gupitar, kalevik, mapedra, qwen2, siditar, zabozen, zuluvik  # noqa: F401

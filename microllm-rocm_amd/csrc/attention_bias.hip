@@ -59,12 +59,12 @@ template <> __device__ inline float dot_row<bf16>(const bf16* key, const float* 
     return sum;
 }
 
-template <typename T>
+template <typename T, typename O>
 __global__ void __launch_bounds__(kWave)
 bias_attention_kernel(const T* __restrict__ q, const T* __restrict__ k_pages, const T* __restrict__ v_pages,
                       const int32_t* __restrict__ block_table, int table_width, const int32_t* __restrict__ seq_of_token,
                       const int32_t* __restrict__ positions, const float* __restrict__ bias, int longest,
-                      const float* __restrict__ sink, T* __restrict__ out, int64_t out_stride, int heads, int kv_heads,
+                      const float* __restrict__ sink, O* __restrict__ out, int64_t out_stride, int heads, int kv_heads,
                       int key_dim, int value_dim, int page_size, float scale, float out_scale,
                       const float* __restrict__ slopes, int window, int chunk, const float* __restrict__ gate,
                       int64_t gate_stride, float softcap, int gate_channels) {
@@ -124,26 +124,27 @@ bias_attention_kernel(const T* __restrict__ q, const T* __restrict__ k_pages, co
     float factor = out_scale / running_sum;
     const float* gate_row = gate ? gate + static_cast<int64_t>(token) * gate_stride + (gate_channels ? head * value_dim : head) : nullptr;
     if (gate_row && !gate_channels) factor *= 1.0f / (1.0f + expf(-gate_row[0]));
-    T* to = out + static_cast<int64_t>(token) * out_stride + static_cast<int64_t>(head) * value_dim;
+    O* to = out + static_cast<int64_t>(token) * out_stride + static_cast<int64_t>(head) * value_dim;
 #pragma unroll
     for (int m = 0; m < kMaxValueChannelsALane; ++m) {
         const int c = lane + m * kWave;
-        if (c < value_dim) to[c] = from_float<T>(gate_row && gate_channels ? acc[m] * factor / (1.0f + expf(-gate_row[c])) : acc[m] * factor);
+        if (c < value_dim) to[c] = from_float<O>(gate_row && gate_channels ? acc[m] * factor / (1.0f + expf(-gate_row[c])) : acc[m] * factor);
     }
 }
 
 constexpr int kNormStoreWaves = 4;
 
 // One wave a (token, head of q, k or v), four to a workgroup: the norm of queries and keys over their head, the queries' factor by
-// position, and the write of keys and values into their pages.
-template <typename T>
+// position, and the write of keys and values into their pages. MORE: with what MllStoreExtras says (a convolution over time
+// before everything else, the norm after the turn, heads stored wider than they are, several keys a key head).
+template <typename T, bool MORE>
 __global__ void __launch_bounds__(kNormStoreWaves * kWave)
 qk_norm_store_kernel(const float* __restrict__ qkv, int n_parts, int64_t part_stride, const float* __restrict__ q_weight,
                      const float* __restrict__ k_weight, float eps, const int32_t* __restrict__ positions,
                      const int32_t* __restrict__ slot_mapping, float temp_coef, int temp_every, T* __restrict__ q_out,
                      T* __restrict__ k_pages, T* __restrict__ v_pages, int heads, int kv_heads, int key_dim, int value_dim,
                      int tiled_page_size, const float* __restrict__ bias, int normed, int queries_only, int64_t row_stride,
-                     const float* __restrict__ cos_sin, int rot_dims, int values_normed, int total) {
+                     const float* __restrict__ cos_sin, int rot_dims, int values_normed, int total, MllStoreExtras more) {
     const int vectors = queries_only ? heads : heads + 2 * kv_heads;
     const int vector = blockIdx.x * kNormStoreWaves + threadIdx.x / kWave;
     if (vector >= total) return;
@@ -153,16 +154,55 @@ qk_norm_store_kernel(const float* __restrict__ qkv, int n_parts, int64_t part_st
     const float* row = qkv + static_cast<int64_t>(token) * row_stride;
     const bool is_q = which < heads, is_k = !is_q && which < heads + kv_heads;
     const int head = is_q ? which : (is_k ? which - heads : which - heads - kv_heads);
-    const int dim = (is_q || is_k) ? key_dim : value_dim;
-    const int offset = is_q ? head * key_dim : (is_k ? (heads + head) * key_dim : (heads + kv_heads) * key_dim + head * value_dim);
+    const int query_dim = MORE && more.maps > 1 ? key_dim / more.maps : key_dim;
+    const int dim = is_q ? query_dim : (is_k ? key_dim : value_dim);
+    const int offset = is_q ? head * query_dim
+                            : (is_k ? heads * query_dim + head * key_dim : heads * query_dim + kv_heads * key_dim + head * value_dim);
     const int slot = is_q ? 0 : slot_mapping[token];
     if (!is_q && slot < 0) return;
+    int tokens_before = 0;              // of the same request in this step
+    const float* tail = nullptr;        // the inputs before the step
+    if (MORE && more.taps != nullptr) {
+        const int seq = more.seq_of_token[token];
+        if (seq < 0) return;            // a row that pads the step
+        tokens_before = token - more.cu_tokens[seq];
+        tail = more.kept + static_cast<int64_t>(more.slots[seq]) * (more.n_taps - 1) * (heads * query_dim + kv_heads * (key_dim + value_dim));
+    }
+    // what the vector holds at channel c before it is normed or turned: the sums (or their convolution over time), the bias
+    auto raw = [&](int c) {
+        float value;
+        if (MORE && more.taps != nullptr) {
+            const int columns = heads * query_dim + kv_heads * (key_dim + value_dim);
+            const float* tap = more.taps + static_cast<int64_t>(offset + c) * more.n_taps;
+            value = 0.0f;
+            for (int j = 0; j < more.n_taps; ++j) {
+                const int back = more.n_taps - 1 - j;       // how many tokens before this one
+                const float input = back <= tokens_before
+                                        ? row[offset + c - static_cast<int64_t>(back) * row_stride]
+                                        : tail[static_cast<int64_t>(more.n_taps - 1 - (back - tokens_before)) * columns + offset + c];
+                value = fmaf(tap[j], input, value);
+            }
+        } else {
+            value = row[offset + c];
+            for (int part = 1; part < n_parts; ++part) value += row[part * part_stride + offset + c];
+        }
+        if (bias) value += bias[offset + c];
+        return value;
+    };
+    // queries and keys turn by the token's position in their first rot_dims channels, channel i with i + rot_dims / 2
+    const bool turns = cos_sin != nullptr && (is_q || is_k);
+    const int half = rot_dims / 2;
+    const float* angles = cos_sin + static_cast<int64_t>(token) * rot_dims;     // [rot_dims / 2][cos, sin]
+    const bool norm_turned = MORE && more.norm_turned && turns;
     float squares = 0.0f;
     for (int c = lane; c < dim; c += kWave) {
-        float value = row[offset + c];
-        for (int part = 1; part < n_parts; ++part) value += row[part * part_stride + offset + c];
-        if (bias) value += bias[offset + c];
-        squares += value * value;
+        const float value = raw(c);
+        float length = 1.0f;
+        if (norm_turned && c < rot_dims) {      // a turned pair is as long as before, but for the factor within cos and sin
+            const int pair = c < half ? c : c - half;
+            length = angles[2 * pair] * angles[2 * pair] + angles[2 * pair + 1] * angles[2 * pair + 1];
+        }
+        squares += value * value * length;
     }
     const float* weight = is_q ? q_weight : (is_k ? k_weight : nullptr);
     const bool norm = (is_q || is_k) ? normed : values_normed;
@@ -172,39 +212,40 @@ qk_norm_store_kernel(const float* __restrict__ qkv, int n_parts, int64_t part_st
         const int steps = (positions[token] + 1) / temp_every;
         factor *= 1.0f + temp_coef * static_cast<float>(log(static_cast<double>(steps) + 1.0));
     }
-    T* to = is_q ? q_out + (static_cast<int64_t>(token) * heads + head) * key_dim
-                 : (is_k ? k_pages + (static_cast<int64_t>(slot) * kv_heads + head) * key_dim
-                         : v_pages + (static_cast<int64_t>(slot) * kv_heads + head) * value_dim);
+    // how wide the vectors are kept, and where among a key head's keys this query's lies
+    const int key_width = MORE && more.stored_dim > 0 ? more.stored_dim : key_dim;
+    const int value_width = MORE && more.stored_dim > 0 ? more.stored_dim : value_dim;
+    const int place = MORE && is_q && more.maps > 1 ? (head % more.maps) * query_dim : 0;
+    T* to = is_q ? q_out + (static_cast<int64_t>(token) * heads + head) * key_width
+                 : (is_k ? k_pages + (static_cast<int64_t>(slot) * kv_heads + head) * key_width
+                         : v_pages + (static_cast<int64_t>(slot) * kv_heads + head) * value_width);
     // tiled_page_size > 0: the pages are in the order the MFMA kernels read them (cache_layout.h; both widths equal)
     const bool tiled = tiled_page_size > 0 && !is_q;
-    const CacheLayout layout(kv_heads, tiled ? tiled_page_size : 16, key_dim);
+    const CacheLayout layout(kv_heads, tiled ? tiled_page_size : 16, key_width);
     const int64_t page = tiled ? slot / tiled_page_size : 0;
     const int in_page = tiled ? slot % tiled_page_size : 0;
-    // what the vector holds at channel c before it is turned: the sums, the bias, the norm
-    auto prepared = [&](int c) {
-        float value = row[offset + c];
-        for (int part = 1; part < n_parts; ++part) value += row[part * part_stride + offset + c];
-        if (bias) value += bias[offset + c];
-        return norm ? (weight ? value * factor * weight[c] : value * factor) : value;
-    };
-    // queries and keys turn by the token's position in their first rot_dims channels, channel i with i + rot_dims / 2
-    const bool turns = cos_sin != nullptr && (is_q || is_k);
-    const int half = rot_dims / 2;
-    const float* angles = cos_sin + static_cast<int64_t>(token) * rot_dims;     // [rot_dims / 2][cos, sin]
-    for (int c = lane; c < dim; c += kWave) {
-        float value = prepared(c);
-        if (turns && c < rot_dims) {
-            const int pair = c < half ? c : c - half;
-            const float other = prepared(c < half ? c + half : c - half);
-            const float cosine = angles[2 * pair], sine = angles[2 * pair + 1];
-            value = c < half ? value * cosine - other * sine : value * cosine + other * sine;
+    auto normed_value = [&](float value, int c) { return norm ? (weight ? value * factor * weight[c] : value * factor) : value; };
+    auto prepared = [&](int c) { return norm_turned ? raw(c) : normed_value(raw(c), c); };      // what is turned
+    const int kept_width = MORE ? (is_q || is_k ? key_width : value_width) : dim;
+    for (int at = lane; at < kept_width; at += kWave) {
+        const int c = at - place;
+        float value = 0.0f;
+        if (!MORE || (c >= 0 && c < dim)) {
+            value = prepared(c);
+            if (turns && c < rot_dims) {
+                const int pair = c < half ? c : c - half;
+                const float other = prepared(c < half ? c + half : c - half);
+                const float cosine = angles[2 * pair], sine = angles[2 * pair + 1];
+                value = c < half ? value * cosine - other * sine : value * cosine + other * sine;
+            }
+            if (norm_turned) value = normed_value(value, c);
         }
         const T rounded = from_float<T>(value);
         if (tiled) {
-            if (is_k) k_pages[layout.k_at(page, head, in_page, c)] = rounded;
-            else v_pages[layout.v_at(page, head, in_page, c)] = rounded;
+            if (is_k) k_pages[layout.k_at(page, head, in_page, at)] = rounded;
+            else v_pages[layout.v_at(page, head, in_page, at)] = rounded;
         } else {
-            to[c] = rounded;
+            to[at] = rounded;
         }
     }
 }
@@ -219,13 +260,22 @@ int mll_qk_norm_store(const float* qkv, int n_parts, int64_t part_stride, const 
                       float eps, const int32_t* positions, const int32_t* slot_mapping, float temp_coef, int temp_every,
                       void* q_out, void* k_pages, void* v_pages, int dtype, int n_tokens, int heads, int kv_heads, int key_dim,
                       int value_dim, int tiled_page_size, const float* bias, int normed, int queries_only, int64_t row_stride,
-                      const float* cos_sin, int rot_dims, int values_normed, hipStream_t stream) {
-    MLL_REQUIRE(tiled_page_size == 0 || (tiled_page_size > 0 && tiled_page_size % 16 == 0 && key_dim == value_dim),
+                      const float* cos_sin, int rot_dims, int values_normed, const MllStoreExtras* more, hipStream_t stream) {
+    const MllStoreExtras given = more ? *more : MllStoreExtras{};
+    const int maps = given.maps > 1 ? given.maps : 1;
+    MLL_REQUIRE(tiled_page_size == 0 || (tiled_page_size > 0 && tiled_page_size % 16 == 0 && (key_dim == value_dim || given.stored_dim > 0)),
                 "qk_norm_store: tiled pages hold a multiple of 16 positions and keys and values of one width");
     MLL_REQUIRE(n_tokens >= 0 && heads > 0 && kv_heads > 0 && key_dim > 0 && value_dim > 0, "qk_norm_store: sizes must be positive");
     MLL_REQUIRE(n_parts >= 1, "qk_norm_store: at least one part");
-    MLL_REQUIRE(row_stride >= (queries_only ? heads * key_dim : (heads + kv_heads) * key_dim + kv_heads * value_dim),
+    MLL_REQUIRE(key_dim % maps == 0 && heads % maps == 0, "qk_norm_store: a key head holds equal keys, and every map has as many query heads");
+    MLL_REQUIRE(row_stride >= (queries_only ? heads * (key_dim / maps) : heads * (key_dim / maps) + kv_heads * (key_dim + value_dim)),
                 "qk_norm_store: the rows are narrower than their queries, keys and values");
+    MLL_REQUIRE(maps == 1 || (!normed && cos_sin == nullptr), "qk_norm_store: several keys a key head are neither normed nor turned");
+    MLL_REQUIRE(given.stored_dim == 0 || (given.stored_dim >= key_dim && given.stored_dim >= value_dim), "qk_norm_store: heads are stored at least as wide as they are");
+    MLL_REQUIRE(given.taps == nullptr || (n_parts == 1 && !queries_only && given.n_taps >= 1 && (given.n_taps == 1 || given.kept != nullptr) &&
+                                          given.seq_of_token && given.cu_tokens && given.slots),
+                "qk_norm_store: a convolution reads whole rows of q, k and v, the request of every token and what requests kept");
+    MLL_REQUIRE(!given.norm_turned || (normed && cos_sin != nullptr), "qk_norm_store: a norm of turned vectors needs both");
     MLL_REQUIRE(cos_sin == nullptr || (rot_dims > 0 && rot_dims % 2 == 0 && rot_dims <= key_dim),
                 "qk_norm_store: an even number of turned channels, at most the head's");
     MLL_REQUIRE((q_weight == nullptr) == (k_weight == nullptr), "qk_norm_store: norm weights for queries and keys, or for neither");
@@ -237,19 +287,19 @@ int mll_qk_norm_store(const float* qkv, int n_parts, int64_t part_stride, const 
     const int64_t total = static_cast<int64_t>(n_tokens) * (queries_only ? heads : heads + 2 * kv_heads);
     MLL_REQUIRE(total < (1ll << 31) - kNormStoreWaves, "qk_norm_store: too many rows for one launch");
     const int64_t blocks = (total + kNormStoreWaves - 1) / kNormStoreWaves;
+#define MLL_NORM_STORE(T, MORE)                                                                                               \
+    qk_norm_store_kernel<T, MORE><<<static_cast<unsigned>(blocks), kNormStoreWaves * kWave, 0, stream>>>(                         \
+        qkv, n_parts, part_stride, q_weight, k_weight, eps, positions, slot_mapping, temp_coef, temp_every, static_cast<T*>(q_out), \
+        static_cast<T*>(k_pages), static_cast<T*>(v_pages), heads, kv_heads, key_dim, value_dim, tiled_page_size, bias, normed,     \
+        queries_only, row_stride, cos_sin, rot_dims, values_normed, static_cast<int>(total), given)
     if (dtype == kF32) {
-        qk_norm_store_kernel<float><<<static_cast<unsigned>(blocks), kNormStoreWaves * kWave, 0, stream>>>(
-            qkv, n_parts, part_stride, q_weight, k_weight, eps, positions, slot_mapping, temp_coef, temp_every,
-            static_cast<float*>(q_out), static_cast<float*>(k_pages), static_cast<float*>(v_pages), heads, kv_heads, key_dim, value_dim,
-            tiled_page_size, bias, normed, queries_only, row_stride, cos_sin, rot_dims, values_normed, static_cast<int>(total));
+        if (more) MLL_NORM_STORE(float, true); else MLL_NORM_STORE(float, false);
     } else if (dtype == kBF16) {
-        qk_norm_store_kernel<bf16><<<static_cast<unsigned>(blocks), kNormStoreWaves * kWave, 0, stream>>>(
-            qkv, n_parts, part_stride, q_weight, k_weight, eps, positions, slot_mapping, temp_coef, temp_every,
-            static_cast<bf16*>(q_out), static_cast<bf16*>(k_pages), static_cast<bf16*>(v_pages), heads, kv_heads, key_dim, value_dim,
-            tiled_page_size, bias, normed, queries_only, row_stride, cos_sin, rot_dims, values_normed, static_cast<int>(total));
+        if (more) MLL_NORM_STORE(bf16, true); else MLL_NORM_STORE(bf16, false);
     } else {
         return fail("qk_norm_store: unknown dtype");
     }
+#undef MLL_NORM_STORE
     return check_launch("qk_norm_store");
 }
 
@@ -257,7 +307,8 @@ int mll_bias_attention(const void* q, const void* k_pages, const void* v_pages, 
                        const int32_t* seq_of_token, const int32_t* positions, const float* bias, int longest,
                        const float* sink, void* out, int64_t out_stride, int dtype, int n_tokens, int heads, int kv_heads,
                        int key_dim, int value_dim, int page_size, float scale, float out_scale, const float* slopes, int window,
-                       int chunk, const float* gate, int64_t gate_stride, float softcap, int gate_channels, hipStream_t stream) {
+                       int chunk, const float* gate, int64_t gate_stride, float softcap, int gate_channels, int out_f32,
+                       hipStream_t stream) {
     MLL_REQUIRE(n_tokens >= 0 && heads > 0 && kv_heads > 0 && key_dim > 0 && value_dim > 0 && page_size > 0 && table_width > 0,
                 "bias_attention: sizes must be positive");
     MLL_REQUIRE(heads % kv_heads == 0, "bias_attention: heads must divide into kv heads");
@@ -272,19 +323,19 @@ int mll_bias_attention(const void* q, const void* k_pages, const void* v_pages, 
     MLL_REQUIRE(blocks < (1ll << 31), "bias_attention: too many rows for one launch");
     const size_t lds = static_cast<size_t>(key_dim) * sizeof(float);
     MLL_REQUIRE(lds <= 64 * 1024, "bias_attention: key heads wider than 16384 are not supported");
+#define MLL_BIAS_ATTENTION(T, O)                                                                                              \
+    bias_attention_kernel<T, O><<<static_cast<unsigned>(blocks), kWave, lds, stream>>>(                                           \
+        static_cast<const T*>(q), static_cast<const T*>(k_pages), static_cast<const T*>(v_pages), block_table, table_width,         \
+        seq_of_token, positions, bias, longest, sink, static_cast<O*>(out), out_stride, heads, kv_heads, key_dim, value_dim,        \
+        page_size, scale, out_scale, slopes, window, chunk, gate, gate_stride, softcap, gate_channels)
     if (dtype == kF32) {
-        bias_attention_kernel<float><<<static_cast<unsigned>(blocks), kWave, lds, stream>>>(
-            static_cast<const float*>(q), static_cast<const float*>(k_pages), static_cast<const float*>(v_pages), block_table,
-            table_width, seq_of_token, positions, bias, longest, sink, static_cast<float*>(out), out_stride, heads, kv_heads,
-            key_dim, value_dim, page_size, scale, out_scale, slopes, window, chunk, gate, gate_stride, softcap, gate_channels);
+        MLL_BIAS_ATTENTION(float, float);
     } else if (dtype == kBF16) {
-        bias_attention_kernel<bf16><<<static_cast<unsigned>(blocks), kWave, lds, stream>>>(
-            static_cast<const bf16*>(q), static_cast<const bf16*>(k_pages), static_cast<const bf16*>(v_pages), block_table,
-            table_width, seq_of_token, positions, bias, longest, sink, static_cast<bf16*>(out), out_stride, heads, kv_heads,
-            key_dim, value_dim, page_size, scale, out_scale, slopes, window, chunk, gate, gate_stride, softcap, gate_channels);
+        if (out_f32) MLL_BIAS_ATTENTION(bf16, float); else MLL_BIAS_ATTENTION(bf16, bf16);
     } else {
         return fail("bias_attention: unknown dtype");
     }
+#undef MLL_BIAS_ATTENTION
     return check_launch("bias_attention");
 }
 

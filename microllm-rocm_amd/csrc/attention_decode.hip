@@ -48,6 +48,13 @@ __device__ inline float result_gate(const MllAttentionExtras& extras, int token,
     return 1.0f / (1.0f + __expf(-extras.gate[static_cast<int64_t>(token) * extras.gate_stride + column]));
 }
 
+// One number of a token's results, in the type the extras name.
+__device__ inline void store_result(const MllAttentionExtras& extras, bf16* out, int token, int column, float value) {
+    const int64_t at = static_cast<int64_t>(token) * extras.out_stride + column;
+    if (extras.out_f32) reinterpret_cast<float*>(out)[at] = value;
+    else out[at] = from_float<bf16>(value);
+}
+
 // EXTRA: the scores also get extras.bias[min(position - key, longest)][head], the softmax's denominator also holds
 // exp(extras.sink[head]) (counted once, where the waves' or the splits' results meet), the result is multiplied by
 // extras.out_scale and by its gate and its rows lie extras.out_stride elements apart; with extras.chunk the keys
@@ -308,7 +315,7 @@ __global__ __launch_bounds__(kDecodeThreads) void paged_attention_decode_kernel(
         const int64_t row = static_cast<int64_t>(token) * heads + head0 + h;
         const int64_t part_row = static_cast<int64_t>(blockIdx.x) * heads + head0 + h;   // partial results are kept densely
         if (n_splits == 1) {
-            if (EXTRA) out[static_cast<int64_t>(token) * extras.out_stride + (head0 + h) * HD + dim] = from_float<bf16>(total / sum * extras.out_scale * result_gate(extras, token, head0 + h, HD, dim));
+            if (EXTRA) store_result(extras, out, token, (head0 + h) * HD + dim, total / sum * extras.out_scale * result_gate(extras, token, head0 + h, HD, dim));
             else out[row * HD + dim] = from_float<bf16>(total / sum);
         } else {
             part_o[(part_row * n_splits + split) * HD + dim] = total;
@@ -362,7 +369,7 @@ __global__ void paged_attention_join_kernel(const float* __restrict__ part_o, co
             }
         }
         if (with_sink) weight_sum += __expf(sink - top);
-        if (EXTRA) out[static_cast<int64_t>(token) * extras.out_stride + (blockIdx.x % heads) * head_dim + dim] = from_float<bf16>(total / weight_sum * extras.out_scale * result_gate(extras, token, blockIdx.x % heads, head_dim, dim));
+        if (EXTRA) store_result(extras, out, token, (blockIdx.x % heads) * head_dim + dim, total / weight_sum * extras.out_scale * result_gate(extras, token, blockIdx.x % heads, head_dim, dim));
         else out[row * head_dim + dim] = from_float<bf16>(total / weight_sum);
     }
 }

@@ -509,6 +509,12 @@ __global__ __launch_bounds__(kPrefillThreads, 1) void paged_attention_prefill_ke
             for (int j = 0; j < 4; ++j) {
                 const int dim = d * 32 + 8 * j + 4 * half;
                 if (HD % 32 != 0 && dim >= HD) continue;
+                if (EXTRA && extras.out_f32) {       // no gates a channel then
+                    float* row = reinterpret_cast<float*>(out) + static_cast<int64_t>(first_token + block_first + column) * extras.out_stride + head * HD;
+                    *reinterpret_cast<float4*>(row + dim) = make_float4(o_acc[d][4 * j] * inverse, o_acc[d][4 * j + 1] * inverse,
+                                                                        o_acc[d][4 * j + 2] * inverse, o_acc[d][4 * j + 3] * inverse);
+                    continue;
+                }
                 bf16x4 four;
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
@@ -562,6 +568,8 @@ extern "C" int mll_paged_attention_prefill_extra(const void* q, const void* k_ca
                                                  int n_tiles, const int32_t* positions, void* out, float scale, int window,
                                                  int heads, int kv_heads, int head_dim, int page_size,
                                                  const MllAttentionExtras* extras, hipStream_t stream) {
+    MLL_REQUIRE(!extras || !extras->out_f32 || (!extras->gate_channels && extras->out_stride % 4 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0),
+                "paged_attention_prefill: float32 results come in aligned rows and without a gate a channel");
     MLL_REQUIRE(!extras || scale > 0.0f, "paged_attention_prefill: a bias, a sink or a cap on the scores needs a positive scale");
     MLL_REQUIRE(!extras || !extras->bias || (extras->longest >= 0 && extras->longest < kPrefillBiasRows),
                 "paged_attention_prefill: the bias table has more rows than the kernel keeps");

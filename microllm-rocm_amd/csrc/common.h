@@ -87,6 +87,15 @@ __device__ inline float activate(float z, int act) {
     return z / (1.0f + expf(-z));
 }
 
+// The fourth kind is for a gated pair alone: both inputs clamped, a sigmoid of steeper argument, one added to the second.
+constexpr int kActClampedGlu = 3;
+__device__ inline float gated_value(float g, float u, int act, float limit, float slope) {
+    if (act != kActClampedGlu) return activate(g, act) * u;
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g / (1.0f + expf(-slope * g)) * (u + 1.0f);
+}
+
 // The gate of a gated product's epilogue, with the fast exponential: silu(z), or the tanh form of gelu, which is
 // z sigmoid(2 sqrt(2 / pi) (z + 0.044715 z^3)).
 template <bool GELU>

@@ -187,11 +187,11 @@ __global__ void softcap_kernel(float* __restrict__ values, int64_t count, float 
 // cos and sin of position * inv_freq for every token of a step: angles in float64, so that the float32 values
 // are the correctly rounded ones for any position. out[token][pair] = (cos, sin).
 __global__ void rope_table_kernel(const int32_t* __restrict__ positions, const double* __restrict__ inv_freq,
-                                  int n_freq, int64_t count, float2* __restrict__ out) {
+                                  int n_freq, int64_t count, double factor, float2* __restrict__ out) {
     const int64_t index = static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x;
     if (index >= count) return;
     const double angle = static_cast<double>(positions[index / n_freq]) * inv_freq[index % n_freq];
-    out[index] = make_float2(static_cast<float>(cos(angle)), static_cast<float>(sin(angle)));
+    out[index] = make_float2(static_cast<float>(cos(angle) * factor), static_cast<float>(sin(angle) * factor));
 }
 
 // One block per token (and group of heads). cos and sin come from the step's table, or are computed here
@@ -604,13 +604,13 @@ int mll_qkv_rope_store(const void* qkv, int in_dtype, int n_partials, int64_t pa
     return check_launch("qkv_rope_store");
 }
 
-int mll_rope_table(const int32_t* positions, const double* inv_freq, int n_freq, int n_tokens, float* out,
+int mll_rope_table(const int32_t* positions, const double* inv_freq, int n_freq, int n_tokens, double factor, float* out,
                    hipStream_t stream) {
     MLL_REQUIRE(n_freq > 0 && n_tokens >= 0, "rope_table: sizes must be positive");
     MLL_REQUIRE(reinterpret_cast<uintptr_t>(out) % 8 == 0, "rope_table: the table must be 8-byte aligned");
     if (n_tokens == 0) return 0;
     const int64_t count = static_cast<int64_t>(n_tokens) * n_freq;
-    rope_table_kernel<<<static_cast<unsigned>((count + 255) / 256), 256, 0, stream>>>(positions, inv_freq, n_freq, count,
+    rope_table_kernel<<<static_cast<unsigned>((count + 255) / 256), 256, 0, stream>>>(positions, inv_freq, n_freq, count, factor,
                                                                                       reinterpret_cast<float2*>(out));
     return check_launch("rope_table");
 }

@@ -42,6 +42,19 @@ int mll_rms_norm_after(float* h, const void* delta, int delta_dtype, int n_parti
                        const float* weight, float eps, void* out, int dtype, int n_rows, int width, int write_h, int groups,
                        hipStream_t stream);
 
+// What several sublayers add to the stream at once: `count` tensors of float32 partial sums, source i in parts[i] parts.
+#define kMllDeltaSources 4
+typedef struct MllDeltas {
+    const float* from[kMllDeltaSources];
+    int parts[kMllDeltaSources];
+    int count;
+} MllDeltas;
+
+// As mll_rms_norm with v = h[r] + every part of every source in order; parts lie part_stride elements apart
+// (csrc/norm_sum.hip).
+int mll_rms_norm_sum(float* h, const MllDeltas* deltas, int64_t part_stride, const int32_t* rows, const float* weight, float eps,
+                     void* out, int dtype, int n_rows, int width, int write_h, hipStream_t stream);
+
 // values[r][c] += bias[c] for n_rows rows of `width` float32 values, in place.
 int mll_add_bias(float* values, const float* bias, int64_t n_rows, int width, hipStream_t stream);
 
@@ -51,8 +64,8 @@ int mll_softcap(float* values, int64_t count, float cap, hipStream_t stream);
 // Adds a pending delta into the residual stream: h[r] += delta[r] for all rows.
 int mll_residual_add(float* h, const void* delta, int dtype, int n_rows, int width, hipStream_t stream);
 
-// out[t][i] = (cos, sin) of positions[t] * inv_freq[i], the angle in float64: float32 [n_tokens][n_freq][2].
-int mll_rope_table(const int32_t* positions, const double* inv_freq, int n_freq, int n_tokens, float* out,
+// out[t][i] = factor * (cos, sin) of positions[t] * inv_freq[i], the angle in float64: float32 [n_tokens][n_freq][2].
+int mll_rope_table(const int32_t* positions, const double* inv_freq, int n_freq, int n_tokens, double factor, float* out,
                    hipStream_t stream);
 
 // Splits fused projections qkv[t] = [q (H*hd) | k (KVH*hd) | v (KVH*hd)], adds `bias` (nullable),
@@ -273,6 +286,7 @@ typedef struct MllAttentionExtras {
     int64_t gate_stride;
     float softcap;          // > 0: the scaled score becomes softcap * tanh(score / softcap), before a bias is added
     int gate_channels;      // with gate: its rows hold heads * head_dim numbers, one for every channel of the result
+    int out_f32;            // the result is float32 (out_stride counts floats)
 } MllAttentionExtras;
 
 int mll_paged_attention_decode_extra(const void* q, const void* k_cache, const void* v_cache,
@@ -328,11 +342,31 @@ int mll_clamped_glu(const float* gate_up, void* out, int dtype, int n_tokens, in
 // [n_tokens][rot_dims / 2][cos, sin]) queries and keys are turned after their norm: channel i < rot_dims / 2 of a head
 // with channel i + rot_dims / 2, (u, v) -> (u cos - v sin, v cos + u sin); the other channels pass. values_normed: values
 // are divided by their root mean square over their head (no weight) before they are stored.
+// more (null: none of it): what MllStoreExtras says.
+typedef struct MllStoreExtras {
+    int stored_dim;         // > 0: queries, keys and values are kept in rows of this width (at least either width), zeros behind
+    int maps;               // > 1: a key head holds that many keys of key_dim / maps channels side by side, and query head h
+                            // is key_dim / maps channels that meet key h % maps: written at that place, zeros in the others
+                            // (then no norm and no rotation)
+    int norm_turned;        // the norm of queries and keys is taken of the turned vectors
+    const float* taps;      // null, or float32 [columns][n_taps]: every column of qkv is first convolved over the request's tokens,
+    int n_taps;             // the last tap on the token itself; `kept` float32 [slot][n_taps - 1][columns] holds the inputs before
+    const float* kept;      // the step (newest last), the step's own come from qkv (in one part); rows of no request are skipped
+    const int32_t* seq_of_token;
+    const int32_t* cu_tokens;
+    const int32_t* slots;
+} MllStoreExtras;
+
 int mll_qk_norm_store(const float* qkv, int n_parts, int64_t part_stride, const float* q_weight, const float* k_weight,
                       float eps, const int32_t* positions, const int32_t* slot_mapping, float temp_coef, int temp_every,
                       void* q_out, void* k_pages, void* v_pages, int dtype, int n_tokens, int heads, int kv_heads, int key_dim,
                       int value_dim, int tiled_page_size, const float* bias, int normed, int queries_only, int64_t row_stride,
-                      const float* cos_sin, int rot_dims, int values_normed, hipStream_t stream);
+                      const float* cos_sin, int rot_dims, int values_normed, const MllStoreExtras* more, hipStream_t stream);
+
+// out[t][h] = o / sqrt(mean(o^2) + eps) * factor over the head's value_dim channels, o = maps[t][2 h] - lambda * maps[t][2 h + 1]:
+// maps float32, its heads map_stride elements apart ([n_tokens][2 * heads][map_stride]); out [n_tokens][heads][value_dim].
+int mll_attention_difference(const float* maps, int64_t map_stride, void* out, int dtype, int n_tokens, int heads, int value_dim,
+                             float lambda, float eps, float factor, hipStream_t stream);
 
 // Causal attention of every token over its request's pages: score_j = (q . k_j) * scale + bias[min(p - j, longest)][head]
 // (bias null: none; float32 [longest + 1][heads]) - slopes[head] * (p - j) (slopes null: none); softmax over j <= p
@@ -342,12 +376,13 @@ int mll_qk_norm_store(const float* qkv, int n_parts, int64_t part_stride, const 
 // With chunk > 0 (and no window) a query at p sees the keys from floor(p / chunk) * chunk on. With gate (float32, rows
 // gate_stride apart, one number a head) the head's result is multiplied by sigmoid(gate[t][head]); with gate_channels its
 // rows hold heads * value_dim numbers, one for every channel. softcap > 0: the scaled score becomes softcap *
-// tanh(score / softcap) before anything is added to it.
+// tanh(score / softcap) before anything is added to it. out_f32: out is float32 whatever dtype is.
 int mll_bias_attention(const void* q, const void* k_pages, const void* v_pages, const int32_t* block_table, int table_width,
                        const int32_t* seq_of_token, const int32_t* positions, const float* bias, int longest,
                        const float* sink, void* out, int64_t out_stride, int dtype, int n_tokens, int heads, int kv_heads,
                        int key_dim, int value_dim, int page_size, float scale, float out_scale, const float* slopes, int window,
-                       int chunk, const float* gate, int64_t gate_stride, float softcap, int gate_channels, hipStream_t stream);
+                       int chunk, const float* gate, int64_t gate_stride, float softcap, int gate_channels, int out_f32,
+                       hipStream_t stream);
 
 // ---- gated linear attention --------------------------------------------------------------------------------
 
@@ -477,36 +512,49 @@ int mll_rglru_scan(const float* proj, int64_t proj_stride, int x_at, const float
 // of z[t][0 .. experts), ties to the lower index; weights are the scores, divided by their sum with renormalize.
 // shared_at >= 0: shared_gate[t] = sigmoid(z[t][shared_at]).
 // groups > 0: the experts form that many equal groups of neighbours; a group's score is its largest, and only experts of
-// the `keep` best groups (ties: the lower) are chosen.
+// the `keep` best groups (ties: the lower) are chosen. With correction (null: none; float32 [experts]) score + correction
+// decides, over experts and over groups, and the weights are the scores as before. renormalize divides by the sum +
+// weight_eps; the weights are then multiplied by weight_scale.
 int mll_moe_route(const float* z, int64_t z_stride, int n_tokens, int experts, int top, int softmax_scores, int renormalize,
-                  int shared_at, int32_t* ids, float* weights, float* shared_gate, int groups, int keep, hipStream_t stream);
+                  int shared_at, int32_t* ids, float* weights, float* shared_gate, int groups, int keep, const float* correction,
+                  float weight_eps, float weight_scale, hipStream_t stream);
+
+// What an expert does between its products, and how many there are. activation: 0 SiLU, 1 gelu (erf), 2 gelu (tanh), each
+// act(g) * u with gated and act(u) without; 3 (gated only): g = min(g, limit), u = clamp(u, -limit, limit),
+// g * sigmoid(slope * g) * (u + 1). An id of `experts` or more names an expert without weights that returns its input.
+typedef struct MllExpertForm {
+    int gated;
+    int activation;
+    float limit;
+    float slope;
+    int experts;
+    int identity;       // how many such ids there are: ids lie below experts + identity
+} MllExpertForm;
 
 // act[t * top + n] = silu(Wg_e xs) * (Wu_e xs), e = ids[t][n], xs = x[t] * weights[t][n] rounded to `dtype`
 // (weight_on_input) or x[t]; gate_up [experts][2 * ff][width] with the gate rows first.
-// gated 0: gate_up is [experts][ff][width] and act = activation(Wu_e xs). activation: 0 SiLU, 1 gelu (erf), 2 gelu (tanh).
+// not gated: gate_up is [experts][ff][width] and act = activation(Wu_e xs). Pairs of an id that returns its input have no act.
 int mll_moe_gate_up(const void* x, const int32_t* ids, const float* weights, int top, const void* gate_up, void* act,
-                    int dtype, int n_tokens, int width, int ff, int weight_on_input, int gated, int activation,
+                    int dtype, int n_tokens, int width, int ff, int weight_on_input, const MllExpertForm* form,
                     hipStream_t stream);
 
-// out[n][t] = Wd_e act[t * top + n] (* weights[t][n] unless weight_on_input): float32 [top][n_tokens][width].
-int mll_moe_down(const void* act, const int32_t* ids, const float* weights, int top, const void* down, float* out, int dtype,
-                 int n_tokens, int width, int ff, int weight_on_input, hipStream_t stream);
-
-// The same for n_tokens tokens of an output whose parts hold part_tokens rows each (a launch for some of a step's tokens).
-int mll_moe_down_rows(const void* act, const int32_t* ids, const float* weights, int top, const void* down, float* out, int dtype,
-                      int n_tokens, int part_tokens, int width, int ff, int weight_on_input, hipStream_t stream);
+// out[n][t] = Wd_e act[t * top + n] (* weights[t][n] unless weight_on_input): float32, in parts of part_tokens rows
+// (part_tokens > n_tokens: a launch for some of a step's tokens); an id that returns its input gives x[t] * weights[t][n].
+int mll_moe_down(const void* x, const void* act, const int32_t* ids, const float* weights, int top, const void* down, float* out,
+                 int dtype, int n_tokens, int part_tokens, int width, int ff, int weight_on_input, const MllExpertForm* form,
+                 hipStream_t stream);
 
 // out[t] = factor[t] * (in[0][t] + in[1][t] + ...), float32; parts part_stride elements apart.
 int mll_scale_rows(const float* in, int n_parts, int64_t part_stride, const float* factor, float* out, int n_tokens, int width,
                    hipStream_t stream);
 
-// The same as mll_moe_gate_up and mll_moe_down together for many bfloat16 pairs: the pairs are sorted by expert (counts
-// [experts], offsets [experts + 1], order [n_tokens * top]: int32 scratch), their inputs gathered into `sorted`
+// The same as mll_moe_gate_up and mll_moe_down together for many bfloat16 pairs: the pairs are sorted by id (counts
+// [ids], offsets [ids + 1], order [n_tokens * top]: int32 scratch, ids = experts + identity), their inputs gathered into `sorted`
 // ([pairs][width]), and every expert multiplies its rows in tiles on the matrix units; `act` is [pairs][ff] scratch.
 // width and ff are multiples of 8.
 int mll_moe_grouped(const void* x, const int32_t* ids, const float* weights, int top, const void* gate_up, const void* down,
                     int32_t* counts, int32_t* offsets, int32_t* order, void* sorted, void* act, float* out, int n_tokens,
-                    int experts, int width, int ff, int weight_on_input, int gated, int activation, hipStream_t stream);
+                    int width, int ff, int weight_on_input, const MllExpertForm* form, hipStream_t stream);
 
 // mll_rglru_scan for steps with long portions: the recurrence in chunks of 64 tokens (every chunk walked from zero,
 // the state carried from chunk to chunk, every chunk walked again from its start), the same result but for the

@@ -3,7 +3,9 @@
 // Wd (act(Wg x) * (Wu x)), or has one inner weight, Wd act(Wu x); act is chosen by number (common.h).
 //
 // Choice: scores are sigmoid(z) or softmax(z) over the experts, the `top` largest are taken (ties: the lower
-// index), their weights are the scores, optionally divided by their sum. Everything float32.
+// index), their weights are the scores, optionally divided by their sum and multiplied by a factor. A correction a
+// expert may be added to the scores for the choice alone. Everything float32. Ids from the number of experts on name
+// experts without weights, which return their input: they are chosen like the others and cost no product.
 //
 // Experts, plain kernels: a workgroup takes one (token, choice) pair and a stretch of the expert's output rows; a
 // wave forms one output at a time with its lanes along the reduction (16-byte loads of the weight's row), so a
@@ -21,7 +23,8 @@ constexpr int kMaxTop = 16;
 __global__ void __launch_bounds__(64)
 moe_route_kernel(const float* __restrict__ z, int64_t z_stride, int n_tokens, int experts, int top, int softmax_scores,
                  int renormalize, int shared_at, int32_t* __restrict__ ids, float* __restrict__ weights,
-                 float* __restrict__ shared_gate, int groups, int keep) {
+                 float* __restrict__ shared_gate, int groups, int keep, const float* __restrict__ correction, float weight_eps,
+                 float weight_scale) {
     const int token = blockIdx.x * blockDim.x + threadIdx.x;
     if (token >= n_tokens) return;
     const float* row = z + static_cast<int64_t>(token) * z_stride;
@@ -31,6 +34,9 @@ moe_route_kernel(const float* __restrict__ z, int64_t z_stride, int n_tokens, in
         total = 0.0f;
         for (int e = 0; e < experts; ++e) total += expf(row[e] - peak);
     }
+    auto score = [&](int e) { return softmax_scores ? expf(row[e] - peak) / total : 1.0f / (1.0f + expf(-row[e])); };
+    // What decides: without a correction the logit itself, since the scores rise with the logits
+    auto deciding = [&](int e) { return correction ? score(e) + correction[e] : row[e]; };
     // Groups of neighbouring experts: a group counts as much as its best expert, and only the experts of the `keep`
     // best groups (ties: the lower group) can be chosen. A bit a group (at most 64).
     unsigned long long open_groups = ~0ull;
@@ -42,8 +48,8 @@ moe_route_kernel(const float* __restrict__ z, int64_t z_stride, int n_tokens, in
             float best_logit = 0.0f;
             for (int g = 0; g < groups; ++g) {
                 if ((open_groups >> g) & 1ull) continue;
-                float top_logit = row[g * group_size];
-                for (int e = 1; e < group_size; ++e) top_logit = fmaxf(top_logit, row[g * group_size + e]);
+                float top_logit = deciding(g * group_size);
+                for (int e = 1; e < group_size; ++e) top_logit = fmaxf(top_logit, deciding(g * group_size + e));
                 if (best_group < 0 || top_logit > best_logit) {
                     best_group = g;
                     best_logit = top_logit;
@@ -62,19 +68,19 @@ moe_route_kernel(const float* __restrict__ z, int64_t z_stride, int n_tokens, in
             bool used = false;
             for (int m = 0; m < n; ++m) used = used || chosen[m] == e;
             if (used || (groups > 0 && !((open_groups >> (e / group_size)) & 1ull))) continue;
-            // the scores rise with the logits, so the largest logit is the largest score; a logit that is no number is never larger
-            if (best < 0 || row[e] > best_logit) {
+            const float value = deciding(e);     // one that is no number is never larger
+            if (best < 0 || value > best_logit) {
                 best = e;
-                best_logit = row[e];
+                best_logit = value;
             }
         }
         chosen[n] = best;
-        taken[n] = softmax_scores ? expf(best_logit - peak) / total : 1.0f / (1.0f + expf(-best_logit));
+        taken[n] = score(best);
         sum += taken[n];
     }
     for (int n = 0; n < top; ++n) {
         ids[static_cast<int64_t>(token) * top + n] = chosen[n];
-        weights[static_cast<int64_t>(token) * top + n] = renormalize ? taken[n] / sum : taken[n];
+        weights[static_cast<int64_t>(token) * top + n] = (renormalize ? taken[n] / (sum + weight_eps) : taken[n]) * weight_scale;
     }
     if (shared_at >= 0 && shared_gate != nullptr) shared_gate[token] = 1.0f / (1.0f + expf(-row[shared_at]));
 }
@@ -106,7 +112,7 @@ template <int PER>
 __global__ void __launch_bounds__(kWave)
 moe_route_wave_kernel(const float* __restrict__ z, int64_t z_stride, int experts, int top, int softmax_scores, int renormalize,
                       int shared_at, int32_t* __restrict__ ids, float* __restrict__ weights, float* __restrict__ shared_gate,
-                      int groups, int keep) {
+                      int groups, int keep, const float* __restrict__ correction, float weight_eps, float weight_scale) {
     const int token = blockIdx.x, lane = threadIdx.x;
     const float* row = z + static_cast<int64_t>(token) * z_stride;
     float logit[PER];
@@ -128,6 +134,19 @@ moe_route_wave_kernel(const float* __restrict__ z, int64_t z_stride, int experts
         for (int n = 0; n < PER; ++n)
             if (lane + n * kWave < experts) part += expf(logit[n] - peak);
         total = wave_sum(part);
+    }
+    auto score_of = [&](float value) { return softmax_scores ? expf(value - peak) / total : 1.0f / (1.0f + expf(-value)); };
+    // What decides over experts and groups: the logits (the scores rise with them), or the scores with their correction;
+    // the scores themselves are kept for the weights.
+    float score[PER];
+#pragma unroll
+    for (int n = 0; n < PER; ++n) {
+        score[n] = correction != nullptr ? score_of(logit[n]) : 0.0f;
+        if (correction != nullptr) {
+            const int e = lane + n * kWave;
+            const float value = e < experts ? score[n] + correction[e] : -INFINITY;
+            logit[n] = value != value ? -INFINITY : value;
+        }
     }
     if (groups > 0 && keep < groups) {
         // lane g learns group g's largest logit; then the best `keep` groups are opened, one after the other
@@ -165,7 +184,16 @@ moe_route_wave_kernel(const float* __restrict__ z, int64_t z_stride, int experts
 #pragma unroll
         for (int n = 0; n < PER; ++n)
             if (lane + n * kWave == best.index) free_to_take[n] = false;
-        const float taken = softmax_scores ? expf(best.value - peak) / total : 1.0f / (1.0f + expf(-best.value));
+        float taken = 0.0f;
+        if (correction != nullptr) {
+#pragma unroll
+            for (int n = 0; n < PER; ++n) {
+                const float theirs = __shfl(score[n], best.index % kWave, kWave);
+                if (best.index / kWave == n) taken = theirs;
+            }
+        } else {
+            taken = score_of(best.value);
+        }
         sum += taken;
         if (lane == choice) {
             my_weight = taken;
@@ -174,7 +202,7 @@ moe_route_wave_kernel(const float* __restrict__ z, int64_t z_stride, int experts
     }
     if (lane < top) {
         ids[static_cast<int64_t>(token) * top + lane] = my_id;
-        weights[static_cast<int64_t>(token) * top + lane] = renormalize ? my_weight / sum : my_weight;
+        weights[static_cast<int64_t>(token) * top + lane] = (renormalize ? my_weight / (sum + weight_eps) : my_weight) * weight_scale;
     }
     if (lane == 0 && shared_at >= 0 && shared_gate != nullptr) shared_gate[token] = 1.0f / (1.0f + expf(-row[shared_at]));
 }
@@ -273,17 +301,19 @@ constexpr int kExpertWaves = 4;
 constexpr int kExpertRowsAWave = 8;     // outputs a wave forms one after the other
 constexpr int kExpertRowsABlock = kExpertWaves * kExpertRowsAWave;
 
-// act[pair][f] = silu(Wg_e[f] . xs) * (Wu_e[f] . xs), xs = x[token] * weight[pair] rounded to T (the weight
+// act[pair][f] = act(Wg_e[f] . xs) * (Wu_e[f] . xs), or another gated form (common.h), xs = x[token] * weight[pair] rounded to T (the weight
 // multiplies the expert's input) or x[token] (weight_on_input 0). gate_up: [experts][2 * ff][width], gate rows first.
 template <typename T>
 __global__ void __launch_bounds__(kExpertWaves * kWave)
 moe_gate_up_kernel(const T* __restrict__ x, const int32_t* __restrict__ ids, const float* __restrict__ weights, int top,
-                   const T* __restrict__ gate_up, T* __restrict__ act, int width, int ff, int weight_on_input, int gated,
-                   int activation) {
+                   const T* __restrict__ gate_up, T* __restrict__ act, int width, int ff, int weight_on_input,
+                   MllExpertForm form) {
     extern __shared__ float xs[];
     const int pair = blockIdx.y;
     const int token = pair / top;
     const int expert = ids[pair];
+    if (expert >= form.experts) return;      // it returns its input (the same for every thread of the workgroup)
+    const int gated = form.gated, activation = form.activation;
     const float factor = weight_on_input ? weights[pair] : 1.0f;
     for (int c = threadIdx.x; c < width; c += blockDim.x)
         xs[c] = to_float(from_float<T>(to_float(x[static_cast<int64_t>(token) * width + c]) * factor));
@@ -316,8 +346,9 @@ moe_gate_up_kernel(const T* __restrict__ x, const int32_t* __restrict__ ids, con
         float sums[4];
         rows_dot4<T>(rows, xs, width, lane, sums);
         if (lane == 0) {
-            act[static_cast<int64_t>(pair) * ff + f] = from_float<T>(activate(sums[0], activation) * sums[1]);
-            if (f + 1 < ff) act[static_cast<int64_t>(pair) * ff + f + 1] = from_float<T>(activate(sums[2], activation) * sums[3]);
+            act[static_cast<int64_t>(pair) * ff + f] = from_float<T>(gated_value(sums[0], sums[1], activation, form.limit, form.slope));
+            if (f + 1 < ff)
+                act[static_cast<int64_t>(pair) * ff + f + 1] = from_float<T>(gated_value(sums[2], sums[3], activation, form.limit, form.slope));
         }
     }
 }
@@ -326,12 +357,19 @@ moe_gate_up_kernel(const T* __restrict__ x, const int32_t* __restrict__ ids, con
 // partial sums that the reader adds in order. down: [experts][width][ff].
 template <typename T>
 __global__ void __launch_bounds__(kExpertWaves * kWave)
-moe_down_kernel(const T* __restrict__ act, const int32_t* __restrict__ ids, const float* __restrict__ weights, int top,
-                const T* __restrict__ down, float* __restrict__ out, int n_tokens, int width, int ff, int weight_on_input) {
+moe_down_kernel(const T* __restrict__ x, const T* __restrict__ act, const int32_t* __restrict__ ids,
+                const float* __restrict__ weights, int top, const T* __restrict__ down, float* __restrict__ out, int n_tokens,
+                int width, int ff, int weight_on_input, int experts) {
     extern __shared__ float as[];
     const int pair = blockIdx.y;
     const int token = pair / top, choice = pair % top;
     const int expert = ids[pair];
+    if (expert >= experts) {        // the input itself times the weight, this workgroup's stretch of it
+        const int c = blockIdx.x * kExpertRowsABlock + threadIdx.x;
+        if (threadIdx.x < kExpertRowsABlock && c < width)
+            out[(static_cast<int64_t>(choice) * n_tokens + token) * width + c] = to_float(x[static_cast<int64_t>(token) * width + c]) * weights[pair];
+        return;
+    }
     for (int c = threadIdx.x; c < ff; c += blockDim.x) as[c] = to_float(act[static_cast<int64_t>(pair) * ff + c]);
     __syncthreads();
     const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
@@ -409,14 +447,21 @@ moe_order_kernel(const int32_t* __restrict__ ids, int n_pairs, int experts, cons
     }
 }
 
-// sorted[row] = x[token of order[row]] (* weight of the pair), rounded to bfloat16.
+// sorted[row] = x[token of order[row]] (* weight of the pair), rounded to bfloat16. The pairs of ids that return their
+// input stand behind the experts' and go straight to the result.
 __global__ void __launch_bounds__(256)
-moe_gather_kernel(const bf16* __restrict__ x, const int32_t* __restrict__ order, const float* __restrict__ weights, int top,
-                  bf16* __restrict__ sorted, int width, int weight_on_input) {
+moe_gather_kernel(const bf16* __restrict__ x, const int32_t* __restrict__ order, const int32_t* __restrict__ ids,
+                  const float* __restrict__ weights, int top, bf16* __restrict__ sorted, float* __restrict__ out, int n_tokens,
+                  int width, int weight_on_input, int experts) {
     const int row = blockIdx.x;
     const int pair = order[row];
-    const float factor = weight_on_input ? weights[pair] : 1.0f;
     const bf16* from = x + static_cast<int64_t>(pair / top) * width;
+    if (ids[pair] >= experts) {
+        float* whole = out + (static_cast<int64_t>(pair % top) * n_tokens + pair / top) * width;
+        for (int c = threadIdx.x; c < width; c += blockDim.x) whole[c] = to_float(from[c]) * weights[pair];
+        return;
+    }
+    const float factor = weight_on_input ? weights[pair] : 1.0f;
     bf16* to = sorted + static_cast<int64_t>(row) * width;
     for (int c = threadIdx.x; c < width; c += blockDim.x) to[c] = from_float<bf16>(to_float(from[c]) * factor);
 }
@@ -425,14 +470,15 @@ constexpr int kGroupRows = 128, kGroupCols = 128, kGroupStep = 64, kGroupPad = 7
 
 // FORM 2: w is [experts][n_out][k] and out (bfloat16 [pairs][n_out], sorted order) gets activation(product).
 // FORM 1 (GATED): w is [experts][2 * n_half][k] (gate rows, then up rows); a tile holds 64 gate rows and the 64 up rows that
-// belong to them, and out (bfloat16 [pairs][n_half], sorted order) gets silu(gate) * up. Otherwise w is
+// belong to them, and out (bfloat16 [pairs][n_half], sorted order) gets act(gate) * up or another gated form. Otherwise w is
 // [experts][n_out][k] and out (float32 [top][n_tokens][n_out]) gets the product at the pair's token and choice,
 // times the pair's weight unless that multiplied the input.
 template <int FORM>
 __global__ void __launch_bounds__(256)
 moe_grouped_kernel(const bf16* __restrict__ a, const bf16* __restrict__ w, const int32_t* __restrict__ offsets,
-                   const int32_t* __restrict__ order, const float* __restrict__ weights, int experts, int n_out, int k,
-                   void* __restrict__ out, int top, int n_tokens, int weight_on_input, int activation) {
+                   const int32_t* __restrict__ order, const float* __restrict__ weights, int n_out, int k,
+                   void* __restrict__ out, int top, int n_tokens, int weight_on_input, MllExpertForm form) {
+    const int experts = form.experts, activation = form.activation;
     constexpr bool GATED = FORM == 1;
     __shared__ __attribute__((aligned(16))) bf16 a_tile[kGroupRows * kGroupPad];
     __shared__ __attribute__((aligned(16))) bf16 w_tile[kGroupCols * kGroupPad];
@@ -534,7 +580,7 @@ moe_grouped_kernel(const bf16* __restrict__ a, const bf16* __restrict__ w, const
                 for (int i = 0; i < 4; ++i) {
                     const int column = col0 + wn * 32 + nt * 16 + quad * 4 + i;
                     const float g = acc[mt][nt][i], u = acc[mt][nt + 2][i];
-                    if (column < n_out) to[column] = from_float<bf16>(activate(g, activation) * u);
+                    if (column < n_out) to[column] = from_float<bf16>(gated_value(g, u, activation, form.limit, form.slope));
                 }
         } else if (FORM == 2) {
             bf16* to = static_cast<bf16*>(out) + static_cast<int64_t>(first_row + row) * n_out;
@@ -567,7 +613,8 @@ using namespace mll;
 extern "C" {
 
 int mll_moe_route(const float* z, int64_t z_stride, int n_tokens, int experts, int top, int softmax_scores, int renormalize,
-                  int shared_at, int32_t* ids, float* weights, float* shared_gate, int groups, int keep, hipStream_t stream) {
+                  int shared_at, int32_t* ids, float* weights, float* shared_gate, int groups, int keep, const float* correction,
+                  float weight_eps, float weight_scale, hipStream_t stream) {
     MLL_REQUIRE(n_tokens >= 0 && experts > 0 && top > 0 && top <= experts, "moe_route: 1 <= top <= experts");
     MLL_REQUIRE(top <= (experts <= 4 * kWave ? kWave : kMaxTop),
                 "moe_route: at most 64 experts a token (16 where there are more than 256 experts)");
@@ -578,22 +625,31 @@ int mll_moe_route(const float* z, int64_t z_stride, int n_tokens, int experts, i
     if (n_tokens == 0) return 0;
 #define MLL_ROUTE_WAVE(PER)                                                                                                  \
     moe_route_wave_kernel<PER><<<n_tokens, kWave, 0, stream>>>(z, z_stride, experts, top, softmax_scores, renormalize, shared_at, \
-                                                              ids, weights, shared_gate, groups, keep)
+                                                              ids, weights, shared_gate, groups, keep, correction,          \
+                                                              weight_eps, weight_scale)
     if (experts <= kWave) MLL_ROUTE_WAVE(1);
     else if (experts <= 2 * kWave) MLL_ROUTE_WAVE(2);
     else if (experts <= 4 * kWave) MLL_ROUTE_WAVE(4);
     else
         moe_route_kernel<<<(n_tokens + 63) / 64, 64, 0, stream>>>(z, z_stride, n_tokens, experts, top, softmax_scores, renormalize,
-                                                                shared_at, ids, weights, shared_gate, groups, keep);
+                                                                shared_at, ids, weights, shared_gate, groups, keep, correction,
+                                                                weight_eps, weight_scale);
 #undef MLL_ROUTE_WAVE
     return check_launch("moe_route");
 }
 
+static int check_form(const MllExpertForm* form, const char* who) {
+    if (form == nullptr || form->experts <= 0 || form->identity < 0) return fail(std::string(who) + ": a form with at least one expert");
+    if (form->activation < 0 || form->activation > (form->gated ? 3 : 2)) return fail(std::string(who) + ": 0 SiLU, 1 gelu (erf), 2 gelu (tanh), 3 clamped (gated)");
+    if (form->activation == 3 && !(form->limit > 0.0f)) return fail(std::string(who) + ": the limit must be positive");
+    return 0;
+}
+
 int mll_moe_gate_up(const void* x, const int32_t* ids, const float* weights, int top, const void* gate_up, void* act,
-                    int dtype, int n_tokens, int width, int ff, int weight_on_input, int gated, int activation,
+                    int dtype, int n_tokens, int width, int ff, int weight_on_input, const MllExpertForm* form,
                     hipStream_t stream) {
     MLL_REQUIRE(n_tokens >= 0 && top > 0 && width > 0 && ff > 0, "moe_gate_up: sizes must be positive");
-    MLL_REQUIRE(activation >= 0 && activation <= 2, "moe_gate_up: 0 SiLU, 1 gelu (erf), 2 gelu (tanh)");
+    if (check_form(form, "moe_gate_up") != 0) return 1;
     MLL_REQUIRE(static_cast<int64_t>(n_tokens) * top < 65536, "moe_gate_up: too many (token, expert) pairs for one launch");
     MLL_REQUIRE(static_cast<size_t>(width) * sizeof(float) <= 64 * 1024, "moe_gate_up: rows wider than 16384 are not supported");
     if (n_tokens == 0) return 0;
@@ -601,23 +657,20 @@ int mll_moe_gate_up(const void* x, const int32_t* ids, const float* weights, int
     const size_t lds = static_cast<size_t>(width) * sizeof(float);
     if (dtype == kF32) {
         moe_gate_up_kernel<float><<<grid, kExpertWaves * kWave, lds, stream>>>(
-            static_cast<const float*>(x), ids, weights, top, static_cast<const float*>(gate_up), static_cast<float*>(act), width, ff, weight_on_input, gated, activation);
+            static_cast<const float*>(x), ids, weights, top, static_cast<const float*>(gate_up), static_cast<float*>(act), width, ff, weight_on_input, *form);
     } else if (dtype == kBF16) {
         moe_gate_up_kernel<bf16><<<grid, kExpertWaves * kWave, lds, stream>>>(
-            static_cast<const bf16*>(x), ids, weights, top, static_cast<const bf16*>(gate_up), static_cast<bf16*>(act), width, ff, weight_on_input, gated, activation);
+            static_cast<const bf16*>(x), ids, weights, top, static_cast<const bf16*>(gate_up), static_cast<bf16*>(act), width, ff, weight_on_input, *form);
     } else {
         return fail("moe_gate_up: unknown dtype");
     }
     return check_launch("moe_gate_up");
 }
 
-int mll_moe_down(const void* act, const int32_t* ids, const float* weights, int top, const void* down, float* out, int dtype,
-                 int n_tokens, int width, int ff, int weight_on_input, hipStream_t stream) {
-    return mll_moe_down_rows(act, ids, weights, top, down, out, dtype, n_tokens, n_tokens, width, ff, weight_on_input, stream);
-}
-
-int mll_moe_down_rows(const void* act, const int32_t* ids, const float* weights, int top, const void* down, float* out, int dtype,
-                      int n_tokens, int part_tokens, int width, int ff, int weight_on_input, hipStream_t stream) {
+int mll_moe_down(const void* x, const void* act, const int32_t* ids, const float* weights, int top, const void* down, float* out,
+                 int dtype, int n_tokens, int part_tokens, int width, int ff, int weight_on_input, const MllExpertForm* form,
+                 hipStream_t stream) {
+    if (check_form(form, "moe_down") != 0) return 1;
     MLL_REQUIRE(n_tokens >= 0 && top > 0 && width > 0 && ff > 0 && part_tokens >= n_tokens, "moe_down: sizes must be positive");
     MLL_REQUIRE(static_cast<int64_t>(n_tokens) * top < 65536, "moe_down: too many (token, expert) pairs for one launch");
     MLL_REQUIRE(static_cast<size_t>(ff) * sizeof(float) <= 64 * 1024, "moe_down: experts wider than 16384 are not supported");
@@ -626,10 +679,12 @@ int mll_moe_down_rows(const void* act, const int32_t* ids, const float* weights,
     const size_t lds = static_cast<size_t>(ff) * sizeof(float);
     if (dtype == kF32) {
         moe_down_kernel<float><<<grid, kExpertWaves * kWave, lds, stream>>>(
-            static_cast<const float*>(act), ids, weights, top, static_cast<const float*>(down), out, part_tokens, width, ff, weight_on_input);
+            static_cast<const float*>(x), static_cast<const float*>(act), ids, weights, top, static_cast<const float*>(down), out, part_tokens,
+            width, ff, weight_on_input, form->experts);
     } else if (dtype == kBF16) {
         moe_down_kernel<bf16><<<grid, kExpertWaves * kWave, lds, stream>>>(
-            static_cast<const bf16*>(act), ids, weights, top, static_cast<const bf16*>(down), out, part_tokens, width, ff, weight_on_input);
+            static_cast<const bf16*>(x), static_cast<const bf16*>(act), ids, weights, top, static_cast<const bf16*>(down), out, part_tokens,
+            width, ff, weight_on_input, form->experts);
     } else {
         return fail("moe_down: unknown dtype");
     }
@@ -647,31 +702,32 @@ int mll_scale_rows(const float* in, int n_parts, int64_t part_stride, const floa
 
 int mll_moe_grouped(const void* x, const int32_t* ids, const float* weights, int top, const void* gate_up, const void* down,
                     int32_t* counts, int32_t* offsets, int32_t* order, void* sorted, void* act, float* out, int n_tokens,
-                    int experts, int width, int ff, int weight_on_input, int gated, int activation, hipStream_t stream) {
-    MLL_REQUIRE(n_tokens > 0 && top > 0 && experts > 0 && width > 0 && ff > 0, "moe_grouped: sizes must be positive");
-    MLL_REQUIRE(activation >= 0 && activation <= 2, "moe_grouped: 0 SiLU, 1 gelu (erf), 2 gelu (tanh)");
+                    int width, int ff, int weight_on_input, const MllExpertForm* form, hipStream_t stream) {
+    MLL_REQUIRE(n_tokens > 0 && top > 0 && width > 0 && ff > 0, "moe_grouped: sizes must be positive");
+    if (check_form(form, "moe_grouped") != 0) return 1;
+    const int experts = form->experts, named = form->experts + form->identity;
     MLL_REQUIRE(width % 8 == 0 && ff % 8 == 0, "moe_grouped: widths must be multiples of 8");
     const int64_t pairs = static_cast<int64_t>(n_tokens) * top;
     MLL_REQUIRE(pairs < (1 << 30), "moe_grouped: too many (token, expert) pairs");
     const int n_pairs = static_cast<int>(pairs);
-    moe_count_kernel<<<experts, kWave, 0, stream>>>(ids, n_pairs, counts);
-    moe_order_kernel<<<experts, kWave, 0, stream>>>(ids, n_pairs, experts, counts, offsets, order);
-    moe_gather_kernel<<<n_pairs, 256, 0, stream>>>(static_cast<const bf16*>(x), order, weights, top, static_cast<bf16*>(sorted), width,
-                                                  weight_on_input);
+    moe_count_kernel<<<named, kWave, 0, stream>>>(ids, n_pairs, counts);
+    moe_order_kernel<<<named, kWave, 0, stream>>>(ids, n_pairs, named, counts, offsets, order);
+    moe_gather_kernel<<<n_pairs, 256, 0, stream>>>(static_cast<const bf16*>(x), order, ids, weights, top, static_cast<bf16*>(sorted), out,
+                                                  n_tokens, width, weight_on_input, experts);
     const int tiles = (n_pairs + kGroupRows - 1) / kGroupRows + experts;
     MLL_REQUIRE(tiles < 65536, "moe_grouped: too many tiles of rows for one launch");
-    if (gated) {
+    if (form->gated) {
         moe_grouped_kernel<1><<<dim3((ff + 63) / 64, tiles), 256, 0, stream>>>(
-            static_cast<const bf16*>(sorted), static_cast<const bf16*>(gate_up), offsets, order, weights, experts, ff, width, act, top,
-            n_tokens, weight_on_input, activation);
+            static_cast<const bf16*>(sorted), static_cast<const bf16*>(gate_up), offsets, order, weights, ff, width, act, top,
+            n_tokens, weight_on_input, *form);
     } else {
         moe_grouped_kernel<2><<<dim3((ff + kGroupCols - 1) / kGroupCols, tiles), 256, 0, stream>>>(
-            static_cast<const bf16*>(sorted), static_cast<const bf16*>(gate_up), offsets, order, weights, experts, ff, width, act, top,
-            n_tokens, weight_on_input, activation);
+            static_cast<const bf16*>(sorted), static_cast<const bf16*>(gate_up), offsets, order, weights, ff, width, act, top,
+            n_tokens, weight_on_input, *form);
     }
     moe_grouped_kernel<0><<<dim3((width + kGroupCols - 1) / kGroupCols, tiles), 256, 0, stream>>>(
-        static_cast<const bf16*>(act), static_cast<const bf16*>(down), offsets, order, weights, experts, width, ff, out, top, n_tokens,
-        weight_on_input, activation);
+        static_cast<const bf16*>(act), static_cast<const bf16*>(down), offsets, order, weights, width, ff, out, top, n_tokens,
+        weight_on_input, *form);
     return check_launch("moe_grouped");
 }
 

@@ -158,6 +158,39 @@ def rms_norm_after(h: torch.Tensor, delta: Optional[torch.Tensor], after_weight:
     return out
 
 
+DELTA_SOURCES = 4
+
+
+class _Deltas(ctypes.Structure):
+    _fields_ = [("source", ctypes.c_void_p * DELTA_SOURCES), ("parts", ctypes.c_int * DELTA_SOURCES), ("count", ctypes.c_int)]
+
+
+def rms_norm_sum(h: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype: torch.dtype, deltas: Sequence[torch.Tensor],
+                 rows: Optional[torch.Tensor] = None, write_h: bool = False) -> torch.Tensor:
+    """``rms_norm(v) * weight`` with ``v = h[rows]`` plus every tensor of ``deltas`` at those rows: float32 ``[tokens, width]``
+    or partial sums ``[parts, tokens, width]``, at most ``DELTA_SOURCES`` of them; with ``write_h`` ``v`` replaces ``h``."""
+    lib = library.load()
+    _device_tensor(h, "residual stream", torch.float32)
+    _device_tensor(weight, "norm weight", torch.float32)
+    _need(h.dim() == 2 and tuple(weight.shape) == (h.shape[1],), "rms_norm_sum weight must match the last dimension")
+    _need(1 <= len(deltas) <= DELTA_SOURCES, f"one to {DELTA_SOURCES} deltas")
+    given = _Deltas(count=len(deltas))
+    for index, delta in enumerate(deltas):
+        _device_tensor(delta, "delta", torch.float32)
+        _need(delta.dim() in (2, 3) and tuple(delta.shape[-2:]) == tuple(h.shape) and delta.shape[0] >= 1,
+              "deltas must have the residual stream's shape, perhaps in parts")
+        given.source[index] = delta.data_ptr()
+        given.parts[index] = delta.shape[0] if delta.dim() == 3 else 1
+    if rows is not None:
+        _device_tensor(rows, "row selection", torch.int32)
+        _need(not write_h, "cannot write h through a row selection")
+    n_rows = rows.shape[0] if rows is not None else h.shape[0]
+    out = torch.empty((n_rows, h.shape[1]), dtype=out_dtype, device=h.device)
+    _check(lib.mll_rms_norm_sum(_ptr(h), ctypes.byref(given), ctypes.c_int64(h.numel()), _ptr(rows), _ptr(weight), ctypes.c_float(eps),
+                                _ptr(out), _code(out_dtype), n_rows, h.shape[1], int(write_h), _stream()), lib)
+    return out
+
+
 def add_bias(values: torch.Tensor, bias: torch.Tensor) -> torch.Tensor:
     """``values[..., c] += bias[c]`` in place: float32 ``[rows, width]``, or partial sums ``[parts, rows, width]``, whose
     first part takes the bias."""
@@ -207,14 +240,15 @@ def residual_add(h: torch.Tensor, delta: torch.Tensor) -> torch.Tensor:
     return h
 
 
-def rope_table(positions: torch.Tensor, inv_freq: torch.Tensor) -> torch.Tensor:
-    """``[tokens, n_freq, 2]`` float32: cos and sin of ``position * inv_freq``, the angle taken in float64."""
+def rope_table(positions: torch.Tensor, inv_freq: torch.Tensor, factor: float = 1.0) -> torch.Tensor:
+    """``[tokens, n_freq, 2]`` float32: ``factor`` times cos and sin of ``position * inv_freq``, the angle taken in float64."""
     lib = library.load()
     _device_tensor(positions, "positions", torch.int32)
     _device_tensor(inv_freq, "inverse frequencies", torch.float64)
     _need(positions.dim() == 1 and inv_freq.dim() == 1 and inv_freq.shape[0] > 0, "rope_table takes [tokens] and [n_freq]")
     out = torch.empty((positions.shape[0], inv_freq.shape[0], 2), dtype=torch.float32, device=positions.device)
-    _check(lib.mll_rope_table(_ptr(positions), _ptr(inv_freq), inv_freq.shape[0], positions.shape[0], _ptr(out), _stream()), lib)
+    _check(lib.mll_rope_table(_ptr(positions), _ptr(inv_freq), inv_freq.shape[0], positions.shape[0], ctypes.c_double(factor), _ptr(out),
+                              _stream()), lib)
     return out
 
 
@@ -717,7 +751,7 @@ def gemm_bf16_split(x: torch.Tensor, weight: torch.Tensor, parts: int) -> torch.
 class _AttentionExtras(ctypes.Structure):
     _fields_ = [("bias", ctypes.c_void_p), ("longest", ctypes.c_int), ("sink", ctypes.c_void_p),
                 ("out_scale", ctypes.c_float), ("out_stride", ctypes.c_int64), ("chunk", ctypes.c_int), ("gate", ctypes.c_void_p),
-                ("gate_stride", ctypes.c_int64), ("softcap", ctypes.c_float), ("gate_channels", ctypes.c_int)]
+                ("gate_stride", ctypes.c_int64), ("softcap", ctypes.c_float), ("gate_channels", ctypes.c_int), ("out_f32", ctypes.c_int)]
 
 
 class AttentionExtras(NamedTuple):
@@ -726,7 +760,8 @@ class AttentionExtras(NamedTuple):
     softmax's denominator; a factor on the result; ``chunk``: a query at ``p`` sees the keys from ``floor(p / chunk) *
     chunk`` on (no window then); ``gate`` float32 ``[tokens, heads]`` (columns of a wider buffer allowed): a head's result
     is multiplied by ``sigmoid(gate)``; ``[tokens, heads * head_dim]``: every channel of the result by its own;
-    ``softcap`` c (0: none): the scaled score becomes ``c * tanh(score / c)`` before a bias is added."""
+    ``softcap`` c (0: none): the scaled score becomes ``c * tanh(score / c)`` before a bias is added. With extras the
+    result may be a float32 tensor (without gates a channel)."""
     bias: Optional[torch.Tensor] = None
     sink: Optional[torch.Tensor] = None
     out_scale: float = 1.0
@@ -771,7 +806,7 @@ def _extras_argument(extras: Optional[AttentionExtras], heads: int, head_dim: in
                                          extras.sink.data_ptr() if extras.sink is not None else None,
                                          float(extras.out_scale), stride, int(extras.chunk),
                                          extras.gate.data_ptr() if extras.gate is not None else None, gate_stride,
-                                         float(extras.softcap), int(gate_channels)))
+                                         float(extras.softcap), int(gate_channels), int(out.dtype == torch.float32)))
 
 
 def decode_splits(n_tokens: int, kv_heads: int, longest: int) -> int:
@@ -810,7 +845,8 @@ def paged_attention_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torc
         n_tokens = token_ids.shape[0]
     if out is None:
         out = torch.empty_like(q)
-    _need(out.is_cuda and out.dtype == q.dtype and out.shape == q.shape, "attention output must have the queries' shape and dtype")
+    _need(out.is_cuda and out.shape == q.shape and (out.dtype == q.dtype or (extras is not None and out.dtype == torch.float32)),
+          "attention output must have the queries' shape and dtype (or be float32, with extras)")
     extra = _extras_argument(extras, heads, head_dim, out)
     part_o = part_ml = None
     if n_splits > 1:
@@ -869,7 +905,8 @@ def paged_attention_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: tor
     _need(positions.shape[0] == q.shape[0], "positions must hold one entry per token")
     if out is None:
         out = torch.empty_like(q)
-    _need(out.is_cuda and out.dtype == q.dtype and out.shape == q.shape, "attention output must have the queries' shape and dtype")
+    _need(out.is_cuda and out.shape == q.shape and (out.dtype == q.dtype or (extras is not None and out.dtype == torch.float32)),
+          "attention output must have the queries' shape and dtype (or be float32, with extras)")
     extra = _extras_argument(extras, heads, head_dim, out)
     _need(extras is None or extras.bias is None or extras.bias.shape[0] <= prefill_bias_rows(), "the bias table has too many rows for the prefill kernel")
     _check(lib.mll_paged_attention_prefill_extra(_ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.shape[1],
@@ -1300,12 +1337,30 @@ def _parts_of(tensor: torch.Tensor, name: str) -> Tuple[int, int]:
     return 1, 0
 
 
+class _StoreExtras(ctypes.Structure):
+    _fields_ = [("stored_dim", ctypes.c_int), ("maps", ctypes.c_int), ("norm_turned", ctypes.c_int), ("taps", ctypes.c_void_p),
+                ("n_taps", ctypes.c_int), ("kept", ctypes.c_void_p), ("seq_of_token", ctypes.c_void_p), ("cu_tokens", ctypes.c_void_p),
+                ("slots", ctypes.c_void_p)]
+
+
+class Convolution(NamedTuple):
+    """A causal convolution over time on every column of a product's rows: ``taps`` float32 ``[columns, n]``, the last on the
+    token itself; ``kept`` float32 ``[slots, n - 1, columns]``, every request's newest inputs before the step, newest last
+    (``conv_keep`` brings them up to date after everything has read them; unused with one tap)."""
+    taps: torch.Tensor
+    kept: Optional[torch.Tensor]
+    seq_of_token: torch.Tensor
+    cu_tokens: torch.Tensor
+    slots: torch.Tensor
+
+
 def qk_norm_store(qkv: torch.Tensor, q_weight: Optional[torch.Tensor], k_weight: Optional[torch.Tensor], eps: float,
                   positions: torch.Tensor, slot_mapping: torch.Tensor, temp_coef: float, temp_every: int,
                   k_pages: torch.Tensor, v_pages: torch.Tensor, heads: int, kv_heads: int, key_dim: int, value_dim: int,
                   out_dtype: torch.dtype, tiled_page_size: int = 0, bias: Optional[torch.Tensor] = None,
                   normed: Optional[bool] = None, queries_only: bool = False, cos_sin: Optional[torch.Tensor] = None,
-                  further_columns: int = 0, values_normed: bool = False) -> torch.Tensor:
+                  further_columns: int = 0, values_normed: bool = False, stored_dim: int = 0, maps: int = 1,
+                  norm_turned: bool = False, convolution: Optional[Convolution] = None) -> torch.Tensor:
     """Norm of queries and keys over their head, the queries' factor by position, keys and values into their pages
     (``[page, position, kv_head, dim]``, or with ``tiled_page_size`` the pages of ``cache.layout`` with that many
     positions each); returns the queries ``[tokens, heads * key_dim]``. ``bias`` (one number a column of a row) is
@@ -1314,11 +1369,17 @@ def qk_norm_store(qkv: torch.Tensor, q_weight: Optional[torch.Tensor], k_weight:
     reads another's keys and values). With ``cos_sin`` (``rope_table``'s ``[tokens, n, 2]``) queries and keys are turned
     after their norm in their first ``2 n`` channels, channel ``i`` with ``i + n``. The rows may hold
     ``further_columns`` after the values (what another kernel reads from the same product). ``values_normed``: values are
-    divided by their root mean square over their head before they are stored."""
+    divided by their root mean square over their head before they are stored. ``norm_turned``: the norm of queries and keys
+    is that of the turned vectors. ``stored_dim`` (0: as they are): queries, keys and values are kept in rows of that width,
+    zeros behind. ``maps``: a key head holds that many keys of ``key_dim / maps`` channels side by side, and query head ``h``
+    has ``key_dim / maps`` channels that meet key ``h % maps``: it is written at that key's place with zeros at the others'.
+    ``convolution``: every column passes it before anything else."""
     lib = library.load()
     n_parts, part_stride = _parts_of(qkv, "q/k/v")
     n_tokens = qkv.shape[-2]
-    row_width = heads * key_dim if queries_only else (heads + kv_heads) * key_dim + kv_heads * value_dim
+    _need(maps >= 1 and key_dim % maps == 0 and heads % maps == 0, "a key head holds equal keys, every one for as many query heads")
+    query_dim = key_dim // maps
+    row_width = heads * query_dim if queries_only else heads * query_dim + kv_heads * (key_dim + value_dim)
     _need(qkv.shape[-1] == row_width + further_columns, "q/k/v rows have the wrong width")
     row_stride = ctypes.c_int64(qkv.shape[-1])
     rot_dims = 0
@@ -1334,7 +1395,29 @@ def qk_norm_store(qkv: torch.Tensor, q_weight: Optional[torch.Tensor], k_weight:
     if bias is not None:
         _device_tensor(bias, "projection bias", torch.float32)
         _need(tuple(bias.shape) == (row_width,), "one bias a column of a row")
-    q_out = torch.empty((n_tokens, heads * key_dim), dtype=out_dtype, device=qkv.device)
+    _need(stored_dim == 0 or stored_dim >= max(key_dim, value_dim), "heads are stored at least as wide as they are")
+    key_width, value_width = stored_dim or key_dim, stored_dim or value_dim
+    more = None
+    if stored_dim or maps > 1 or norm_turned or convolution is not None:
+        more = _StoreExtras(stored_dim=int(stored_dim), maps=int(maps), norm_turned=int(norm_turned))
+        if convolution is not None:
+            taps, kept = convolution.taps, convolution.kept
+            _device_tensor(taps, "convolution taps", torch.float32)
+            _need(taps.dim() == 2 and taps.shape[0] == row_width and taps.shape[1] >= 1 and n_parts == 1 and not queries_only,
+                  "a convolution has taps [columns of q, k and v, n] and reads whole rows")
+            if taps.shape[1] > 1:
+                _device_tensor(kept, "kept inputs", torch.float32)
+                _need(kept.dim() == 3 and tuple(kept.shape[1:]) == (taps.shape[1] - 1, row_width), "kept inputs are [slots, n - 1, columns]")
+            for name, index in (("request of every token", convolution.seq_of_token), ("token offsets", convolution.cu_tokens),
+                                ("state slots", convolution.slots)):
+                _device_tensor(index, name, torch.int32)
+            _need(convolution.seq_of_token.shape[0] >= n_tokens, "a request for every token")
+            more.taps, more.n_taps = taps.data_ptr(), taps.shape[1]
+            more.kept = kept.data_ptr() if taps.shape[1] > 1 else None
+            more.seq_of_token, more.cu_tokens = convolution.seq_of_token.data_ptr(), convolution.cu_tokens.data_ptr()
+            more.slots = convolution.slots.data_ptr()
+        more = ctypes.byref(more)
+    q_out = torch.empty((n_tokens, heads * key_width), dtype=out_dtype, device=qkv.device)
     if queries_only:
         _need(q_weight is None or (q_weight.is_cuda and q_weight.dtype == torch.float32 and tuple(q_weight.shape) == (key_dim,)),
               "the query norm weight must be float32 of the head's size")
@@ -1342,7 +1425,7 @@ def qk_norm_store(qkv: torch.Tensor, q_weight: Optional[torch.Tensor], k_weight:
                                      ctypes.c_float(eps), _ptr(positions), None, ctypes.c_float(temp_coef),
                                      int(temp_every), _ptr(q_out), None, None, _code(out_dtype), n_tokens,
                                      heads, kv_heads, key_dim, value_dim, 0, _ptr(bias), int(normed), 1, row_stride, _ptr(cos_sin),
-                                     rot_dims, 0, _stream()), lib)
+                                     rot_dims, 0, more, _stream()), lib)
         return q_out
     _device_tensor(slot_mapping, "slot mapping", torch.int32)
     _need(slot_mapping.shape[0] >= n_tokens, "a slot for every token")
@@ -1353,18 +1436,33 @@ def qk_norm_store(qkv: torch.Tensor, q_weight: Optional[torch.Tensor], k_weight:
     _device_tensor(k_pages, "key pages", out_dtype)
     _device_tensor(v_pages, "value pages", out_dtype)
     if tiled_page_size:
-        _need(key_dim == value_dim, "tiled pages hold keys and values of one width")
-        _check_pages(k_pages, v_pages, out_dtype, kv_heads, key_dim, tiled_page_size)
+        _need(key_width == value_width, "tiled pages hold keys and values of one width")
+        _check_pages(k_pages, v_pages, out_dtype, kv_heads, key_width, tiled_page_size)
     else:
-        _need(k_pages.dim() == 4 and tuple(k_pages.shape[2:]) == (kv_heads, key_dim), "key pages are [page, position, kv_head, key_dim]")
-        _need(v_pages.dim() == 4 and tuple(v_pages.shape[2:]) == (kv_heads, value_dim) and v_pages.shape[:2] == k_pages.shape[:2],
+        _need(k_pages.dim() == 4 and tuple(k_pages.shape[2:]) == (kv_heads, key_width), "key pages are [page, position, kv_head, key_dim]")
+        _need(v_pages.dim() == 4 and tuple(v_pages.shape[2:]) == (kv_heads, value_width) and v_pages.shape[:2] == k_pages.shape[:2],
               "value pages are [page, position, kv_head, value_dim]")
     _check(lib.mll_qk_norm_store(_ptr(qkv), n_parts, ctypes.c_int64(part_stride), _ptr(q_weight), _ptr(k_weight),
                                  ctypes.c_float(eps), _ptr(positions), _ptr(slot_mapping), ctypes.c_float(temp_coef),
                                  int(temp_every), _ptr(q_out), _ptr(k_pages), _ptr(v_pages), _code(out_dtype), n_tokens,
                                  heads, kv_heads, key_dim, value_dim, int(tiled_page_size), _ptr(bias), int(normed), 0,
-                                 row_stride, _ptr(cos_sin), rot_dims, int(values_normed), _stream()), lib)
+                                 row_stride, _ptr(cos_sin), rot_dims, int(values_normed), more, _stream()), lib)
     return q_out
+
+
+def attention_difference(maps: torch.Tensor, heads: int, value_dim: int, factor_on_second: float, eps: float, factor: float,
+                         out_dtype: torch.dtype) -> torch.Tensor:
+    """``maps`` float32 ``[tokens, 2 * heads * width]``: for every head two results side by side, of which the first
+    ``value_dim`` channels count. ``o = first - factor_on_second * second``, divided by its root mean square over the head and
+    multiplied by ``factor``: ``[tokens, heads * value_dim]``."""
+    lib = library.load()
+    _device_tensor(maps, "the maps' results", torch.float32)
+    _need(maps.dim() == 2 and maps.shape[1] % (2 * heads) == 0 and maps.shape[1] // (2 * heads) >= value_dim, "two results for every head")
+    out = torch.empty((maps.shape[0], heads * value_dim), dtype=out_dtype, device=maps.device)
+    _check(lib.mll_attention_difference(_ptr(maps), ctypes.c_int64(maps.shape[1] // (2 * heads)), _ptr(out), _code(out_dtype), maps.shape[0],
+                                        heads, value_dim, ctypes.c_float(factor_on_second), ctypes.c_float(eps), ctypes.c_float(factor),
+                                        _stream()), lib)
+    return out
 
 
 def bias_attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, block_table: torch.Tensor,
@@ -1377,7 +1475,7 @@ def bias_attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor
     itself and the ``window - 1`` keys before it; with ``chunk`` the keys from ``floor(p / chunk) * chunk`` on; with ``gate``
     (float32 ``[tokens, heads]``, columns of a wider buffer allowed) a head's result is multiplied by ``sigmoid(gate)``, with
     ``[tokens, heads * value_dim]`` every channel by its own; ``softcap`` c (0: none): the scaled score becomes ``c * tanh(score
-    / c)`` before anything is added to it; ``out`` may be columns of a wider buffer (its row stride is taken)."""
+    / c)`` before anything is added to it; ``out`` may be columns of a wider buffer (its row stride is taken), or float32."""
     lib = library.load()
     _device_tensor(q, "queries")
     n_tokens = q.shape[0]
@@ -1408,7 +1506,7 @@ def bias_attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor
     gate_stride, gate_channels = _gate_stride(gate, n_tokens, heads, value_dim)
     if out is None:
         out = torch.empty((n_tokens, heads * value_dim), dtype=q.dtype, device=q.device)
-    _need(out.is_cuda and out.dtype == q.dtype and out.dim() == 2 and tuple(out.shape) == (n_tokens, heads * value_dim)
+    _need(out.is_cuda and out.dtype in (q.dtype, torch.float32) and out.dim() == 2 and tuple(out.shape) == (n_tokens, heads * value_dim)
           and out.stride(1) == 1, "the output is [tokens, heads * value_dim] with unit column stride")
     _check(lib.mll_bias_attention(_ptr(q), _ptr(k_pages), _ptr(v_pages), _ptr(block_table), block_table.shape[1],
                                   _ptr(seq_of_token), _ptr(positions), _ptr(bias), longest, _ptr(sink),
@@ -1416,7 +1514,7 @@ def bias_attention(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor
                                   _code(q.dtype), n_tokens, heads, kv_heads, key_dim, value_dim, page_size,
                                   ctypes.c_float(scale), ctypes.c_float(out_scale), _ptr(slopes), int(window), int(chunk),
                                   ctypes.c_void_p(gate.data_ptr()) if gate is not None else None, ctypes.c_int64(gate_stride),
-                                  ctypes.c_float(softcap), int(gate_channels), _stream()), lib)
+                                  ctypes.c_float(softcap), int(gate_channels), int(out.dtype == torch.float32), _stream()), lib)
     return out
 
 
@@ -1829,11 +1927,14 @@ def router_logits(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
 
 
 def moe_route(z: torch.Tensor, experts: int, top: int, softmax_scores: bool = False, renormalize: bool = False,
-              shared_at: int = -1, groups: int = 0, keep: int = 0):
+              shared_at: int = -1, groups: int = 0, keep: int = 0, correction: Optional[torch.Tensor] = None,
+              weight_eps: float = 0.0, weight_scale: float = 1.0):
     """The ``top`` experts of every token from router logits ``z`` float32 ``[tokens, columns]`` (experts first):
     ``(ids int32 [tokens, top], weights float32 [tokens, top], sigmoid(z[:, shared_at]) or None)``. With ``groups``
     the experts form that many equal groups of neighbours, a group counts as its best expert, and only experts of the
-    ``keep`` best groups are chosen."""
+    ``keep`` best groups are chosen. ``correction`` float32 ``[experts]`` is added to the scores for the choice (of experts
+    and of groups) alone. ``renormalize`` divides the weights by their sum ``+ weight_eps``; then they are multiplied by
+    ``weight_scale``."""
     lib = library.load()
     _device_tensor(z, "router logits", torch.float32)
     _need(z.dim() == 2 and z.shape[1] >= experts and shared_at < z.shape[1], "router logits are [tokens, experts (+ gate)]")
@@ -1841,8 +1942,12 @@ def moe_route(z: torch.Tensor, experts: int, top: int, softmax_scores: bool = Fa
     ids = torch.empty((n_tokens, top), dtype=torch.int32, device=z.device)
     weights = torch.empty((n_tokens, top), dtype=torch.float32, device=z.device)
     shared = torch.empty((n_tokens,), dtype=torch.float32, device=z.device) if shared_at >= 0 else None
+    if correction is not None:
+        _device_tensor(correction, "correction of the scores", torch.float32)
+        _need(tuple(correction.shape) == (experts,), "one correction an expert")
     _check(lib.mll_moe_route(_ptr(z), ctypes.c_int64(z.shape[1]), n_tokens, experts, top, int(softmax_scores), int(renormalize),
-                             int(shared_at), _ptr(ids), _ptr(weights), _ptr(shared), int(groups), int(keep), _stream()), lib)
+                             int(shared_at), _ptr(ids), _ptr(weights), _ptr(shared), int(groups), int(keep), _ptr(correction),
+                             ctypes.c_float(weight_eps), ctypes.c_float(weight_scale), _stream()), lib)
     return ids, weights, shared
 
 
@@ -1852,15 +1957,25 @@ MOE_PAIRS_A_LAUNCH = 65535
 MOE_GROUPED_PAIRS = 64      # from this many (token, choice) pairs on, bfloat16 experts multiply their rows in tiles
 
 
+CLAMPED_GLU = "clamped_glu"     # g = min(g, limit), u = clamp(u, -limit, limit): g * sigmoid(slope * g) * (u + 1)
+EXPERT_ACTIVATIONS = {**ACTIVATIONS, CLAMPED_GLU: 3}
+
+
+class _ExpertForm(ctypes.Structure):
+    _fields_ = [("gated", ctypes.c_int), ("activation", ctypes.c_int), ("limit", ctypes.c_float), ("slope", ctypes.c_float),
+                ("experts", ctypes.c_int), ("identity", ctypes.c_int)]
+
+
 def moe_experts(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor,
                 weight_on_input: bool, out: Optional[torch.Tensor] = None, grouped: Optional[bool] = None, gated: bool = True,
-                activation: str = "silu") -> torch.Tensor:
+                activation: str = "silu", limit: float = 0.0, slope: float = 1.0, identity: int = 0) -> torch.Tensor:
     """Every (token, choice) pair through its expert's gated feed-forward: ``gate_up`` ``[experts, 2 * ff, width]``
     (gate rows first), ``down`` ``[experts, width, ff]``. Returns float32 ``[top, tokens, width]``, a part per choice,
     for the reader to add in order (``out``: at least that many leading parts of a larger buffer). ``grouped``: the
     pairs sorted by expert and multiplied in tiles on the matrix units (bfloat16, widths in steps of 8) instead of
     one reading of the expert's weights a pair; by default by the number of pairs. With ``gated`` false an expert is
-    ``down act(up x)`` and ``gate_up`` holds ``[experts, ff, width]``; ``activation`` is one of ``ACTIVATIONS``."""
+    ``down act(up x)`` and ``gate_up`` holds ``[experts, ff, width]``; ``activation`` is one of ``ACTIVATIONS``, or
+    ``clamped_glu`` with its ``limit`` and ``slope`` (gated). The ``identity`` ids after the experts' return their input."""
     lib = library.load()
     _device_tensor(x, "expert input")
     _device_tensor(gate_up, "experts' gate and up weights", x.dtype)
@@ -1871,8 +1986,11 @@ def moe_experts(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, gate_
     top = ids.shape[1]
     experts, inner_rows, _ = gate_up.shape
     ff = inner_rows // 2 if gated else inner_rows
-    _need(activation in ACTIVATIONS, f"unknown activation {activation!r}")
-    act_code = ACTIVATIONS[activation]
+    _need(activation in EXPERT_ACTIVATIONS and (gated or activation != CLAMPED_GLU), f"unknown activation {activation!r}")
+    _need(activation != CLAMPED_GLU or limit > 0.0, "the limit must be positive")
+    _need(identity >= 0, "the number of ids that return their input")
+    form = ctypes.byref(_ExpertForm(int(gated), EXPERT_ACTIVATIONS[activation], float(limit), float(slope), experts, int(identity)))
+    named = experts + identity
     _need(gate_up.shape[2] == width and tuple(down.shape) == (experts, width, ff) and tuple(ids.shape) == (n_tokens, top)
           and tuple(weights.shape) == (n_tokens, top), "the experts' weights, ids and weights do not fit the input")
     if out is None:
@@ -1884,12 +2002,12 @@ def moe_experts(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, gate_
         grouped = x.dtype == torch.bfloat16 and n_tokens * top >= MOE_GROUPED_PAIRS and width % 8 == 0 and ff % 8 == 0
     if grouped:
         _need(x.dtype == torch.bfloat16 and width % 8 == 0 and ff % 8 == 0, "the tiled experts take bfloat16 and widths in steps of 8")
-        scratch = torch.empty((2 * experts + 1 + n_tokens * top,), dtype=torch.int32, device=x.device)
-        counts, offsets, order = scratch[:experts], scratch[experts:2 * experts + 1], scratch[2 * experts + 1:]
+        scratch = torch.empty((2 * named + 1 + n_tokens * top,), dtype=torch.int32, device=x.device)
+        counts, offsets, order = scratch[:named], scratch[named:2 * named + 1], scratch[2 * named + 1:]
         in_order = torch.empty((n_tokens * top, width), dtype=x.dtype, device=x.device)
         _check(lib.mll_moe_grouped(_ptr(x), _ptr(ids), _ptr(weights), top, _ptr(gate_up), _ptr(down), ctypes.c_void_p(counts.data_ptr()),
                                    ctypes.c_void_p(offsets.data_ptr()), ctypes.c_void_p(order.data_ptr()), _ptr(in_order), _ptr(act),
-                                   _ptr(out), n_tokens, experts, width, ff, int(weight_on_input), int(gated), act_code, _stream()), lib)
+                                   _ptr(out), n_tokens, width, ff, int(weight_on_input), form, _stream()), lib)
         return out
     step = max(1, MOE_PAIRS_A_LAUNCH // top)       # tokens a launch: its grid has a row of workgroups a pair
     element = x.element_size()
@@ -1898,10 +2016,11 @@ def moe_experts(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, gate_
         here = dict(x=ctypes.c_void_p(x.data_ptr() + first * width * element), ids=ctypes.c_void_p(ids.data_ptr() + first * top * 4),
                     weights=ctypes.c_void_p(weights.data_ptr() + first * top * 4), act=ctypes.c_void_p(act.data_ptr() + first * top * ff * element))
         _check(lib.mll_moe_gate_up(here["x"], here["ids"], here["weights"], top, _ptr(gate_up), here["act"], _code(x.dtype), count, width, ff,
-                                   int(weight_on_input), int(gated), act_code, _stream()), lib)
+                                   int(weight_on_input), form, _stream()), lib)
         # the output keeps its rows n_tokens apart in every part: the launch writes its tokens' rows of each
-        _check(lib.mll_moe_down_rows(here["act"], here["ids"], here["weights"], top, _ptr(down), ctypes.c_void_p(out.data_ptr() + first * width * 4),
-                                     _code(x.dtype), count, n_tokens, width, ff, int(weight_on_input), _stream()), lib)
+        _check(lib.mll_moe_down(here["x"], here["act"], here["ids"], here["weights"], top, _ptr(down),
+                                ctypes.c_void_p(out.data_ptr() + first * width * 4), _code(x.dtype), count, n_tokens, width, ff,
+                                int(weight_on_input), form, _stream()), lib)
     return out
 
 

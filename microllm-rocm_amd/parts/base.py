@@ -113,6 +113,11 @@ class FeedForward(Part):
         """``[tokens, hidden]`` -> the delta for the residual stream, as a mixer's."""
         raise NotImplementedError
 
+    def forward_sums(self, x: torch.Tensor, ctx) -> list:
+        """The same delta as a list of tensors like ``forward``'s whose sum it is: what a feed-forward makes in several
+        products need not lie in one buffer."""
+        return [self.forward(x, ctx)]
+
 
 class Norm(Part):
     category = "norm"

@@ -18,20 +18,23 @@ import torch
 
 from .base import Part, Runtime, TensorDecl
 from .linear import Residual, UnscaledRows
-from .norm import NormedDelta
+from .norm import NormedDelta, SummedDelta
 from .registry import build_part, register_part
 from .spec import LayerSpec
 
 
 class Block:
     """One layer built from a ``LayerSpec``. ``forward`` returns the delta still to be added to ``h``."""
+    ffn_has_norm = True     # the feed-forward stands behind a norm of its own
 
     def __init__(self, spec: LayerSpec, runtime: Runtime):
         self.spec = spec
         self.mixer_norm = build_part("norm", spec.mixer_norm, runtime)
         self.mixer = build_part("mixer", spec.mixer, runtime)
-        if (spec.ffn is None) != (spec.ffn_norm is None):
+        if self.ffn_has_norm and (spec.ffn is None) != (spec.ffn_norm is None):
             raise ValueError("a layer has a feed-forward and its norm, or neither")
+        if not self.ffn_has_norm and spec.ffn_norm is not None:
+            raise ValueError("in this arrangement the feed-forward has no norm of its own")
         self.ffn_norm = build_part("norm", spec.ffn_norm, runtime) if spec.ffn_norm is not None else None
         self.ffn = build_part("ffn", spec.ffn, runtime) if spec.ffn is not None else None
         self.extra: Dict[str, Part] = {name: build_part(category, part_spec, runtime)
@@ -124,7 +127,24 @@ class SandwichNormBlock(Block):
         return pending
 
 
-_ARRANGEMENTS = {"pre_norm": PreNormBlock, "sandwich_norm": SandwichNormBlock}
+class ParallelSublayersBlock(Block):
+    """One norm that both sublayers read: ``h' = h + (Mixer(Norm(h)) + FFN(Norm(h)))``; a layer may have no feed-forward. What
+    the sublayers leave is handed on as a ``SummedDelta`` of their partial sums, which the norm that reads the stream next
+    adds in one kernel: no product adds into the stream itself here."""
+    ffn_has_norm = False
+
+    def first_norm_after(self, producer, rows, h):
+        return None         # both sublayers want the normed rows themselves
+
+    def forward(self, h, pending, ctx, cache, next_block=None):
+        x = self.mixer_norm.forward(h, delta=pending, write_h=True)
+        sums = [self.mixer.forward(x, ctx, cache)]
+        if self.ffn is not None:
+            sums += self.ffn.forward_sums(x, ctx)
+        return SummedDelta(sums)
+
+
+_ARRANGEMENTS = {"pre_norm": PreNormBlock, "sandwich_norm": SandwichNormBlock, "parallel_sublayers": ParallelSublayersBlock}
 
 
 def register_arrangement(name: str, block_class, replace: bool = False) -> None:

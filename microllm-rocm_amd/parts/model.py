@@ -15,7 +15,7 @@ from ..ops import kernels
 from .base import CacheNeed, MATRIX, Part, Runtime, TensorDecl
 from .block import Block, build_block
 from .linear import UnscaledRows, Weight, linear
-from .norm import NormedDelta
+from .norm import NormedDelta, SummedDelta
 from .registry import build_part, register_part
 from .spec import ModelSpec, PartSpec
 
@@ -177,7 +177,7 @@ class Model:
     def _add_to_stream(h: torch.Tensor, pending, rows: torch.Tensor):
         """``h + pending + rows`` before the next entry: a delta that is still to be normed takes the rows along, so
         that the norm which reads the stream next adds both in its one kernel; anything else is added here."""
-        if isinstance(pending, NormedDelta):
+        if isinstance(pending, (NormedDelta, SummedDelta)):
             return pending.with_extra(rows)
         if h.dim() != 2 or isinstance(pending, UnscaledRows):
             raise TypeError("rows join a single residual stream that no product has already summed and normed")

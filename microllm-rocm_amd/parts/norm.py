@@ -50,6 +50,25 @@ class NormedDelta:
         return joined
 
 
+class SummedDelta:
+    """What several sublayers add to the residual stream at once: tensors ``[tokens, hidden]`` or partial sums ``[parts, tokens,
+    hidden]``, each in a place of its own. The norm that reads the stream next adds them all in its kernel."""
+
+    def __init__(self, sources):
+        self.sources = [source if source.dtype == torch.float32 else source.to(torch.float32) for source in sources]
+
+    def with_extra(self, rows: torch.Tensor) -> "SummedDelta":
+        return SummedDelta([*self.sources, rows])
+
+    def resolved(self) -> torch.Tensor:
+        """The sum as one float32 tensor ``[tokens, hidden]`` (for observers, and for norms that take no several sources)."""
+        total = torch.zeros(self.sources[0].shape[-2:], dtype=torch.float32, device=self.sources[0].device)
+        for source in self.sources:
+            for part in (source if source.dim() == 3 else (source,)):
+                kernels.residual_add(total, part)
+        return total
+
+
 class RMSNorm(Norm):
     graph_safe = True
     def __init__(self, spec: PartSpec, runtime: Runtime):
@@ -84,6 +103,10 @@ class RMSNorm(Norm):
 
     def forward(self, h, delta=None, write_h=True, rows=None):
         dtype = self.runtime.dtype
+        if isinstance(delta, SummedDelta):
+            if self.groups == 1 and len(delta.sources) <= kernels.DELTA_SOURCES:
+                return kernels.rms_norm_sum(h, self.weight, self.eps, dtype, delta.sources, rows=rows, write_h=write_h and rows is None)
+            delta = delta.resolved()
         if self.groups != (delta.groups if isinstance(delta, NormedDelta) else 1):
             # the sum's own norm has other runs than the delta's (or a plain delta joins a norm in groups): the sum first
             keeps = write_h and rows is None
@@ -118,6 +141,8 @@ class Unnormed(Norm):
 
     def forward(self, h, delta=None, write_h=True, rows=None):
         dtype = self.runtime.dtype
+        if isinstance(delta, SummedDelta):
+            delta = delta.resolved()
         if delta is not None and not isinstance(delta, NormedDelta):
             delta = delta.to(torch.float32)
             if not write_h:

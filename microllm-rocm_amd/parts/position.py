@@ -9,7 +9,10 @@ shared by the layers whose encoding has the same parameters; the attention
 mixer's fused kernels apply the rotation. With ``scaling_factor`` every rate is
 divided by that number (positions stretched linearly). With ``scaling_bands``
 (``factor``, ``low``, ``high``, ``original``) only slow rates are divided by the
-factor (``stretched_by_bands``).
+factor (``stretched_by_bands``). With ``scaling_ramp`` (``factor``, ``original``,
+``fast``, ``slow``, ``magnitude_slope``) slow pairs' rates are divided by the
+factor along a ramp over the pairs (``stretched_by_ramp``), and what is turned is
+multiplied by ``magnitude_slope * ln(factor) + 1``: the table's cos and sin are.
 
 ``rope_neighbours`` pairs channel ``2i`` with ``2i + 1`` instead. Moving channel
 ``2i`` to ``i`` and ``2i + 1`` to ``i + d/2`` makes it the split-half rule, and a
@@ -40,6 +43,23 @@ def stretched_by_bands(rates: torch.Tensor, factor: float, low: float, high: flo
     return torch.where(turns < low, rates / factor, torch.where(turns > high, rates, mixed))
 
 
+def stretched_by_ramp(rates: torch.Tensor, base: float, factor: float, original: float, fast: float, slow: float) -> torch.Tensor:
+    """Rates ``base^(-2i/n)`` (float64, ``n / 2`` of them) of which those of pairs that turn ``slow`` times or less over
+    ``original`` positions are divided by ``factor``, those of pairs that turn ``fast`` times or more stay, and between the
+    two the stretched and the plain rate are blended, linearly in the pair's number ``i``. A pair that turns ``t`` times has
+    the number ``n ln(original / (2 pi t)) / (2 ln base)``; the ramp's ends are rounded outwards to whole numbers and kept
+    within ``0 .. n - 1``."""
+    n = 2 * rates.shape[0]
+
+    def pair_that_turns(times: float) -> float:
+        return n * math.log(original / (2.0 * math.pi * times)) / (2.0 * math.log(base))
+
+    low = max(math.floor(pair_that_turns(fast)), 0)
+    high = min(math.ceil(pair_that_turns(slow)), n - 1)
+    ramp = ((torch.arange(n // 2, dtype=rates.dtype) - low) / max(high - low, 0.001)).clamp(0.0, 1.0)
+    return rates / factor * ramp + rates * (1.0 - ramp)
+
+
 class RopeSplitHalf(PositionEncoding):
     graph_safe = True
     fused_split_half = True
@@ -60,13 +80,19 @@ class RopeSplitHalf(PositionEncoding):
         self.scaling_bands = tuple(float(bands[key]) for key in ("factor", "low", "high", "original")) if bands is not None else None
         if self.scaling_bands is not None:
             rates = stretched_by_bands(rates, *self.scaling_bands)
+        ramp = spec.params.get("scaling_ramp")
+        self.scaling_ramp = tuple(float(ramp[key]) for key in ("factor", "original", "fast", "slow")) if ramp is not None else None
+        self.magnitude = 1.0        # of what is turned
+        if self.scaling_ramp is not None:
+            rates = stretched_by_ramp(rates, self.theta, *self.scaling_ramp)
+            self.magnitude = float(ramp.get("magnitude_slope", 0.0)) * math.log(self.scaling_ramp[0]) + 1.0
         self.inv_freq = rates.to(runtime.device)
 
     def table(self, ctx) -> torch.Tensor:
         """``[tokens, rotary_dim / 2, 2]`` float32: cos and sin for the step's tokens."""
-        key = ("rope_split_half", self.theta, self.rotary_dim, self.scaling_factor, self.scaling_bands)
+        key = ("rope_split_half", self.theta, self.rotary_dim, self.scaling_factor, self.scaling_bands, self.scaling_ramp, self.magnitude)
         if key not in ctx.memo:
-            ctx.memo[key] = kernels.rope_table(ctx.positions, self.inv_freq)
+            ctx.memo[key] = kernels.rope_table(ctx.positions, self.inv_freq, self.magnitude)
         return ctx.memo[key]
 
 
