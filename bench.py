@@ -155,6 +155,27 @@ def mapedra_config(size: dict):
                          embedding_scale=width ** 0.5)
 
 
+def zuluvik_config(size: dict):
+    """A Zuluvik configuration of the given layer sizes: layers in turn a differential attention (the model's heads and
+    key/value heads, two maps of half the head size each, values of the whole, four taps), a rotary attention (the same
+    heads of the whole head size, half of every head turned), a latent attention (heads of 96 unrotated and 64 rotated
+    query/key dims and 128 value dims, cached rows of 192 + 64 elements, as Kalevik's) and a rotary attention; every layer
+    with 16 experts of a quarter of the feed-forward width and four places that return their input, four a token out of
+    the best two of five groups, and a shared expert of half of it. Every layer has weights of its own."""
+    from microllm_rocm_amd.config.zuluvik import (DifferentialAttentionConfig, ExpertConfig, LatentAttentionConfig, MoeMlpConfig,
+                                                  RampScalingConfig, RotaryAttentionConfig, RotationConfig, ZuluvikConfig, ZuluvikLayerConfig)
+    width, heads, kv_heads, dim, ff = size["width"], size["heads"], size["kv_heads"], size["head_dim"], size["ff"]
+    scaling = RampScalingConfig(factor=16.0, original=8192.0, fast=24.0, slow=1.5)
+    differential = DifferentialAttentionConfig(heads=heads, kv_heads=kv_heads, dim=dim // 2, vdim=dim, conv=4, diff=0.7, scale=(dim // 2) ** -0.5)
+    rotary = RotaryAttentionConfig(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, scale=dim ** -0.5, rot=RotationConfig(1e6, dim // 2, scaling))
+    latent = LatentAttentionConfig(heads=heads, dim=96, rot_dim=64, vdim=dim, kv_rank=192, scale=160 ** -0.5, rot=RotationConfig(1e6, 64, scaling))
+    moe = MoeMlpConfig(experts=16, top=4, expert=ExpertConfig(ff // 4, 7.0), identity=4, groups=5, keep_groups=2, scale=2.5,
+                       shared=ExpertConfig(ff // 2, 7.0))
+    kinds = (("attention", differential), ("attention_2", rotary), ("latent_attention", latent), ("attention_2", rotary))
+    layers = [ZuluvikLayerConfig(*kinds[index % 4], moe) for index in range(size["layers"])]
+    return ZuluvikConfig(vocab=DESIGN_VOCAB, width=width, norm_eps=1e-6, layers=tuple(layers), embedding_scale=width ** 0.5)
+
+
 def design_configs(size: dict, design: str = "siditar"):
     """The design's configuration at the given layer sizes and the Qwen2 configuration of equal width, heads, head size,
     feed-forward width, depth and vocabulary."""
@@ -173,6 +194,8 @@ def design_configs(size: dict, design: str = "siditar"):
     if design == "mapedra":     # beside the designs whose parts are most like its own (norms after sublayers; a linear attention)
         return {"mapedra": mapedra_config(size), "zabozen": zabozen_config(size), "siditar": design_configs(size, "siditar")["siditar"],
                 "qwen2": qwen2}
+    if design == "zuluvik":     # beside the designs whose parts are most like its own (latents and experts; a rotary attention)
+        return {"zuluvik": zuluvik_config(size), "kalevik": kalevik_config(size), "mapedra": mapedra_config(size), "qwen2": qwen2}
     from microllm_rocm_amd.config.siditar import (BiasAttentionConfig, DenseMlpConfig, LinearAttentionConfig,
                                                   ParallelMixerConfig, SiditarConfig, SiditarLayerConfig)
     left = BiasAttentionConfig(heads=size["heads"], kv_heads=size["kv_heads"], dim=size["head_dim"], vdim=size["head_dim"],
@@ -252,11 +275,11 @@ def main() -> int:
     parser.add_argument("--no-extras", action="store_true",
                         help="leave out what the default run adds to its line after the main figures: decoding on the 32-bit path "
                              "at batch 8 and the continuous-batching workload at Qwen2-0.5B sizes")
-    parser.add_argument("--design", default=None, choices=["siditar", "gupitar", "zabozen", "kalevik", "mapedra"],
+    parser.add_argument("--design", default=None, choices=["siditar", "gupitar", "zabozen", "kalevik", "mapedra", "zuluvik"],
                         help="instead of the default workload: prefill and decode throughput of this design beside Qwen2 at equal "
                              "layer sizes (--design-sizes), random weights; --batch, --context, --prefill-tokens, --steps apply")
     parser.add_argument("--design-sizes", default="1k,2k,4k", help="of " + ", ".join(sorted(DESIGN_SIZES)))
-    parser.add_argument("--design-only", default=None, choices=["siditar", "gupitar", "zabozen", "kalevik", "mapedra", "qwen2"], help="one of the designs alone (profiles)")
+    parser.add_argument("--design-only", default=None, choices=["siditar", "gupitar", "zabozen", "kalevik", "mapedra", "zuluvik", "qwen2"], help="one of the designs alone (profiles)")
     args = parser.parse_args()
     if args.gpus != 1:
         print(f"bench.py measures one GPU; --gpus {args.gpus} is not supported (this engine runs on a single MI355X)")

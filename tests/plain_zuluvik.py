@@ -183,7 +183,9 @@ def moe(a: torch.Tensor, tensors, prefix: str, mlp: Mapping, margins: Optional[l
         took = weight[:, e].nonzero()[:, 0]
         if len(took):
             out[took] += weight[took, e:e + 1] * clamped_expert(a[took], tensors, f"{prefix}.e{e}", mlp["expert"]["limit"])
-    return out + clamped_expert(a, tensors, f"{prefix}.shared", mlp["shared"]["limit"])
+    if mlp.get("shared"):
+        out = out + clamped_expert(a, tensors, f"{prefix}.shared", mlp["shared"]["limit"])
+    return out
 
 
 MIXERS = {"attention": differential_attention, "attention_2": rotary_attention, "latent_attention": latent_attention}
