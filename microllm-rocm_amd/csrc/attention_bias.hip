@@ -145,8 +145,10 @@ qk_norm_store_kernel(const float* __restrict__ qkv, int n_parts, int64_t part_st
                      T* __restrict__ k_pages, T* __restrict__ v_pages, int heads, int kv_heads, int key_dim, int value_dim,
                      int tiled_page_size, const float* __restrict__ bias, int normed, int queries_only, int64_t row_stride,
                      const float* __restrict__ cos_sin, int rot_dims, int values_normed, int total, MllStoreExtras more) {
+    extern __shared__ float kept_sums[];        // a wave's vector, as it is before norm and turn: read from memory once
     const int vectors = queries_only ? heads : heads + 2 * kv_heads;
     const int vector = blockIdx.x * kNormStoreWaves + threadIdx.x / kWave;
+    float* own = kept_sums + threadIdx.x / kWave * max(key_dim, value_dim);
     if (vector >= total) return;
     const int token = vector / vectors;
     const int which = vector % vectors;
@@ -197,6 +199,7 @@ qk_norm_store_kernel(const float* __restrict__ qkv, int n_parts, int64_t part_st
     float squares = 0.0f;
     for (int c = lane; c < dim; c += kWave) {
         const float value = raw(c);
+        own[c] = value;
         float length = 1.0f;
         if (norm_turned && c < rot_dims) {      // a turned pair is as long as before, but for the factor within cos and sin
             const int pair = c < half ? c : c - half;
@@ -225,7 +228,11 @@ qk_norm_store_kernel(const float* __restrict__ qkv, int n_parts, int64_t part_st
     const int64_t page = tiled ? slot / tiled_page_size : 0;
     const int in_page = tiled ? slot % tiled_page_size : 0;
     auto normed_value = [&](float value, int c) { return norm ? (weight ? value * factor * weight[c] : value * factor) : value; };
-    auto prepared = [&](int c) { return norm_turned ? raw(c) : normed_value(raw(c), c); };      // what is turned
+    auto prepared = [&](int c) { return norm_turned ? own[c] : normed_value(own[c], c); };      // what is turned
+    // the wave's lanes read what its other lanes wrote
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
     const int kept_width = MORE ? (is_q || is_k ? key_width : value_width) : dim;
     for (int at = lane; at < kept_width; at += kWave) {
         const int c = at - place;
@@ -287,8 +294,10 @@ int mll_qk_norm_store(const float* qkv, int n_parts, int64_t part_stride, const 
     const int64_t total = static_cast<int64_t>(n_tokens) * (queries_only ? heads : heads + 2 * kv_heads);
     MLL_REQUIRE(total < (1ll << 31) - kNormStoreWaves, "qk_norm_store: too many rows for one launch");
     const int64_t blocks = (total + kNormStoreWaves - 1) / kNormStoreWaves;
+    const size_t lds = static_cast<size_t>(key_dim > value_dim ? key_dim : value_dim) * kNormStoreWaves * sizeof(float);
+    MLL_REQUIRE(lds <= 64 * 1024, "qk_norm_store: heads wider than 4096 are not supported");
 #define MLL_NORM_STORE(T, MORE)                                                                                               \
-    qk_norm_store_kernel<T, MORE><<<static_cast<unsigned>(blocks), kNormStoreWaves * kWave, 0, stream>>>(                         \
+    qk_norm_store_kernel<T, MORE><<<static_cast<unsigned>(blocks), kNormStoreWaves * kWave, lds, stream>>>(                       \
         qkv, n_parts, part_stride, q_weight, k_weight, eps, positions, slot_mapping, temp_coef, temp_every, static_cast<T*>(q_out), \
         static_cast<T*>(k_pages), static_cast<T*>(v_pages), heads, kv_heads, key_dim, value_dim, tiled_page_size, bias, normed,     \
         queries_only, row_stride, cos_sin, rot_dims, values_normed, static_cast<int>(total), given)

@@ -301,7 +301,8 @@ __global__ __launch_bounds__(kDecodeThreads) void paged_attention_decode_kernel(
         float top = m_shared[0][h];
 #pragma unroll
         for (int w = 1; w < kSlots; ++w) top = fmaxf(top, m_shared[w][h]);
-        const bool sink_here = EXTRA && extras.sink != nullptr && n_splits == 1;      // else the join kernel counts it
+        const bool whole = n_splits == 1 && !(EXTRA && extras.difference > 0);      // nothing is left to be joined
+        const bool sink_here = EXTRA && extras.sink != nullptr && whole;      // else the join kernel counts it
         if (sink_here) top = fmaxf(top, extras.sink[head0 + h]);
         float total = 0.0f, sum = 0.0f;
 #pragma unroll
@@ -314,7 +315,7 @@ __global__ __launch_bounds__(kDecodeThreads) void paged_attention_decode_kernel(
         if (sink_here) sum += __expf(extras.sink[head0 + h] - top);
         const int64_t row = static_cast<int64_t>(token) * heads + head0 + h;
         const int64_t part_row = static_cast<int64_t>(blockIdx.x) * heads + head0 + h;   // partial results are kept densely
-        if (n_splits == 1) {
+        if (whole) {
             if (EXTRA) store_result(extras, out, token, (head0 + h) * HD + dim, total / sum * extras.out_scale * result_gate(extras, token, head0 + h, HD, dim));
             else out[row * HD + dim] = from_float<bf16>(total / sum);
         } else {
@@ -374,6 +375,58 @@ __global__ void paged_attention_join_kernel(const float* __restrict__ part_o, co
     }
 }
 
+// Joins the splits of two neighbouring heads of a token and combines them (MllAttentionExtras.difference): a thread a channel.
+constexpr int kMostChannels = 256;
+
+__global__ void __launch_bounds__(kMostChannels)
+paged_attention_join_difference_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml,
+                                       const int32_t* __restrict__ token_ids, bf16* __restrict__ out, int heads, int head_dim,
+                                       int n_splits, MllAttentionExtras extras) {
+    __shared__ float scratch[16];
+    const int twos = heads / 2;
+    const int token = token_ids ? token_ids[blockIdx.x / twos] : blockIdx.x / twos;
+    if (token < 0) return;      // an entry that only pads the list to a fixed length
+    const int two = blockIdx.x % twos, dim = threadIdx.x;
+    float result[2];
+#pragma unroll
+    for (int map = 0; map < 2; ++map) {
+        const int64_t part_row = static_cast<int64_t>(blockIdx.x / twos) * heads + 2 * two + map;
+        const float2* ml = reinterpret_cast<const float2*>(part_ml) + part_row * n_splits;
+        float top = -INFINITY, total = 0.0f, weight_sum = 0.0f;
+        for (int base = 0; base < n_splits; base += 8) {        // eight splits asked for at a time, used in their order
+            float2 pair[8];
+            float part[8];
+#pragma unroll
+            for (int j = 0; j < 8; ++j) {
+                const int split = min(base + j, n_splits - 1);
+                pair[j] = ml[split];
+                part[j] = part_o[(part_row * n_splits + split) * head_dim + min(dim, head_dim - 1)];
+            }
+            float new_top = top;
+#pragma unroll
+            for (int j = 0; j < 8; ++j) new_top = fmaxf(new_top, pair[j].x);
+            const float keep = top == -INFINITY ? 0.0f : __expf(top - new_top);
+            total *= keep;
+            weight_sum *= keep;
+            top = new_top;
+#pragma unroll
+            for (int j = 0; j < 8; ++j) {
+                if (base + j >= n_splits || pair[j].x == -INFINITY) continue;       // past the end, or a split without keys
+                const float weight = __expf(pair[j].x - top);
+                total += weight * part[j];
+                weight_sum += weight * pair[j].y;
+            }
+        }
+        result[map] = total / weight_sum;
+    }
+    const bool live = dim < extras.difference;
+    const float o = live ? result[0] - extras.difference_lambda * result[1] : 0.0f;
+    const float squares = block_sum(o * o, scratch);
+    if (live)
+        store_result(extras, out, token, two * extras.difference + dim,
+                     o * (extras.difference_factor / sqrtf(squares / static_cast<float>(extras.difference) + extras.difference_eps)));
+}
+
 template <int HD_TILES>
 static int launch_decode(const void* q, const void* k_cache, const void* v_cache, const int32_t* block_table,
                          int table_width, const int32_t* seq_of_token, const int32_t* positions,
@@ -418,14 +471,18 @@ extern "C" int mll_paged_attention_decode_extra(const void* q, const void* k_cac
                                                 float* part_ml, float scale, int window, int n_tokens, int heads, int kv_heads,
                                                 int head_dim, int page_size, int n_splits, const MllAttentionExtras* extras,
                                                 hipStream_t stream) {
-    MLL_REQUIRE(!extras || extras->out_stride >= static_cast<int64_t>(heads) * head_dim, "paged_attention_decode: the output rows overlap");
+    const bool twos = extras && extras->difference > 0;
+    MLL_REQUIRE(!extras || extras->out_stride >= (twos ? static_cast<int64_t>(heads / 2) * extras->difference : static_cast<int64_t>(heads) * head_dim),
+                "paged_attention_decode: the output rows overlap");
+    MLL_REQUIRE(!twos || (heads % 2 == 0 && extras->difference <= head_dim && extras->difference_eps > 0.0f && !extras->sink && !extras->gate),
+                "paged_attention_decode: combined heads come in twos, without sinks and gates");
     MLL_REQUIRE(!extras || !extras->bias || extras->longest >= 0, "paged_attention_decode: the bias table needs a row");
     MLL_REQUIRE(heads > 0 && kv_heads > 0 && heads % kv_heads == 0, "paged_attention_decode: heads must divide into kv_heads groups");
     MLL_REQUIRE(head_dim % 16 == 0 && head_dim >= 16 && head_dim <= 256,
                 "paged_attention_decode: head_dim must be a multiple of 16 in [16, 256]");
     MLL_REQUIRE(page_size > 0 && page_size % 16 == 0, "paged_attention_decode: page_size must be a multiple of 16");
     MLL_REQUIRE(n_splits >= 1 && n_splits <= 65535, "paged_attention_decode: bad number of splits");
-    MLL_REQUIRE(n_splits == 1 || (part_o && part_ml), "paged_attention_decode: splits need the partial buffers");
+    MLL_REQUIRE((n_splits == 1 && !twos) || (part_o && part_ml), "paged_attention_decode: splits need the partial buffers");
     MLL_REQUIRE(kv_heads * ((heads / kv_heads + 15) / 16) <= 65535, "paged_attention_decode: too many heads");
     if (n_tokens == 0) return 0;
     int status = 0;
@@ -444,6 +501,11 @@ extern "C" int mll_paged_attention_decode_extra(const void* q, const void* k_cac
     }
 #undef MLL_DECODE_CASE
     if (status != 0) return status;
+    if (twos) {
+        paged_attention_join_difference_kernel<<<n_tokens * (heads / 2), (extras->difference + kWave - 1) / kWave * kWave, 0, stream>>>(
+            part_o, part_ml, token_ids, static_cast<bf16*>(out), heads, head_dim, n_splits, *extras);
+        return check_launch("paged_attention_join_difference");
+    }
     if (n_splits > 1) {
         const int threads = head_dim <= 64 ? 64 : (head_dim <= 128 ? 128 : 256);
         if (extras) {

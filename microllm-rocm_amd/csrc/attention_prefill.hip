@@ -568,6 +568,7 @@ extern "C" int mll_paged_attention_prefill_extra(const void* q, const void* k_ca
                                                  int n_tiles, const int32_t* positions, void* out, float scale, int window,
                                                  int heads, int kv_heads, int head_dim, int page_size,
                                                  const MllAttentionExtras* extras, hipStream_t stream) {
+    MLL_REQUIRE(!extras || extras->difference == 0, "paged_attention_prefill: results are combined after the kernel");
     MLL_REQUIRE(!extras || !extras->out_f32 || (!extras->gate_channels && extras->out_stride % 4 == 0 && reinterpret_cast<uintptr_t>(out) % 16 == 0),
                 "paged_attention_prefill: float32 results come in aligned rows and without a gate a channel");
     MLL_REQUIRE(!extras || scale > 0.0f, "paged_attention_prefill: a bias, a sink or a cap on the scores needs a positive scale");

@@ -32,7 +32,7 @@ union Piece {
 // float32 residual stream and the sum, times the next norm's weight, is written as the next product's input,
 // with each workgroup's share of the rows' sums of squares (at most 16 rows; see MllResidualNorm).
 // 5 = 2 with the tanh form of gelu for silu. 6 = bfloat16 [M, N] = gelu_tanh(product) * the token's columns of a side
-// table (at most 16 rows; see MllSideTable).
+// table (at most 16 rows; see MllSideTable). 7 = 2 with the clamped form (gated_value in common.h; at most 16 rows).
 // Whatever the epilogue, a row of the product is first multiplied by the factor that MllRowScale describes,
 // if one is given (at most 16 rows).
 // W is read past the caches (non-temporal loads): a step reads every weight once, and all of them together are far
@@ -298,6 +298,14 @@ __global__ __launch_bounds__(1024) void gemm_skinny_kernel(
                     const int column = n_tile * 16 + quad * 4 + i;
                     if (column < n) target[column] = from_float<bf16>(activate(acc[nt][mt][i], kActGeluTanh) * side[nt][i]);
                 }
+            } else if (EPILOGUE == 7) {
+                bf16* target = static_cast<bf16*>(out) + static_cast<int64_t>(row) * (n / 2);
+#pragma unroll
+                for (int i = 0; i < 4; i += 2) {
+                    const int column = n_tile * 8 + quad * 2 + i / 2;
+                    if (column < n / 2)
+                        target[column] = from_float<bf16>(gated_value(acc[nt][mt][i], acc[nt][mt][i + 1], kActClampedGlu, extras.glu_limit, extras.glu_slope));
+                }
             } else if (EPILOGUE == 2 || EPILOGUE == 5) {
                 bf16* target = static_cast<bf16*>(out) + static_cast<int64_t>(row) * (n / 2);
 #pragma unroll
@@ -403,7 +411,7 @@ static int launch_skinny(const void* a, const void* w_packed, void* out, int m, 
     const bf16* w_ = static_cast<const bf16*>(w_packed);
     const int m_tiles = (m + 15) / 16;
     const bool two = tiles_per_group(m, n_tiles) == 2;
-    if constexpr (EPILOGUE == 3 || EPILOGUE == 4 || EPILOGUE == 6) {
+    if constexpr (EPILOGUE == 3 || EPILOGUE == 4 || EPILOGUE == 6 || EPILOGUE == 7) {
         if (m_tiles != 1) return fail("gemm_skinny: this epilogue takes at most 16 rows");
         if (two) launch_one<1, 2, EPILOGUE>(a_, w_, out, m, n, k, n_tiles, k_steps, extras, stream);
         else launch_one<1, 1, EPILOGUE>(a_, w_, out, m, n, k, n_tiles, k_steps, extras, stream);
@@ -455,6 +463,18 @@ extern "C" int mll_gemm_skinny(const void* a, const void* w_packed, void* out, i
         case 5: return launch_skinny<5>(a, w_packed, out, m, n, k, extras, stream);
         default: return fail("gemm_skinny: unknown epilogue");
     }
+}
+
+extern "C" int mll_gemm_skinny_clamped(const void* a, const void* w_packed, void* out, int m, int n, int k, float limit, float slope,
+                                       hipStream_t stream) {
+    MLL_REQUIRE(m >= 0 && m <= 16, "gemm_skinny_clamped: takes at most 16 rows");
+    MLL_REQUIRE(n > 0 && n % 2 == 0 && k > 0 && k % 8 == 0, "gemm_skinny_clamped: an even number of weight rows, k a multiple of 8");
+    MLL_REQUIRE(limit > 0.0f, "gemm_skinny_clamped: the limit must be positive");
+    if (m == 0) return 0;
+    MllSkinnyExtras extras{};
+    extras.glu_limit = limit;
+    extras.glu_slope = slope;
+    return launch_skinny<7>(a, w_packed, out, m, n, k, extras, stream);
 }
 
 extern "C" int mll_gemm_skinny_side(const void* a, const void* w_packed, void* out, int m, int n, int k, const MllSideTable* side,

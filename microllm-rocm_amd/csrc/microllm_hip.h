@@ -205,12 +205,18 @@ struct MllSideTable {
 int mll_gemm_skinny_side(const void* a, const void* w_packed, void* out, int m, int n, int k, const MllSideTable* side,
                          hipStream_t stream);
 
+// The product of at most 16 rows with the gated weight's interleaved rows, finished as mll_clamped_glu does: bfloat16 out [m, n / 2].
+int mll_gemm_skinny_clamped(const void* a, const void* w_packed, void* out, int m, int n, int k, float limit, float slope,
+                            hipStream_t stream);
+
 // What the kernel takes beside the product's operands (internal to the library's launches).
 struct MllSkinnyExtras {
     MllSideTable side;
     MllQkvStore store;
     MllRowScale scale;
     MllResidualNorm residual;
+    float glu_limit;        // of the clamped gate
+    float glu_slope;
 };
 
 // The same product for up to 64 rows with the activations shared through LDS by the waves of a workgroup
@@ -287,6 +293,12 @@ typedef struct MllAttentionExtras {
     float softcap;          // > 0: the scaled score becomes softcap * tanh(score / softcap), before a bias is added
     int gate_channels;      // with gate: its rows hold heads * head_dim numbers, one for every channel of the result
     int out_f32;            // the result is float32 (out_stride counts floats)
+    int difference;         // > 0, decoding only: heads come in twos, whose results a_1 and a_2 are combined where the splits meet:
+                            // out[t][h] = o / sqrt(mean(o^2) + eps) * factor over the first `difference` channels, o = a_1 - lambda a_2
+                            // (rows of heads / 2 * difference channels; no sink, gate or factor then)
+    float difference_lambda;
+    float difference_eps;
+    float difference_factor;
 } MllAttentionExtras;
 
 int mll_paged_attention_decode_extra(const void* q, const void* k_cache, const void* v_cache,
@@ -323,9 +335,9 @@ int mll_stream_norm(float* x, const float* y, int n_parts, int64_t part_stride, 
                     int n_rows, int streams, int width, int write_x, hipStream_t stream);
 
 // gate_up[t] = [gate (width) | up (width)] in float32: g = min(gate, limit), u = clamp(up, -limit, limit),
-// out[t] = g * sigmoid(slope * g) * (u + 1) in `dtype`.
+// out[t] = g * sigmoid(slope * g) * (u + 1) in `dtype`. interleaved: gate_up[t] holds gate and up by turns.
 int mll_clamped_glu(const float* gate_up, void* out, int dtype, int n_tokens, int width, float limit, float slope,
-                    hipStream_t stream);
+                    int interleaved, hipStream_t stream);
 
 // ---- attention with a bias by distance and a sink, keys and values of different widths in plain pages --------
 
@@ -519,6 +531,12 @@ int mll_moe_route(const float* z, int64_t z_stride, int n_tokens, int experts, i
                   int shared_at, int32_t* ids, float* weights, float* shared_gate, int groups, int keep, const float* correction,
                   float weight_eps, float weight_scale, hipStream_t stream);
 
+// mll_router_logits and mll_moe_route in one kernel, for at most 64 experts: w float32 [n_out][width], the experts' rows first
+// (n_out at most 65; shared_at may name the one row behind them).
+int mll_moe_choose(const void* x, int dtype, const float* w, int n_tokens, int n_out, int width, int experts, int top, int softmax_scores,
+                   int renormalize, int shared_at, int32_t* ids, float* weights, float* shared_gate, int groups, int keep,
+                   const float* correction, float weight_eps, float weight_scale, hipStream_t stream);
+
 // What an expert does between its products, and how many there are. activation: 0 SiLU, 1 gelu (erf), 2 gelu (tanh), each
 // act(g) * u with gated and act(u) without; 3 (gated only): g = min(g, limit), u = clamp(u, -limit, limit),
 // g * sigmoid(slope * g) * (u + 1). An id of `experts` or more names an expert without weights that returns its input.
@@ -534,26 +552,31 @@ typedef struct MllExpertForm {
 // act[t * top + n] = silu(Wg_e xs) * (Wu_e xs), e = ids[t][n], xs = x[t] * weights[t][n] rounded to `dtype`
 // (weight_on_input) or x[t]; gate_up [experts][2 * ff][width] with the gate rows first.
 // not gated: gate_up is [experts][ff][width] and act = activation(Wu_e xs). Pairs of an id that returns its input have no act.
-int mll_moe_gate_up(const void* x, const int32_t* ids, const float* weights, int top, const void* gate_up, void* act,
-                    int dtype, int n_tokens, int width, int ff, int weight_on_input, const MllExpertForm* form,
-                    hipStream_t stream);
+// offsets and order: mll_moe_sort's (null where there are at most 64 pairs: the kernels look through them).
+int mll_moe_gate_up(const void* x, const int32_t* ids, const float* weights, int top, const int32_t* offsets, const int32_t* order,
+                    const void* gate_up, void* act, int dtype, int n_tokens, int width, int ff, int weight_on_input,
+                    const MllExpertForm* form, hipStream_t stream);
 
-// out[n][t] = Wd_e act[t * top + n] (* weights[t][n] unless weight_on_input): float32, in parts of part_tokens rows
-// (part_tokens > n_tokens: a launch for some of a step's tokens); an id that returns its input gives x[t] * weights[t][n].
-int mll_moe_down(const void* x, const void* act, const int32_t* ids, const float* weights, int top, const void* down, float* out,
-                 int dtype, int n_tokens, int part_tokens, int width, int ff, int weight_on_input, const MllExpertForm* form,
-                 hipStream_t stream);
+// out[n][t] = Wd_e act[t * top + n] (* weights[t][n] unless weight_on_input): float32 [top][n_tokens][width]; an id that returns
+// its input gives x[t] * weights[t][n].
+int mll_moe_down(const void* x, const void* act, const int32_t* ids, const float* weights, int top, const int32_t* offsets,
+                 const int32_t* order, const void* down, float* out, int dtype, int n_tokens, int width, int ff, int weight_on_input,
+                 const MllExpertForm* form, hipStream_t stream);
+
+// The pairs in the order of their ids, of which there are `named`: offsets [named + 1], order [n_pairs], a pair keeping its place
+// among its id's.
+int mll_moe_sort(const int32_t* ids, int n_pairs, int named, int32_t* offsets, int32_t* order, hipStream_t stream);
 
 // out[t] = factor[t] * (in[0][t] + in[1][t] + ...), float32; parts part_stride elements apart.
 int mll_scale_rows(const float* in, int n_parts, int64_t part_stride, const float* factor, float* out, int n_tokens, int width,
                    hipStream_t stream);
 
-// The same as mll_moe_gate_up and mll_moe_down together for many bfloat16 pairs: the pairs are sorted by id (counts
-// [ids], offsets [ids + 1], order [n_tokens * top]: int32 scratch, ids = experts + identity), their inputs gathered into `sorted`
-// ([pairs][width]), and every expert multiplies its rows in tiles on the matrix units; `act` is [pairs][ff] scratch.
+// The same as mll_moe_gate_up and mll_moe_down together for many bfloat16 pairs: the pairs are sorted by id (offsets
+// [ids + 1], order [n_tokens * top]: int32 scratch, ids = experts + identity), with weight_on_input their inputs
+// are gathered into `sorted` ([pairs][width]; else it may be null), and every expert multiplies its rows in tiles on the matrix units; `act` is [pairs][ff] scratch.
 // width and ff are multiples of 8.
 int mll_moe_grouped(const void* x, const int32_t* ids, const float* weights, int top, const void* gate_up, const void* down,
-                    int32_t* counts, int32_t* offsets, int32_t* order, void* sorted, void* act, float* out, int n_tokens,
+                    int32_t* offsets, int32_t* order, void* sorted, void* act, float* out, int n_tokens,
                     int width, int ff, int weight_on_input, const MllExpertForm* form, hipStream_t stream);
 
 // mll_rglru_scan for steps with long portions: the recurrence in chunks of 64 tokens (every chunk walked from zero,

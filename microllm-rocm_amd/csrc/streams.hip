@@ -110,15 +110,14 @@ __global__ void stream_norm_kernel(float* __restrict__ x, const float* __restric
 // gu[t] = [gate (width) | up (width)] in float32: g = min(gate, limit), u = clamp(up, -limit, limit),
 // out = g * sigmoid(slope * g) * (u + 1).
 template <typename T>
-__global__ void clamped_glu_kernel(const float* __restrict__ gu, T* __restrict__ out, int width, float limit, float slope) {
+__global__ void clamped_glu_kernel(const float* __restrict__ gu, T* __restrict__ out, int width, float limit, float slope,
+                                   int interleaved) {
     const int token = blockIdx.y;
     const int column = blockIdx.x * blockDim.x + threadIdx.x;
     if (column >= width) return;
     const float* row = gu + static_cast<int64_t>(token) * 2 * width;
-    const float g = fminf(row[column], limit);
-    const float u = fminf(fmaxf(row[width + column], -limit), limit);
-    const float gate = g / (1.0f + expf(-slope * g));
-    out[static_cast<int64_t>(token) * width + column] = from_float<T>(gate * (u + 1.0f));
+    const float gate = row[interleaved ? 2 * column : column], up = row[interleaved ? 2 * column + 1 : width + column];
+    out[static_cast<int64_t>(token) * width + column] = from_float<T>(gated_value(gate, up, kActClampedGlu, limit, slope));
 }
 
 }  // namespace mll
@@ -174,16 +173,16 @@ int mll_stream_norm(float* x, const float* y, int n_parts, int64_t part_stride, 
 }
 
 int mll_clamped_glu(const float* gate_up, void* out, int dtype, int n_tokens, int width, float limit, float slope,
-                    hipStream_t stream) {
+                    int interleaved, hipStream_t stream) {
     MLL_REQUIRE(n_tokens >= 0 && width > 0, "clamped_glu: sizes must be positive");
     MLL_REQUIRE(limit > 0.0f, "clamped_glu: the limit must be positive");
     if (n_tokens == 0) return 0;
     MLL_REQUIRE(n_tokens <= 65535, "clamped_glu: more than 65535 tokens in one call");
     const dim3 grid((width + 255) / 256, n_tokens);
     if (dtype == kF32) {
-        clamped_glu_kernel<float><<<grid, 256, 0, stream>>>(gate_up, static_cast<float*>(out), width, limit, slope);
+        clamped_glu_kernel<float><<<grid, 256, 0, stream>>>(gate_up, static_cast<float*>(out), width, limit, slope, interleaved);
     } else if (dtype == kBF16) {
-        clamped_glu_kernel<bf16><<<grid, 256, 0, stream>>>(gate_up, static_cast<bf16*>(out), width, limit, slope);
+        clamped_glu_kernel<bf16><<<grid, 256, 0, stream>>>(gate_up, static_cast<bf16*>(out), width, limit, slope, interleaved);
     } else {
         return fail("clamped_glu: unknown dtype");
     }

@@ -751,7 +751,18 @@ def gemm_bf16_split(x: torch.Tensor, weight: torch.Tensor, parts: int) -> torch.
 class _AttentionExtras(ctypes.Structure):
     _fields_ = [("bias", ctypes.c_void_p), ("longest", ctypes.c_int), ("sink", ctypes.c_void_p),
                 ("out_scale", ctypes.c_float), ("out_stride", ctypes.c_int64), ("chunk", ctypes.c_int), ("gate", ctypes.c_void_p),
-                ("gate_stride", ctypes.c_int64), ("softcap", ctypes.c_float), ("gate_channels", ctypes.c_int), ("out_f32", ctypes.c_int)]
+                ("gate_stride", ctypes.c_int64), ("softcap", ctypes.c_float), ("gate_channels", ctypes.c_int), ("out_f32", ctypes.c_int),
+                ("difference", ctypes.c_int), ("difference_lambda", ctypes.c_float), ("difference_eps", ctypes.c_float),
+                ("difference_factor", ctypes.c_float)]
+
+
+class HeadDifference(NamedTuple):
+    """Heads in twos whose results are combined: ``o = first - on_second * second`` over the first ``value_dim`` channels, divided
+    by its root mean square and multiplied by ``factor``."""
+    value_dim: int
+    on_second: float
+    eps: float
+    factor: float
 
 
 class AttentionExtras(NamedTuple):
@@ -761,13 +772,15 @@ class AttentionExtras(NamedTuple):
     chunk`` on (no window then); ``gate`` float32 ``[tokens, heads]`` (columns of a wider buffer allowed): a head's result
     is multiplied by ``sigmoid(gate)``; ``[tokens, heads * head_dim]``: every channel of the result by its own;
     ``softcap`` c (0: none): the scaled score becomes ``c * tanh(score / c)`` before a bias is added. With extras the
-    result may be a float32 tensor (without gates a channel)."""
+    result may be a float32 tensor (without gates a channel). ``difference`` (``paged_attention`` alone): heads in twos give
+    one result of ``value_dim`` channels each."""
     bias: Optional[torch.Tensor] = None
     sink: Optional[torch.Tensor] = None
     out_scale: float = 1.0
     chunk: int = 0
     gate: Optional[torch.Tensor] = None
     softcap: float = 0.0
+    difference: Optional[HeadDifference] = None
 
 
 def _gate_stride(gate: Optional[torch.Tensor], n_tokens: int, heads: int, value_dim: int) -> Tuple[int, bool]:
@@ -797,8 +810,12 @@ def _extras_argument(extras: Optional[AttentionExtras], heads: int, head_dim: in
     if extras.sink is not None:
         _device_tensor(extras.sink, "sink", torch.float32)
         _need(tuple(extras.sink.shape) == (heads,), "one sink a head")
-    _need(out.dim() == 2 and out.stride(1) == 1 and out.shape[1] == heads * head_dim, "the output is [tokens, heads * head_dim] with unit column stride")
-    stride = max(out.stride(0), heads * head_dim)
+    two = extras.difference
+    columns = heads * head_dim if two is None else heads // 2 * two.value_dim
+    _need(out.dim() == 2 and out.stride(1) == 1 and out.shape[1] == columns, "the output is [tokens, heads * head_dim] with unit column stride")
+    _need(two is None or (heads % 2 == 0 and 1 <= two.value_dim <= head_dim and extras.sink is None and extras.gate is None and extras.out_scale == 1.0),
+          "heads in twos, without a sink, gates or a factor")
+    stride = max(out.stride(0), columns)
     gate_stride, gate_channels = _gate_stride(extras.gate, out.shape[0], heads, head_dim)
     _need(extras.softcap >= 0.0, "the cap on the scores is positive, or 0 for none")
     _need(extras.chunk >= 0, "chunks of positions are positive, or 0 for none")
@@ -806,7 +823,9 @@ def _extras_argument(extras: Optional[AttentionExtras], heads: int, head_dim: in
                                          extras.sink.data_ptr() if extras.sink is not None else None,
                                          float(extras.out_scale), stride, int(extras.chunk),
                                          extras.gate.data_ptr() if extras.gate is not None else None, gate_stride,
-                                         float(extras.softcap), int(gate_channels), int(out.dtype == torch.float32)))
+                                         float(extras.softcap), int(gate_channels), int(out.dtype == torch.float32),
+                                         *((int(two.value_dim), float(two.on_second), float(two.eps), float(two.factor)) if two is not None
+                                           else (0, 0.0, 0.0, 0.0))))
 
 
 def decode_splits(n_tokens: int, kv_heads: int, longest: int) -> int:
@@ -845,11 +864,13 @@ def paged_attention_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torc
         n_tokens = token_ids.shape[0]
     if out is None:
         out = torch.empty_like(q)
-    _need(out.is_cuda and out.shape == q.shape and (out.dtype == q.dtype or (extras is not None and out.dtype == torch.float32)),
+    two = extras.difference if extras is not None else None
+    _need(out.is_cuda and (out.shape == q.shape or (two is not None and out.shape[0] == q.shape[0]))
+          and (out.dtype == q.dtype or (extras is not None and out.dtype == torch.float32)),
           "attention output must have the queries' shape and dtype (or be float32, with extras)")
     extra = _extras_argument(extras, heads, head_dim, out)
     part_o = part_ml = None
-    if n_splits > 1:
+    if n_splits > 1 or two is not None:
         part_o = torch.empty((n_tokens, heads, n_splits, head_dim), dtype=torch.float32, device=q.device)
         part_ml = torch.empty((n_tokens, heads, n_splits, 2), dtype=torch.float32, device=q.device)
     _check(lib.mll_paged_attention_decode_extra(_ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.shape[1],
@@ -923,25 +944,37 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
 
     bfloat16 with a head size in steps of 16: the MFMA kernels, split over the keys when every request brings
     one token, tiled over the queries otherwise (``planner``: the attention part's, whose plan for the step
-    holds the tiles). Everything else (float32, other head sizes): the plain kernel.
+    holds the tiles). Everything else (float32, other head sizes): the plain kernel. With ``extras.difference`` the result is
+    ``[tokens, heads / 2 * value_dim]``: the split kernel's join combines the heads itself, the tiled kernel leaves float32 results
+    that ``attention_difference`` combines (for every row; the rows of single tokens are then written over).
     """
     mfma_fits = q.dtype == torch.bfloat16 and head_dim % 16 == 0 and head_dim <= 256
     _need(mfma_fits or (extras is None and out is None), "a bias, a sink or an output of its own need the MFMA kernels")
     _need(extras is None or not (extras.chunk and window), "a window or chunks of positions, not both")
+    two = extras.difference if extras is not None else None
     if mfma_fits and ctx.max_count == 1:
         longest = max(ctx.planned_total, ctx.max_total)
         reach = window if window > 0 else (extras.chunk if extras is not None else 0)      # the most keys a query sees, 0: all
         visible = min(longest, reach) if reach > 0 else longest
         splits = decode_splits(ctx.n_tokens, kv_heads, visible)
+        if out is None and two is not None:
+            out = torch.empty((q.shape[0], heads // 2 * two.value_dim), dtype=q.dtype, device=q.device)
         return paged_attention_decode(q, k_cache, v_cache, view.block_table, ctx.seq_of_token, ctx.positions,
                                       scale, window, heads, kv_heads, head_dim, splits, out=out, extras=extras)
     if mfma_fits:
         # Portions go to the tiled kernel; requests that bring one token, if any, to the split kernel.
         _need(planner is not None, "portions of prompts need the attention part's planner for their tiles")
         plan = ctx.plan_of(planner)
-        if out is None:
+        if two is not None:
+            _need(out is None, "heads that are combined bring an output of their own")
+            maps = torch.empty(q.shape, dtype=torch.float32, device=q.device)
+            if plan.tiles.shape[0] > 0:
+                paged_attention_prefill(q, k_cache, v_cache, view.block_table, plan.tiles, ctx.positions, scale, window, heads, kv_heads,
+                                        head_dim, out=maps, extras=extras._replace(difference=None))
+            out = attention_difference(maps, heads // 2, two.value_dim, two.on_second, two.eps, two.factor, q.dtype)
+        elif out is None:
             out = torch.empty_like(q)
-        if plan.tiles.shape[0] > 0:
+        if two is None and plan.tiles.shape[0] > 0:
             paged_attention_prefill(q, k_cache, v_cache, view.block_table, plan.tiles, ctx.positions,
                                     scale, window, heads, kv_heads, head_dim, out=out, extras=extras)
         if plan.single_tokens.shape[0] > 0:
@@ -1037,6 +1070,21 @@ def gemm_skinny_side(x: torch.Tensor, packed: torch.Tensor, n: int, table: torch
     out = torch.empty((m, n), dtype=torch.bfloat16, device=x.device)
     side = _SideTable(table.data_ptr(), ids.data_ptr(), table.shape[1], _code(table.dtype), int(column_at), table.shape[0])
     _check(lib.mll_gemm_skinny_side(_ptr(x), _ptr(packed), _ptr(out), m, n, k, ctypes.byref(side), _stream()), lib)
+    return out
+
+
+def gemm_skinny_clamped(x: torch.Tensor, packed: torch.Tensor, n: int, limit: float, slope: float) -> torch.Tensor:
+    """``clamped_glu`` of ``x @ W.T`` in the product's epilogue: at most 16 bfloat16 rows and a packed weight of ``n`` rows, gate and
+    up interleaved (``pack_weight(interleave_halves=True)``)."""
+    lib = library.load()
+    _device_tensor(x, "gemm input", torch.bfloat16)
+    _device_tensor(packed, "packed weight", torch.bfloat16)
+    _need(x.dim() == 2 and packed.dim() == 5 and tuple(packed.shape[2:]) == (4, 16, 8), "gemm_skinny_clamped takes [m, k] and a packed weight")
+    m, k = x.shape
+    _need(m <= 16 and k % 8 == 0 and n % 2 == 0, "at most 16 rows of a multiple of 8, an even number of weight rows")
+    _need(packed.shape[0] == -(-n // 16) and packed.shape[1] == -(-k // 32), "the packed weight does not fit n and k")
+    out = torch.empty((m, n // 2), dtype=torch.bfloat16, device=x.device)
+    _check(lib.mll_gemm_skinny_clamped(_ptr(x), _ptr(packed), _ptr(out), m, n, k, ctypes.c_float(limit), ctypes.c_float(slope), _stream()), lib)
     return out
 
 
@@ -1312,9 +1360,9 @@ def stream_norm(x: torch.Tensor, weight: Optional[torch.Tensor], eps: float, out
     return out
 
 
-def clamped_glu(gate_up: torch.Tensor, limit: float, slope: float, out_dtype: torch.dtype) -> torch.Tensor:
+def clamped_glu(gate_up: torch.Tensor, limit: float, slope: float, out_dtype: torch.dtype, interleaved: bool = False) -> torch.Tensor:
     """``g * sigmoid(slope * g) * (u + 1)`` with ``g = min(gate, limit)``, ``u = clamp(up, -limit, limit)`` of float32
-    rows ``[tokens, 2 * width]`` (gate first)."""
+    rows ``[tokens, 2 * width]`` (gate first, or gate and up by turns where ``interleaved``)."""
     lib = library.load()
     _device_tensor(gate_up, "gate/up", torch.float32)
     _need(gate_up.dim() == 2 and gate_up.shape[1] % 2 == 0, "gate/up must be [tokens, 2 * width]")
@@ -1324,7 +1372,7 @@ def clamped_glu(gate_up: torch.Tensor, limit: float, slope: float, out_dtype: to
         count = min(65535, n_tokens - start)
         _check(lib.mll_clamped_glu(ctypes.c_void_p(gate_up.data_ptr() + start * 2 * width * 4),
                                    ctypes.c_void_p(out.data_ptr() + start * width * out.element_size()), _code(out_dtype),
-                                   count, width, ctypes.c_float(limit), ctypes.c_float(slope), _stream()), lib)
+                                   count, width, ctypes.c_float(limit), ctypes.c_float(slope), int(interleaved), _stream()), lib)
     return out
 
 
@@ -1951,10 +1999,36 @@ def moe_route(z: torch.Tensor, experts: int, top: int, softmax_scores: bool = Fa
     return ids, weights, shared
 
 
-MOE_PAIRS_A_LAUNCH = 65535
+MOE_CHOOSE_PLACES = 64      # up to so many places (and one row beside them) the router's product and the choice are one kernel
 
 
-MOE_GROUPED_PAIRS = 64      # from this many (token, choice) pairs on, bfloat16 experts multiply their rows in tiles
+def moe_choose(x: torch.Tensor, weight: torch.Tensor, experts: int, top: int, softmax_scores: bool = False, renormalize: bool = False,
+               shared_at: int = -1, groups: int = 0, keep: int = 0, correction: Optional[torch.Tensor] = None,
+               weight_eps: float = 0.0, weight_scale: float = 1.0):
+    """``moe_route`` of ``router_logits(x, weight)``: one kernel for up to ``MOE_CHOOSE_PLACES`` experts."""
+    if experts > MOE_CHOOSE_PLACES or weight.shape[0] > experts + 1:
+        return moe_route(router_logits(x, weight), experts, top, softmax_scores, renormalize, shared_at, groups, keep, correction,
+                         weight_eps, weight_scale)
+    lib = library.load()
+    _device_tensor(x, "router input")
+    _device_tensor(weight, "router weight", torch.float32)
+    _need(x.dim() == 2 and weight.dim() == 2 and weight.shape[1] == x.shape[1] and experts <= weight.shape[0] and shared_at < weight.shape[0],
+          "moe_choose takes [tokens, width] and [experts (+ 1), width]")
+    n_tokens = x.shape[0]
+    ids = torch.empty((n_tokens, top), dtype=torch.int32, device=x.device)
+    weights = torch.empty((n_tokens, top), dtype=torch.float32, device=x.device)
+    shared = torch.empty((n_tokens,), dtype=torch.float32, device=x.device) if shared_at >= 0 else None
+    if correction is not None:
+        _device_tensor(correction, "correction of the scores", torch.float32)
+        _need(tuple(correction.shape) == (experts,), "one correction an expert")
+    _check(lib.mll_moe_choose(_ptr(x), _code(x.dtype), _ptr(weight), n_tokens, weight.shape[0], x.shape[1], experts, top, int(softmax_scores),
+                              int(renormalize), int(shared_at), _ptr(ids), _ptr(weights), _ptr(shared), int(groups), int(keep),
+                              _ptr(correction), ctypes.c_float(weight_eps), ctypes.c_float(weight_scale), _stream()), lib)
+    return ids, weights, shared
+
+
+MOE_PAIRS_LOOKED_THROUGH = 64   # the experts' kernels find their pairs among so many themselves; more come sorted
+MOE_GROUPED_PAIRS = 160     # from this many (token, choice) pairs on, bfloat16 experts multiply their rows in tiles
 
 
 CLAMPED_GLU = "clamped_glu"     # g = min(g, limit), u = clamp(u, -limit, limit): g * sigmoid(slope * g) * (u + 1)
@@ -1973,7 +2047,7 @@ def moe_experts(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, gate_
     (gate rows first), ``down`` ``[experts, width, ff]``. Returns float32 ``[top, tokens, width]``, a part per choice,
     for the reader to add in order (``out``: at least that many leading parts of a larger buffer). ``grouped``: the
     pairs sorted by expert and multiplied in tiles on the matrix units (bfloat16, widths in steps of 8) instead of
-    one reading of the expert's weights a pair; by default by the number of pairs. With ``gated`` false an expert is
+    one reading of the expert's weights for every four of its pairs; by default by the number of pairs. With ``gated`` false an expert is
     ``down act(up x)`` and ``gate_up`` holds ``[experts, ff, width]``; ``activation`` is one of ``ACTIVATIONS``, or
     ``clamped_glu`` with its ``limit`` and ``slope`` (gated). The ``identity`` ids after the experts' return their input."""
     lib = library.load()
@@ -2000,27 +2074,24 @@ def moe_experts(x: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, gate_
     act = torch.empty((n_tokens * top, ff), dtype=x.dtype, device=x.device)
     if grouped is None:
         grouped = x.dtype == torch.bfloat16 and n_tokens * top >= MOE_GROUPED_PAIRS and width % 8 == 0 and ff % 8 == 0
+    n_pairs = n_tokens * top
+    offsets = order = None
+    if grouped or n_pairs > MOE_PAIRS_LOOKED_THROUGH:
+        scratch = torch.empty((named + 1 + n_pairs,), dtype=torch.int32, device=x.device)
+        offsets, order = scratch.data_ptr(), scratch.data_ptr() + 4 * (named + 1)
     if grouped:
         _need(x.dtype == torch.bfloat16 and width % 8 == 0 and ff % 8 == 0, "the tiled experts take bfloat16 and widths in steps of 8")
-        scratch = torch.empty((2 * named + 1 + n_tokens * top,), dtype=torch.int32, device=x.device)
-        counts, offsets, order = scratch[:named], scratch[named:2 * named + 1], scratch[2 * named + 1:]
-        in_order = torch.empty((n_tokens * top, width), dtype=x.dtype, device=x.device)
-        _check(lib.mll_moe_grouped(_ptr(x), _ptr(ids), _ptr(weights), top, _ptr(gate_up), _ptr(down), ctypes.c_void_p(counts.data_ptr()),
-                                   ctypes.c_void_p(offsets.data_ptr()), ctypes.c_void_p(order.data_ptr()), _ptr(in_order), _ptr(act),
-                                   _ptr(out), n_tokens, width, ff, int(weight_on_input), form, _stream()), lib)
+        in_order = torch.empty((n_pairs, width), dtype=x.dtype, device=x.device) if weight_on_input else None
+        _check(lib.mll_moe_grouped(_ptr(x), _ptr(ids), _ptr(weights), top, _ptr(gate_up), _ptr(down), ctypes.c_void_p(offsets),
+                                   ctypes.c_void_p(order), _ptr(in_order), _ptr(act), _ptr(out), n_tokens, width, ff, int(weight_on_input),
+                                   form, _stream()), lib)
         return out
-    step = max(1, MOE_PAIRS_A_LAUNCH // top)       # tokens a launch: its grid has a row of workgroups a pair
-    element = x.element_size()
-    for first in range(0, n_tokens, step):
-        count = min(step, n_tokens - first)
-        here = dict(x=ctypes.c_void_p(x.data_ptr() + first * width * element), ids=ctypes.c_void_p(ids.data_ptr() + first * top * 4),
-                    weights=ctypes.c_void_p(weights.data_ptr() + first * top * 4), act=ctypes.c_void_p(act.data_ptr() + first * top * ff * element))
-        _check(lib.mll_moe_gate_up(here["x"], here["ids"], here["weights"], top, _ptr(gate_up), here["act"], _code(x.dtype), count, width, ff,
-                                   int(weight_on_input), form, _stream()), lib)
-        # the output keeps its rows n_tokens apart in every part: the launch writes its tokens' rows of each
-        _check(lib.mll_moe_down(here["x"], here["act"], here["ids"], here["weights"], top, _ptr(down),
-                                ctypes.c_void_p(out.data_ptr() + first * width * 4), _code(x.dtype), count, n_tokens, width, ff,
-                                int(weight_on_input), form, _stream()), lib)
+    if offsets is not None:
+        _check(lib.mll_moe_sort(_ptr(ids), n_pairs, named, ctypes.c_void_p(offsets), ctypes.c_void_p(order), _stream()), lib)
+    _check(lib.mll_moe_gate_up(_ptr(x), _ptr(ids), _ptr(weights), top, ctypes.c_void_p(offsets), ctypes.c_void_p(order), _ptr(gate_up),
+                               _ptr(act), _code(x.dtype), n_tokens, width, ff, int(weight_on_input), form, _stream()), lib)
+    _check(lib.mll_moe_down(_ptr(x), _ptr(act), _ptr(ids), _ptr(weights), top, ctypes.c_void_p(offsets), ctypes.c_void_p(order), _ptr(down),
+                            _ptr(out), _code(x.dtype), n_tokens, width, ff, int(weight_on_input), form, _stream()), lib)
     return out
 
 

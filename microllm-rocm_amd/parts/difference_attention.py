@@ -10,7 +10,8 @@ padding to one width) is the softmax attention's that this part extends.
 The maps are query heads of one attention: a key head caches ``[k1 | k2]`` as one key of ``2 dim`` channels, and the two
 queries of a head are written as ``[q1 | 0]`` and ``[0 | q2]``, so ``2 * heads`` query heads over ``kv_heads`` key/value heads run
 on the attention kernels as they are, and every key and value is cached and read once. The kernels leave the maps' results in
-float32; one kernel forms the difference, its norm and the factor, and rounds once.
+float32; the difference, its norm and the factor are formed where the split kernel's splits meet (single tokens) or by one
+kernel more, and rounded once.
 """
 from __future__ import annotations
 
@@ -52,10 +53,15 @@ class DifferentialAttention(BucketBiasAttention):
 
     def forward_inner(self, x, ctx, cache, out: Optional[torch.Tensor] = None, out_scale: float = 1.0) -> torch.Tensor:
         q, _, pages = self._store(x, ctx, cache)
-        maps = torch.empty((x.shape[0], self.heads * self.result_dim), dtype=torch.float32, device=x.device)
-        self._attend(q, None, pages, ctx, maps, 1.0)
-        result = kernels.attention_difference(maps, self.result_heads, self.value_dim, self.factor_on_second, self.eps,
-                                              (1.0 - self.difference) * out_scale, self.runtime.dtype)
+        combined = kernels.HeadDifference(self.value_dim, self.factor_on_second, self.eps, (1.0 - self.difference) * out_scale)
+        if self.tiled:
+            result = kernels.paged_attention(q, pages.k, pages.v, ctx.paged[pages.group], ctx, self.scale, self.window, self.heads, self.kv_heads,
+                                             self.stored_dim, planner=self.planner, extras=kernels.AttentionExtras(difference=combined))
+        else:
+            maps = torch.empty((x.shape[0], self.heads * self.result_dim), dtype=torch.float32, device=x.device)
+            self._attend(q, None, pages, ctx, maps, 1.0)
+            result = kernels.attention_difference(maps, self.result_heads, combined.value_dim, combined.on_second, combined.eps, combined.factor,
+                                                  self.runtime.dtype)
         if out is None:
             return result
         out.copy_(result)

@@ -30,7 +30,7 @@ import torch
 
 from ..ops import kernels
 from .base import FeedForward, MATRIX, Runtime, TensorDecl, VECTOR
-from .linear import Weight, linear
+from .linear import Weight, linear, linear_clamped_glu
 from .registry import register_part
 from .spec import PartSpec
 
@@ -124,8 +124,7 @@ class RoutedExperts(FeedForward):
             keep = self.runtime.keep_plain_weights
             if self.gated:
                 gate, up = tensors[self.name("shared.gate")], tensors[self.name("shared.up")]
-                # the clamped form reads the product's sums as they are, so its weight is packed in the rows' own order
-                self.shared_gate_up = Weight(torch.cat([gate, up], dim=0).contiguous(), gated=not self.clamped, keep_plain=keep)
+                self.shared_gate_up = Weight(torch.cat([gate, up], dim=0).contiguous(), gated=True, keep_plain=keep)
                 del gate, up
             else:
                 self.shared_gate_up = Weight(tensors[self.name("shared.up")], keep_plain=keep)
@@ -148,23 +147,22 @@ class RoutedExperts(FeedForward):
     def _routed(self, x, parts: Optional[torch.Tensor]):
         """The chosen experts' results as partial sums, a part a choice (the first parts of ``parts`` if given), and the
         shared expert's factor a token, if it has one."""
-        z = kernels.router_logits(x, self.route_weight)
-        ids, weights, shared_factor = kernels.moe_route(z, self.places, self.top, softmax_scores=self.score == "softmax",
-                                                        renormalize=self.renormalize,
-                                                        shared_at=self.places if self.shared_scale is not None else -1,
-                                                        groups=self.groups, keep=self.keep_groups, correction=self.correction,
-                                                        weight_eps=self.weight_eps, weight_scale=self.weight_scale)
+        ids, weights, shared_factor = kernels.moe_choose(x, self.route_weight, self.places, self.top, softmax_scores=self.score == "softmax",
+                                                         renormalize=self.renormalize,
+                                                         shared_at=self.places if self.shared_scale is not None else -1,
+                                                         groups=self.groups, keep=self.keep_groups, correction=self.correction,
+                                                         weight_eps=self.weight_eps, weight_scale=self.weight_scale)
         routed = kernels.moe_experts(x, ids, weights, self.gate_up, self.down, self.weight_on == "input", out=parts, gated=self.gated,
                                      activation=self.activation, limit=self.limit, slope=self.slope, identity=self.identity)
         return routed, shared_factor
 
     def _shared(self, x, partials: bool) -> torch.Tensor:
         """The shared expert's result, float32; with ``partials`` perhaps in parts."""
-        if self.clamped:        # its activation and the plain form's read the product's float32 sums and round once
-            inner = kernels.clamped_glu(linear(x, self.shared_gate_up, out_dtype=torch.float32), self.shared_limit, self.slope, x.dtype)
+        if self.clamped:
+            inner = linear_clamped_glu(x, self.shared_gate_up, self.shared_limit, self.slope)
         elif self.gated:
             inner = linear(x, self.shared_gate_up, gated=True)
-        else:
+        else:       # the activation reads the product's float32 sums and rounds once
             inner = kernels.activation(linear(x, self.shared_gate_up, out_dtype=torch.float32, partials=True), self.activation, x.dtype)
         return linear(inner, self.shared_down, out_dtype=torch.float32, partials=partials)
 

@@ -13,7 +13,7 @@ import torch
 
 from ..ops import kernels
 from .base import FeedForward, MATRIX, Runtime, TensorDecl
-from .linear import Weight, linear, linear_into_stream, takes_unscaled
+from .linear import Weight, linear, linear_clamped_glu, linear_into_stream, takes_unscaled
 from .registry import register_part
 from .spec import PartSpec
 
@@ -64,8 +64,8 @@ register_part("ffn", "swiglu", SwiGLU)
 
 class ClampedGLU(FeedForward):
     """A gated feed-forward with clamped inputs: ``g = min(gate(x), limit)``, ``u = clamp(up(x), -limit, limit)``,
-    ``down(g * sigmoid(slope * g) * (u + 1))``, no biases. Gate and up are one stacked product whose float32 result
-    the activation rounds once."""
+    ``down(g * sigmoid(slope * g) * (u + 1))``, no biases. Gate and up are one stacked product; its float32 sums pass the
+    activation (in the product's epilogue for few rows) and are rounded once."""
     graph_safe = True
 
     def __init__(self, spec: PartSpec, runtime: Runtime):
@@ -86,13 +86,12 @@ class ClampedGLU(FeedForward):
         gate, up = tensors[self.name("gate")], tensors[self.name("up")]
         if gate.dtype != up.dtype:
             raise TypeError("the gate and up weights of one layer must share a dtype to be stacked")
-        self.gate_up_weight = Weight(torch.cat([gate, up], dim=0).contiguous(), keep_plain=self.runtime.keep_plain_weights)
+        self.gate_up_weight = Weight(torch.cat([gate, up], dim=0).contiguous(), gated=True, keep_plain=self.runtime.keep_plain_weights)
         del gate, up
         self.down_weight = Weight(tensors[self.name("down")], keep_plain=self.runtime.keep_plain_weights)
 
     def forward(self, x, ctx):
-        gate_up = linear(x, self.gate_up_weight, out_dtype=torch.float32)
-        z = kernels.clamped_glu(gate_up, self.limit, self.slope, self.runtime.dtype)
+        z = linear_clamped_glu(x, self.gate_up_weight, self.limit, self.slope)
         return linear(z, self.down_weight, out_dtype=torch.float32, partials=True)
 
 

@@ -100,6 +100,17 @@ def takes_packed(weight: "Weight", rows: int, gated: bool = False) -> bool:
     return rows <= (MEDIUM_WIDE_ROWS if wide else MEDIUM_ROWS)
 
 
+def linear_clamped_glu(x: torch.Tensor, weight: "Weight", limit: float, slope: float) -> torch.Tensor:
+    """``g * sigmoid(slope * g) * (u + 1)`` of half the width, in x's dtype, with ``g = min(gate, limit)`` and ``u = clamp(up,
+    -limit, limit)`` of a gated weight's product (rows ``[gate; up]``): in the product's epilogue for few rows, else from its
+    float32 sums, rounded once."""
+    if x.dtype == torch.bfloat16 and weight.packed is not None and weight.gated and x.shape[0] <= SKINNY_ROWS:
+        return kernels.gemm_skinny_clamped(x, weight.packed, weight.out_features, limit, slope)
+    # the packed copy's rows, and so its products' columns, hold gate and up by turns
+    by_turns = weight.gated and x.dtype == weight.dtype and takes_packed(weight, x.shape[0])
+    return kernels.clamped_glu(linear(x, weight, out_dtype=torch.float32), limit, slope, x.dtype, interleaved=by_turns)
+
+
 def linear(x: Union[torch.Tensor, UnscaledRows], weight, out_dtype: Optional[torch.dtype] = None, gated: bool = False,
            partials: bool = False, activation: str = "silu") -> torch.Tensor:
     """``x @ W.T`` with float32 accumulation; the result has ``out_dtype`` (default: x's).

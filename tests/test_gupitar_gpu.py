@@ -419,12 +419,12 @@ def test_experts_of_every_pair(dtype, on_input):
             want = plain.gated_ff((w * x[token:token + 1]) if on_input else x[token:token + 1], t, "")[0] * (1.0 if on_input else w)
             bound = 1e-5 if dtype == torch.float32 else 0.03
             assert np.abs(parts[choice, token] - want).max() < bound * max(1.0, np.abs(want).max()), (token, choice)
-    limit, kernels.MOE_PAIRS_A_LAUNCH = kernels.MOE_PAIRS_A_LAUNCH, 7        # a step of more pairs than a launch takes goes in several
+    limit, kernels.MOE_PAIRS_LOOKED_THROUGH = kernels.MOE_PAIRS_LOOKED_THROUGH, 7        # more pairs than the kernels look through come sorted
     try:
-        in_pieces = kernels.moe_experts(device(x, dtype), device(ids, torch.int32), device(weights), device(gate_up, dtype), device(down, dtype), on_input)
+        sorted_first = kernels.moe_experts(device(x, dtype), device(ids, torch.int32), device(weights), device(gate_up, dtype), device(down, dtype), on_input)
     finally:
-        kernels.MOE_PAIRS_A_LAUNCH = limit
-    assert np.array_equal(in_pieces.cpu().numpy(), parts)
+        kernels.MOE_PAIRS_LOOKED_THROUGH = limit
+    assert np.array_equal(sorted_first.cpu().numpy(), parts)
 
 
 @pytest.mark.parametrize("n,width,ff,experts,top", [(300, 64, 40, 6, 2), (70, 200, 136, 3, 3), (513, 96, 264, 16, 1), (5, 48, 8, 4, 2)])

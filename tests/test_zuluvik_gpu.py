@@ -231,14 +231,15 @@ def differenced(q, k, v, taps, scale, factor, diff, portions_of, mfma, eps=1e-5,
                                         convolution=convolution)
         if kept is not None:
             kernels.conv_keep(proj, 0, kept, ctx.cu_tokens, ctx.slots, 1)
-        maps = torch.empty((portion, 2 * heads * (kept_dim or vdim)), dtype=torch.float32, device="cuda")
         if mfma:
-            kernels.paged_attention(queries, store.k, store.v, view, ctx, scale, 0, 2 * heads, kv_heads, kept_dim, planner=store.planner,
-                                    extras=kernels.AttentionExtras(), out=maps)
+            combined = kernels.HeadDifference(vdim, factor, eps, 1.0 - diff)
+            found = kernels.paged_attention(queries, store.k, store.v, view, ctx, scale, 0, 2 * heads, kv_heads, kept_dim, planner=store.planner,
+                                            extras=kernels.AttentionExtras(difference=combined))
         else:
+            maps = torch.empty((portion, 2 * heads * vdim), dtype=torch.float32, device="cuda")
             kernels.bias_attention(queries, store.k, store.v, view.block_table, ctx.seq_of_token, ctx.positions, None, None, scale, 1.0,
                                    2 * heads, kv_heads, 2 * dim, vdim, out=maps)
-        found = kernels.attention_difference(maps, heads, vdim, factor, eps, 1.0 - diff, dtype)
+            found = kernels.attention_difference(maps, heads, vdim, factor, eps, 1.0 - diff, dtype)
         out.append(found.float().cpu().numpy().reshape(portion, heads, vdim))
     if kept is not None:
         assert float(kept[0].min()) == 1e4 and float(kept[2].max()) == 1e4
@@ -276,6 +277,26 @@ def test_differential_attention(heads, kv_heads, dim, vdim, n_taps, n, mfma):
         assert np.abs(again - want).max() < bound, portions_of
         if not mfma:
             assert np.array_equal(again, got), portions_of      # a row does not depend on how the request was cut
+
+
+@pytest.mark.parametrize("heads,kv_heads,dim,vdim,n", [(2, 1, 16, 32, 1100), (3, 1, 24, 20, 5200)])
+def test_difference_where_the_splits_meet(heads, kv_heads, dim, vdim, n):
+    """Decoding over so many keys that they go to several workgroups, whose results meet in the kernel that combines the maps
+    (two splits, and more than eight of them)."""
+    from microllm_rocm_amd.ops import kernels
+    assert kernels.decode_splits(1, kv_heads, n) == (2 if n == 1100 else 10)
+    rng = np.random.default_rng(n)
+    q, k, v = (as_bf16(rng.normal(size=shape)) for shape in ((n, heads, 2, dim), (n, kv_heads, 2, dim), (n, kv_heads, vdim)))
+    q[n - 3:] *= 4.0        # the last queries single out a few keys
+    taps = np.ones((2 * (heads + kv_heads) * dim + kv_heads * vdim, 1))
+    got = differenced(q, k, v, taps, dim ** -0.5, 0.4, 0.6, [n - 3, 1, 1, 1], True)[n - 3:]
+    for back, query in enumerate(range(n - 3, n)):
+        maps = []
+        for m in (0, 1):
+            s = torch.einsum("hd,jhd->hj", t64(q[query, :, m]), t64(k[:query + 1, :, m]).repeat_interleave(heads // kv_heads, 1)) * dim ** -0.5
+            maps.append(torch.einsum("hj,jhd->hd", torch.softmax(s, -1), t64(v[:query + 1]).repeat_interleave(heads // kv_heads, 1)))
+        want = (plain.rms(maps[0] - 0.4 * maps[1], 1e-5) * 0.4).numpy()
+        assert np.abs(got[back] - want).max() < 0.03 * np.abs(want).max(), query
 
 
 def test_differential_attention_on_plain_pages_in_bfloat16():
@@ -539,6 +560,90 @@ def test_clamped_experts_and_places_that_return_their_input(dtype, grouped, widt
                 inner = t64(as_bf16(inner.numpy()))
             want[choice, token] = weights[token, choice] * (t64(down[e]) @ inner).numpy()
     assert np.abs(got - want).max() < (3e-5 if dtype == torch.float32 else 4e-3) * max(1.0, np.abs(want).max())
+
+
+@pytest.mark.parametrize("keep_plain", [True, False])
+@pytest.mark.parametrize("width,ff", [(64, 40), (96, 64), (256, 24)])
+def test_clamped_gate_after_a_product_of_any_number_of_rows(width, ff, keep_plain):
+    """In the product's epilogue, or after products whose columns come in the weight's order or by turns."""
+    from microllm_rocm_amd.parts.linear import Weight, linear_clamped_glu
+    rng = np.random.default_rng(ff)
+    weight = as_bf16(rng.normal(size=(2 * ff, width)) * (2.0 / math.sqrt(width)))
+    held = Weight(device(weight, torch.bfloat16), gated=True, keep_plain=keep_plain)
+    for rows in (1, 3, 16, 17, 40, 64, 65, 300):
+        x = as_bf16(rng.normal(size=(rows, width)))
+        inner = t64(x) @ t64(weight).T
+        g, u = torch.clamp(inner[:, :ff], max=1.1), torch.clamp(inner[:, ff:], min=-1.1, max=1.1)
+        want = (g * torch.sigmoid(1.702 * g) * (u + 1.0)).numpy()
+        got = linear_clamped_glu(device(x, torch.bfloat16), held, 1.1, 1.702).float().cpu().numpy()
+        assert np.abs(got - want).max() < 0.006 * np.abs(want).max(), rows
+    exact = Weight(device(weight), gated=True)
+    got = linear_clamped_glu(device(x), exact, 1.1, 1.702).cpu().numpy()
+    assert np.abs(got - want).max() < 2e-5
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("experts,top,groups,keep,shared", [(8, 3, 4, 2, False), (20, 6, 5, 3, True), (64, 8, 0, 0, True), (64, 5, 8, 2, False),
+                                                            (3, 3, 0, 0, True), (70, 4, 7, 3, True)])
+def test_router_and_choice_in_one_kernel(dtype, experts, top, groups, keep, shared):
+    """The same places and weights as the two kernels give one after the other, with and without a correction."""
+    from microllm_rocm_amd.ops import kernels
+    rng = np.random.default_rng(experts)
+    x = device(rng.normal(size=(77, 144)), dtype)
+    weight = device(rng.normal(size=(experts + int(shared), 144)) * 0.2)
+    for softmax_scores in (True, False):
+        for correction in (None, device(rng.normal(size=experts) * 0.05)):
+            options = dict(softmax_scores=softmax_scores, renormalize=True, shared_at=experts if shared else -1, groups=groups, keep=keep,
+                           correction=correction, weight_eps=1e-20, weight_scale=1.5)
+            ids, weights, gate = kernels.moe_choose(x, weight, experts, top, **options)
+            z = kernels.router_logits(x, weight)
+            want_ids, want_weights, want_gate = kernels.moe_route(z, experts, top, **options)
+            assert torch.equal(ids, want_ids) and torch.equal(weights, want_weights)
+            assert (gate is None) == (not shared) and (not shared or torch.equal(gate, want_gate))
+            scores = torch.softmax(z[:, :experts].double(), -1) if softmax_scores else torch.sigmoid(z[:, :experts].double())
+            decides = scores if correction is None else scores + correction.double()
+            if not groups:
+                best = torch.topk(decides, top, dim=-1).indices
+                assert (ids.long().sort(-1).values == best.sort(-1).values).all()
+            chosen = torch.gather(scores, 1, ids.long())
+            assert torch.allclose(weights.double(), chosen / chosen.sum(-1, keepdim=True) * 1.5, atol=1e-6)
+
+
+@pytest.mark.parametrize("width,ff,experts,identity,top,n", [(256, 288, 4, 1, 3, 9), (512, 256, 9, 3, 5, 21), (1024, 320, 3, 0, 2, 20), (4096, 1280, 5, 2, 4, 8),
+                                                             (320, 256, 2, 2, 2, 31), (256, 64, 6, 0, 2, 40)])
+@pytest.mark.parametrize("form", ["clamped_glu", "silu", "plain"])
+@pytest.mark.parametrize("on_input", [False, True])
+def test_few_pairs_on_the_matrix_units(width, ff, experts, identity, top, n, form, on_input):
+    """Reductions of a multiple of 32 from 256 on: an expert with no pair, with one, with more than the 16 columns of a product;
+    the last wave's steps overlap another's where the reduction is no multiple of 256."""
+    from microllm_rocm_amd.ops import kernels
+    rng = np.random.default_rng(width + n)
+    gated = form != "plain"
+    x, down = as_bf16(rng.normal(size=(n, width))), as_bf16(rng.normal(size=(experts, width, ff)) / math.sqrt(ff))
+    inner_weight = as_bf16(rng.normal(size=(experts, (2 if gated else 1) * ff, width)) * (2.0 / math.sqrt(width)))
+    places = rng.permutation(experts + identity)[:max(top, experts + identity - 1)]        # one place no token takes
+    ids = np.stack([rng.permutation(places)[:top] for _ in range(n)])
+    weights = rng.uniform(0.2, 1.6, size=(n, top))
+    options = dict(gated=gated, activation={"clamped_glu": "clamped_glu", "silu": "silu", "plain": "gelu_erf"}[form], identity=identity,
+                   **(dict(limit=1.25, slope=1.702) if form == "clamped_glu" else {}))
+    got = kernels.moe_experts(device(x, torch.bfloat16), device(ids, torch.int32), device(weights), device(inner_weight, torch.bfloat16),
+                              device(down, torch.bfloat16), on_input, grouped=False, **options).cpu().numpy()
+    for token in range(n):
+        for choice in range(top):
+            e, w = ids[token, choice], float(np.float32(weights[token, choice]))
+            if e >= experts:
+                assert np.abs(got[choice, token] - w * x[token]).max() < 1e-5
+                continue
+            inner = t64(inner_weight[e]) @ t64(as_bf16(x[token] * w) if on_input else x[token])
+            if form == "clamped_glu":
+                g, u = torch.clamp(inner[:ff], max=1.25), torch.clamp(inner[ff:], min=-1.25, max=1.25)
+                inner = g * torch.sigmoid(1.702 * g) * (u + 1.0)
+            elif form == "silu":
+                inner = inner[:ff] * torch.sigmoid(inner[:ff]) * inner[ff:]
+            else:
+                inner = 0.5 * inner * (1.0 + torch.erf(inner / math.sqrt(2.0)))
+            want = ((1.0 if on_input else w) * (t64(down[e]) @ inner)).numpy()
+            assert np.abs(got[choice, token] - want).max() < 0.015 * np.abs(want).max(), (token, choice)
 
 
 # ---- the engine ---------------------------------------------------------------------------------------------------
